@@ -48,6 +48,14 @@ extern "C" {
 
 #define TMX_FAMILY_LLAMA3 0
 #define TMX_FAMILY_QWEN3 1
+#define TMX_FAMILY_LATENT 2 /* dense weights, latent attention, several residual streams: tmx_latent_layer_desc */
+
+#define TMX_ACT_BF16 0 /* activations, caches and matrix products in bf16 with f32 accumulation */
+#define TMX_ACT_F32 1  /* everything in f32 (no matrix pipe) */
+
+#define TMX_MAX_STREAMS 8      /* residual streams of a model */
+#define TMX_MAX_LATENT_RANK 512 /* padded latent width of latent attention: 64, 128, 256 or 512 */
+#define TMX_MAX_LATENT_ROT 128  /* padded width of its shared rotated key part: 64 or 128 */
 
 #define TMX_MAX_RPAD 128   /* widest padded LoRA projection (sum of fused ranks, rounded up to 32) */
 #define TMX_MAX_SPLITS 16  /* most K-slices a projection is split into */
@@ -64,9 +72,9 @@ extern "C" {
                               :207-226 selective_log_softmax) */
 
 const char* tmx_status_string(int status);
-/* Bumped whenever a struct of this header grows or an entry point changes: 7 = tmx_model_desc.head_tiles and the
- * tmx_decode_state.share_* fields are present.  A caller that fills the structs checks it once after loading. */
-#define TMX_ABI_VERSION 7
+/* Bumped whenever a struct of this header grows or an entry point changes: 8 = TMX_FAMILY_LATENT and the fields of
+ * tmx_model_desc behind head_tiles are present.  A caller that fills the structs checks it once after loading. */
+#define TMX_ABI_VERSION 8
 int tmx_abi_version(void);
 
 /* w_out[K, N] bf16 = bf16(q) * scale evaluated in bf16, bit-exact.
@@ -314,8 +322,92 @@ int tmx_moe_experts(void* stream, const void* x, int ldx, const void* qweight, c
                     const int32_t* expert_of, int P, int top_k, int E, int K, int N, int G, int down,
                     void* out, int ldo);
 
+/* ---- dense projections, residual streams, latent attention ------------------------
+ * No counterpart in the reference: the mechanisms of TMX_FAMILY_LATENT models, each usable alone.  `act` is
+ * TMX_ACT_*; an "act tensor" holds bf16 or f32 accordingly.  Every width below is padded: columns past the real
+ * width hold zeros in the weights and come out as zeros. */
+
+/* y[m, h, n] = epilogue(sum_k x[m, h, k] W[h, n, k] + bias[n]) for `heads` matrices W (1: a plain projection).
+ * x row m of matrix h starts at x + m ldx + h x_head, y row m at y + m ldy + h y_head (elements).
+ *   w     : TMX_ACT_BF16: every matrix in the tile layout of tmx_head_tiles_pack (V = N, D = K), one after another;
+ *           TMX_ACT_F32: f32 row-major [heads][N][K].  K % 64 == 0, N % 32 == 0
+ *   bias  : f32 [N] or NULL (heads == 1)
+ *   epilogue TMX_DENSE_PLAIN; TMX_DENSE_SWIGLU: W holds N / 2 gate rows, then N / 2 up rows ((N / 2) % 32 == 0),
+ *           y[m, n] = silu(gate) * up, N / 2 columns; TMX_DENSE_GATED: y = product * sigmoid(gate[m ldg + h y_head + n])
+ * Up to 128 rows stream the weights once; more rows run in 256-row blocks. */
+#define TMX_DENSE_PLAIN 0
+#define TMX_DENSE_SWIGLU 1
+#define TMX_DENSE_GATED 2
+int tmx_dense_linear(void* stream, int act, const void* x, int ldx, int x_head, const void* w, const float* bias,
+                     const void* gate, int ldg, void* y, int ldy, int y_head, int M, int K, int N, int heads,
+                     int epilogue);
+
+/* Residual streams x_1 .. x_S (f32 [M][S][Dp]): x_t <- sum_s mix[s, t] x_s + out[t] y, then u = sum_s in[s] x_s and
+ * xn = u / sqrt(mean(u^2) + eps) * norm_w (mean over the real width D).  One launch per sublayer boundary.
+ *   y    : act tensor [M][Dp], the sublayer's result; NULL: the streams stay as they are
+ *   mix  : f32 [S][S] ([from, to]), out / in: f32 [S]; norm_w: f32 [Dp]; xn: act tensor [M][Dp]
+ *   store: 0 leaves the streams in memory untouched (the last boundary of a model needs only xn) */
+int tmx_stream_rows(void* stream, int act, float* streams, const void* y, const float* mix, const float* out,
+                    const float* in, const float* norm_w, void* xn, int M, int S, int D, int Dp, float eps, int store);
+
+/* Row kernel of latent attention: takes the fused projection row z[m] = [query, unrotated: H dim_p | query,
+ * rotated: H rot | latent: rank | shared key part: rot | ...] and writes
+ *   q[m][H][ld], columns rank_p .. rank_p + rot - 1 = the rotated query part (columns below rank_p are not touched,
+ *                the rest is zero),  ld = rank_p + rot_p
+ *   cache row [sequence m / T][slot *step + m % T][ld] = [RMSNorm(latent) * norm_w | 0 | rotated key part | 0]
+ *   (off_kv < 0: no latent in z, the cache is another layer's and only q is written)
+ * table: f32 [positions_max][rot / 2][2] cos, sin of every position (scaled as the rotation wants them);
+ * the pair of dimension i is i + rot / 2. */
+int tmx_latent_rows(void* stream, int act, const void* z, int ldz, int off_qr, int off_kv, const float* norm_w,
+                    float eps, const float* table, int positions_max, const int32_t* positions, const int32_t* step,
+                    int buf_len, void* q, void* cache, int M, int T, int H, int rot, int rank, int rank_p, int rot_p,
+                    int C);
+
+/* out[m][H][rank_p] = sum_j softmax_j(q[m, h] . cache[j] * scale) cache[j][0 .. rank_p) over the slots
+ * j <= *step + m % T with input_mask[m / T, j]; with sink (f32 [H]) the denominator also holds exp(sink[h]).
+ * Every head reads the same cache row: keys of width rank_p + rot_p, values its first rank_p columns.
+ * rank_p in {64, 128, 256, 512}, rot_p in {64, 128}.
+ * workspace: tmx_latent_attention_workspace_bytes(M / T, T, H, rank_p, C) bytes (may be 0 -> NULL allowed). */
+size_t tmx_latent_attention_workspace_bytes(int n_seq, int T, int H, int rank_p, int C);
+int tmx_latent_attention(void* stream, int act, const void* q, const void* cache, const float* sink,
+                         const uint8_t* input_mask, const int32_t* step, int buf_len, void* out, void* workspace,
+                         int n_seq, int T, int H, int rank_p, int rot_p, int C, float scale);
+
 /* ---- whole decode steps ------------------------------------------------------ */
 
+typedef struct {
+  const void* w;     /* see tmx_dense_linear; NULL: the layer has no such matrix */
+  const float* bias; /* f32 [N] or NULL */
+  int K, N, heads;
+} tmx_dense_desc;
+
+typedef struct { /* coefficients of a sublayer's stream mixing, f32 on the device */
+  const float* in;  /* [S] */
+  const float* out; /* [S] */
+  const float* mix; /* [S][S], [from, to] */
+} tmx_streams_desc;
+
+typedef struct {
+  const float *norm1_w, *norm2_w; /* f32 [Dp] */
+  tmx_streams_desc hc1, hc2;      /* mixer, feed-forward */
+  /* latent attention */
+  int heads, rot_dim, kv_rank;    /* real sizes */
+  int dim_p, rot_p, rank_p, vdim_p; /* padded: dim_p, vdim_p % 64 == 0; rank_p, rot_p as tmx_latent_attention */
+  int off_qr, off_kv, off_gate;   /* columns of the fused projection (tmx_latent_rows); off_kv < 0: the cache of layer
+                                     kv_layer is used; off_gate < 0: no output gate */
+  int kv_layer;                   /* layer whose cache this layer reads (itself unless off_kv < 0) */
+  float scale;
+  tmx_dense_desc in;              /* fused projection of the normed input */
+  tmx_dense_desc uk;              /* heads x [rank_p, dim_p]: the query moved into the latent space */
+  tmx_dense_desc uv;              /* heads x [vdim_p, rank_p]: the latent result to values */
+  tmx_dense_desc o;               /* [Dp, heads vdim_p] */
+  const float* kv_norm_w;         /* f32 [kv_rank] */
+  const float* table;             /* rotation table, see tmx_latent_rows */
+  const float* sink;              /* f32 [heads] or NULL */
+  /* feed-forward (gate_up.w == NULL: none) */
+  tmx_dense_desc gate_up;         /* gate rows, then up rows: [2 Fp, Dp] */
+  tmx_dense_desc down;            /* [Dp, Fp] */
+} tmx_latent_layer_desc;
 
 typedef struct {
   const void* qweight;  /* q4t tiles of the (column-fused) weight [K, N] */
@@ -352,6 +444,16 @@ typedef struct {
   const void* head_tiles;   /* NULL, or the head matrix once more in the layout tmx_head_tiles_pack writes (V % 32
                                == 0, D % 64 == 0): steps of up to 64 sequences then stream that copy, every byte
                                in whole cache lines (the 1.05 GB head of the 8B shape: 190 us against 252 us) */
+  /* TMX_FAMILY_LATENT: num_layers, vocab_size, embed_dim and norm_eps hold the real sizes; embed [V, Dp] and
+   * pos_embed are bf16; head is [Vp, Dp] bf16 (+ head_tiles) or f32; final_norm_w is f32 [Dp], with Dp = embed_dim
+   * rounded up to 64 and Vp = vocab_size rounded up to 32; layers is NULL */
+  const tmx_latent_layer_desc* latent_layers; /* HOST array of num_layers entries */
+  int act;                  /* TMX_ACT_* */
+  int streams;              /* 1 .. TMX_MAX_STREAMS */
+  int max_positions;        /* rows of pos_embed and of every rotation table (positions are clamped to it) */
+  const void* pos_embed;    /* bf16 [max_positions, Dp], added to the embedding; NULL: none */
+  const float* final_in;    /* f32 [streams]: weights of the streams in the final sum */
+  float logit_scale;
 } tmx_model_desc;
 
 /* Mirrors _SamplingState (tunix/generate/sampler.py:53-109); all arrays on the device. */
@@ -363,7 +465,8 @@ typedef struct {
   float* logprobs;       /* [B, buf_len] or NULL */
   uint8_t* done;         /* [B] */
   int32_t* step;         /* device scalar: decoding_step */
-  void* kv_cache;        /* bf16 [layers][2 (k, v)][B][C][Kh][H] */
+  void* kv_cache;        /* bf16 [layers][2 (k, v)][B][C][Kh][H]; TMX_FAMILY_LATENT: for every layer with a latent of
+                            its own, in layer order, an act tensor [B][C][rank_p + rot_p] (zero-filled before use) */
   int sampling_mode;     /* TMX_SAMPLE_* */
   float temperature, top_p;
   int top_k;
@@ -372,7 +475,8 @@ typedef struct {
   int n_eos;
   const int32_t* forbidden;
   int n_forbidden;
-  float* logits_out;     /* optional f32 [B, V]: logits of the last executed step */
+  float* logits_out;     /* optional f32 [B * tokens_per_pass, V] (TMX_FAMILY_LATENT: V rounded up to 32): logits of
+                            the last executed pass */
   void* workspace;
   size_t workspace_bytes;
   void* nucleus_workspace; /* tmx_nucleus_workspace_bytes(B, V); needed when top_p < 1 or top_k > 0 */
@@ -383,7 +487,7 @@ typedef struct {
                               attending to the slots up to its own column; *step advances by T.
                               Rows of a pass (batch * T, also for T <= 1): up to TMX_MAX_FILL_ROWS when
                               every projection has K % 128 == 0 (MoE models: rows * experts_per_tok <=
-                              TMX_MAX_MOE_PAIRS), else 128.
+                              TMX_MAX_MOE_PAIRS; TMX_FAMILY_LATENT: always), else 128.
                               The workspace must be sized for batch * T rows. */
   int share_group;         /* 0 or 1: nothing is shared.  g > 1: the batch is made of consecutive groups of g
                               sequences whose cache slots [0, share_len) and input_mask entries are identical
@@ -394,6 +498,7 @@ typedef struct {
   int share_len;
 } tmx_decode_state;
 
+/* batch: rows of a pass (sequences x tokens_per_pass). */
 size_t tmx_decode_workspace_bytes(const tmx_model_desc* model, int batch, int cache_size);
 
 /* Contract on the step counter: the caller keeps *step + n_steps * max(tokens_per_pass, 1) < buf_len
@@ -447,7 +552,9 @@ int tmx_decode_steps_graph(const tmx_model_desc* model, const tmx_decode_state* 
 #define TMX_K_ADVANCE 9
 #define TMX_K_EMPTY 10   /* one empty launch per layer: what an event pair costs by itself */
 #define TMX_K_ROUTER 11  /* MoE router: scores, softmax, top-k */
-#define TMX_NUM_KERNEL_CLASSES 12
+#define TMX_K_LATENT_Q 12 /* latent attention: queries into the latent space */
+#define TMX_K_LATENT_V 13 /* latent attention: latent results to values (+ output gate) */
+#define TMX_NUM_KERNEL_CLASSES 14
 int tmx_decode_steps_profiled(const tmx_model_desc* model, const tmx_decode_state* state, void* stream,
                               int n_steps, int sample, float* class_ms_host, int* class_launches_host);
 

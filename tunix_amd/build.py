@@ -1,5 +1,6 @@
 """Builds the HIP library (libtmx.so) in-tree for gfx950 with hipcc."""
 import concurrent.futures
+import fcntl
 import os
 import subprocess
 
@@ -49,13 +50,25 @@ def build(verbose=False, jobs=6, host_sanitizers=False):
   with concurrent.futures.ThreadPoolExecutor(max_workers=jobs) as ex:
     outs = list(ex.map(lambda so: _run([hipcc] + HIPCC_FLAGS + extra + inc + ['-c', so[0], '-o', so[1]]),
                        zip(srcs, objs)))
-  link = [hipcc, '--offload-arch=gfx950', '-shared', '-fPIC', '-o', lib_path]
+  part = lib_path + '.part'
+  link = [hipcc, '--offload-arch=gfx950', '-shared', '-fPIC', '-o', part]
   # the sanitizer runtime is supplied by the loading process (preloaded), so its symbols stay undefined here
   link += ['-shared-libsan', '-fsanitize=address', '-fsanitize=undefined'] if host_sanitizers else ['-Wl,--no-undefined']
   outs.append(_run(link + objs))
+  os.replace(part, lib_path)  # the library appears complete or not at all
   if verbose:
     print('\n'.join(o for o in outs if o.strip()))
   return lib_path
+
+
+def ensure():
+  """Builds the library if there is none; callers that start at the same time wait for one build."""
+  if os.path.exists(LIB_PATH):
+    return LIB_PATH
+  os.makedirs(OBJ, exist_ok=True)
+  with open(os.path.join(OBJ, '.lock'), 'w') as lock:
+    fcntl.flock(lock, fcntl.LOCK_EX)
+    return LIB_PATH if os.path.exists(LIB_PATH) else build(jobs=min(16, os.cpu_count() or 1))
 
 
 def sanitizer_runtime():

@@ -8,13 +8,9 @@
 // live in device memory exactly like _SamplingState (sampler.py:53-109), and the
 // counter is advanced on the device, so the host never reads anything back
 // between steps.
-#include <vector>
-
-#include "tmx_kernels.h"
+#include "tmx_decoder.h"
 
 namespace tmx {
-
-static size_t align256(size_t v) { return (v + 255) & ~(size_t)255; }
 
 struct Workspace {
   uint16_t* delta;   // LoRA delta of a split projection, made by its LoRA blocks (up to 128 rows)
@@ -133,19 +129,6 @@ static Workspace carve(const tmx_model_desc* m, int B, int C, char* base) {
   return w;
 }
 
-// Optional per-kernel-class timing with HIP events (used by the benchmark only).
-struct Prof {
-  std::vector<hipEvent_t> ev[TMX_NUM_KERNEL_CLASSES];
-  void before(int k, hipStream_t st) { push(k, st); }
-  void after(int k, hipStream_t st) { push(k, st); }
-  void push(int k, hipStream_t st) {
-    hipEvent_t e;
-    if (hipEventCreate(&e) != hipSuccess) return;
-    (void)hipEventRecord(e, st);
-    ev[k].push_back(e);
-  }
-};
-
 static int check_linear(const tmx_qlinear_desc& l, int K, int N) {
   if (!l.qweight || !l.scales) return TMX_ERR_ARG;
   if (l.K != K || l.N != N) return TMX_ERR_SHAPE;
@@ -159,15 +142,20 @@ using namespace tmx;
 
 extern "C" size_t tmx_decode_workspace_bytes(const tmx_model_desc* m, int batch, int cache_size) {
   if (!m || batch <= 0) return 0;
+  if (m->family == TMX_FAMILY_LATENT) return latent_check(m) == TMX_OK ? latent_carve(m, batch, nullptr).total : 0;
   return carve(m, batch, cache_size, nullptr).total;
 }
 
 static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s, void* stream,
                              int n_steps, int sample, Prof* prof) {
-  if (!m || !s || !m->layers || !m->embed || !m->final_norm_w || !m->head) return TMX_ERR_ARG;
+  if (!m || !s || !m->embed || !m->final_norm_w || !m->head) return TMX_ERR_ARG;
   if (!s->token_buffer || !s->positions || !s->input_mask || !s->done || !s->step || !s->kv_cache ||
       !s->workspace)
     return TMX_ERR_ARG;
+  const bool latent = m->family == TMX_FAMILY_LATENT;
+  if (!latent && !m->layers) return TMX_ERR_ARG;
+  int rc = latent ? latent_check(m) : TMX_OK;
+  if (rc != TMX_OK) return rc;
   const bool moe = m->num_experts > 0;
   // rows of a pass: one per sequence, or tokens_per_pass consecutive tokens of every sequence
   // (cache fill and scoring only: sampling needs the previous token)
@@ -186,11 +174,10 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
   if (nucleus && !s->nucleus_workspace) return TMX_ERR_ARG;
   const int D = m->embed_dim, N = m->num_heads, Kh = m->num_kv_heads, H = m->head_dim;
   const int F = m->hidden_dim, NH = N * H, QKV = (N + 2 * Kh) * H;
-  if (carve(m, B, C, nullptr).total > s->workspace_bytes) return TMX_ERR_SHAPE;
-  for (int i = 0; i < m->num_layers; ++i) {
+  if ((latent ? latent_carve(m, B, nullptr).total : carve(m, B, C, nullptr).total) > s->workspace_bytes) return TMX_ERR_SHAPE;
+  for (int i = 0; !latent && i < m->num_layers; ++i) {
     const tmx_layer_desc& l = m->layers[i];
     if (!l.norm1_w || !l.norm2_w) return TMX_ERR_ARG;
-    int rc;
     if ((rc = check_linear(l.qkv, D, QKV)) || (rc = check_linear(l.o, NH, D))) return rc;
     if (moe) {
       if (!l.router_w || l.gate_up.lora_a_t || l.down.lora_a_t) return TMX_ERR_ARG;
@@ -199,20 +186,13 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
     if ((rc = check_linear(l.gate_up, D, 2 * F)) || (rc = check_linear(l.down, F, D))) return rc;
   }
   hipStream_t st = (hipStream_t)stream;
-  const Workspace w = carve(m, B, C, (char*)s->workspace);
+  const LatentWorkspace lw = latent ? latent_carve(m, B, (char*)s->workspace) : LatentWorkspace();
+  const Workspace w = latent ? Workspace() : carve(m, B, C, (char*)s->workspace);
   const size_t kv_elems = (size_t)NSEQ * C * Kh * H;
   const float theta = m->family == TMX_FAMILY_LLAMA3 ? 1000000.0f : m->rope_theta;
-  int rc;
-#define TMX_TRY(kind, expr)            \
-  {                                    \
-    if (prof) prof->before(kind, st);  \
-    rc = (expr);                       \
-    if (prof) prof->after(kind, st);   \
-    if (rc != TMX_OK) return rc;       \
-  }
 
-  const Splits sp = plan_splits(m, B);
-  const bool small = small_batch_ok(m, B, T);
+  const Splits sp = latent ? Splits() : plan_splits(m, B);
+  const bool small = !latent && small_batch_ok(m, B, T);
   auto lora_of = [&](const tmx_qlinear_desc& l, int) {
     LoraIn li = {};
     if (l.lora_a_t) {
@@ -251,14 +231,17 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
                              w.y16, w.t_part, w.t16, B, l.K, l.N, l.G, l.r_pad);
   };
   // the hand-over words of the fused gate | up launch start at zero (the kernel leaves them so)
-  if (!moe && B <= kFusedGateUpMaxRows && w.gu_sync && n_steps > 0) {
+  if (!latent && !moe && B <= kFusedGateUpMaxRows && w.gu_sync && n_steps > 0) {
     rc = zero_words(st, (uint32_t*)w.gu_sync, 64);
     if (rc != TMX_OK) return rc;
   }
   // samples of one prompt in consecutive rows: decode attention reads the prompt slots once per group
   const bool share_walk = T == 1 && !small && w.attn_partial && attn_share_ok(B, N, Kh, H, C, s->share_group, s->share_len);
   for (int it = 0; it < n_steps; ++it) {
-    {  // embedding gather + first input norm + this step's RoPE table
+    if (latent) {
+      rc = latent_layers(st, m, s, lw, NSEQ, T, sample != 0, prof);
+      if (rc != TMX_OK) return rc;
+    } else {  // embedding gather + first input norm + this step's RoPE table
       RowNormArgs a = {};
       a.embed = (const uint16_t*)m->embed;
       a.vocab = m->vocab_size;
@@ -346,7 +329,7 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
         if (sample) TMX_TRY(TMX_K_ROWNORM, row_norm(st, a, B));
       }
     }
-    for (int i = 0; !small && i < m->num_layers; ++i) {
+    for (int i = 0; !small && !latent && i < m->num_layers; ++i) {
       const tmx_layer_desc& l = m->layers[i];
       // gate | up with LoRA + SwiGLU in its epilogue: K % 256 == 0 below 8192, unsplit, 2 r <= 32
       const bool fused_gu = !moe && B <= kFusedGateUpMaxRows && sp.gate_up == 1 && D % 256 == 0 && D < 8192 && F % 64 == 0 &&
@@ -510,57 +493,59 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
       }
       if (prof) TMX_TRY(TMX_K_EMPTY, empty_launch(st));
     }
-    if (sample && !nucleus && B > 64 && !s->logits_out && s->n_forbidden == 0 && D % 128 == 0) {
-      // more than 64 rows: the head in 256 x 256 blocks, one pass over the head matrix (the 64-row kernel
-      // would take one pass per 64 rows)
+    if (sample) {
       HeadArgs a = {};
-      a.x = w.xn;
+      a.x = (const uint16_t*)(latent ? lw.xn : w.xn);
       a.w = (const uint16_t*)m->head;
-      a.M = B; a.D = D; a.V = m->vocab_size;
+      a.M = B;
+      a.D = latent ? pad_to(D, 64) : D;
+      a.V = latent ? pad_to(m->vocab_size, 32) : m->vocab_size;
       a.mode = s->sampling_mode;
       a.temperature = s->temperature;
       a.k0 = s->seed_hi; a.k1 = s->seed_lo;
       a.step = s->step;
-      a.part_f = (float*)w.head_partial;
-      a.part_i = (int32_t*)((float*)w.head_partial + (size_t)B * ((m->vocab_size + 255) / 256) * 4);
+      void* partial = latent ? lw.head_partial : w.head_partial;
+      a.part_f = (float*)partial;
       a.token_buffer = s->token_buffer;
       a.logprobs = s->logprobs;
       a.done = s->done;
       a.eos = s->eos_ids; a.n_eos = s->n_eos;
       a.buf_len = L;
       a.tpp = T;
-      TMX_TRY(TMX_K_HEAD, head_wide(st, a));
-    } else if (sample) {
-      HeadArgs a = {};
-      a.x = w.xn;
-      a.w = (const uint16_t*)m->head;
-      a.w_tiles = (const uint16_t*)m->head_tiles;
-      a.M = B; a.D = D; a.V = m->vocab_size;
-      a.mode = s->sampling_mode;
-      a.temperature = s->temperature;
-      a.k0 = s->seed_hi; a.k1 = s->seed_lo;
-      a.step = s->step;
-      a.forbidden = s->forbidden; a.n_forbidden = s->n_forbidden;
-      a.logits_out = s->logits_out;
-      const size_t nwg = (m->vocab_size + 127) / 128;
-      a.part_f = (float*)w.head_partial;
-      a.part_i = (int32_t*)((float*)w.head_partial + (size_t)B * nwg * 4);
-      a.token_buffer = s->token_buffer;
-      a.logprobs = s->logprobs;
-      a.done = s->done;
-      a.eos = s->eos_ids; a.n_eos = s->n_eos;
-      a.buf_len = L;
-      a.tpp = T;
-      if (nucleus) {
-        TMX_TRY(TMX_K_HEAD, head_sample_nucleus(st, a, s->top_p, s->top_k, s->nucleus_workspace,
-                                                s->nucleus_workspace_bytes));
+      if (latent) {
+        a.v_live = m->vocab_size;
+        a.logit_scale = m->logit_scale;
+      }
+      if (latent && m->act == TMX_ACT_F32) {
+        // the products in f32 first; selection then reads them from memory
+        DenseArgs d = {};
+        d.x = lw.xn; d.ldx = a.D; d.w = m->head;
+        d.y = s->logits_out ? s->logits_out : lw.logits; d.ldy = a.V;
+        d.M = B; d.K = a.D; d.N = a.V; d.heads = 1; d.epi = TMX_DENSE_PLAIN;
+        TMX_TRY(TMX_K_HEAD, dense_linear(st, m->act, d));
+        a.logits_out = (float*)d.y;
+        a.logits_ready = true;
+      }
+      if (!a.logits_ready && !nucleus && B > 64 && !s->logits_out && s->n_forbidden == 0 && a.D % 128 == 0) {
+        // more than 64 rows: the head in 256 x 256 blocks, one pass over the head matrix (the 64-row kernel
+        // would take one pass per 64 rows)
+        a.part_i = (int32_t*)((float*)partial + (size_t)B * ((a.V + 255) / 256) * 4);
+        TMX_TRY(TMX_K_HEAD, head_wide(st, a));
       } else {
-        TMX_TRY(TMX_K_HEAD, head_sample(st, a));
+        a.w_tiles = (const uint16_t*)m->head_tiles;
+        a.forbidden = s->forbidden; a.n_forbidden = s->n_forbidden;
+        if (!a.logits_ready) a.logits_out = s->logits_out;
+        a.part_i = (int32_t*)((float*)partial + (size_t)B * ((a.V + 127) / 128) * 4);
+        if (nucleus) {
+          TMX_TRY(TMX_K_HEAD, head_sample_nucleus(st, a, s->top_p, s->top_k, s->nucleus_workspace,
+                                                  s->nucleus_workspace_bytes));
+        } else {
+          TMX_TRY(TMX_K_HEAD, head_sample(st, a));
+        }
       }
     }
     TMX_TRY(TMX_K_ADVANCE, advance_step(st, s->step, T));
   }
-#undef TMX_TRY
   return TMX_OK;
 }
 
@@ -570,7 +555,7 @@ extern "C" int tmx_decode_steps(const tmx_model_desc* m, const tmx_decode_state*
 }
 
 extern "C" int tmx_decode_status(const tmx_model_desc* m, const tmx_decode_state* s, void* stream) {
-  if (!m || !s || !s->workspace || !m->layers) return TMX_ERR_ARG;
+  if (!m || !s || !s->workspace) return TMX_ERR_ARG;
   hipStream_t st = (hipStream_t)stream;
   if (s->workspace_bytes < 256) return TMX_ERR_ARG;
   uint32_t flag = 0;

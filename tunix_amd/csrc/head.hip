@@ -162,8 +162,9 @@ __global__ __launch_bounds__(256, MT == 4 ? 1 : 2) void head_kernel(HeadArgs a) 
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int v = v0 + acc_row(r, lane);
-        float logit = rbf(acc[m][r]);
+        float logit = rbf(acc[m][r] * a.logit_scale);
         if (a.logits_out) a.logits_out[(size_t)row * a.V + v] = logit;
+        if (v >= a.v_live) logit = -INFINITY;
         for (int f = 0; f < a.n_forbidden; ++f)
           if (a.forbidden[f] == v) logit = -INFINITY;
         float z = logit, key = logit;
@@ -429,7 +430,7 @@ __global__ __launch_bounds__(512, 1) void head_wide_kernel(HeadArgs a, int tok_b
       constexpr int m = decltype(ic)::value / 16, r = decltype(ic)::value % 16;
       const int v = v0 + m * 32 + acc_row(r, lane);
       if (v >= a.V) return;  // (V % 32 == 0 where keys are written: a group of four rows is in or out as one)
-      const float logit = rbf(acc[m][r]);
+      const float logit = v < a.v_live ? rbf(acc[m][r] * a.logit_scale) : -INFINITY;
       float z = logit, key = logit;
       if (score) {
         z = score_clip(rbf(logit / a.temperature));  // bf16 logits divided in place stay bf16 (rl/common.py:591-592)
@@ -517,7 +518,78 @@ int head_wide(hipStream_t st, HeadArgs a) {
   return check_launch();
 }
 
+// One workgroup per row of f32 logits: scale, then the statistics and the best candidate of the whole row (the
+// epilogue of head_kernel over a row in memory).  Keys of the sorting branch are made from the bf16 value of the
+// logit, and that branch then works with those values.
+__global__ __launch_bounds__(256) void head_select_f32_kernel(HeadArgs a) {
+  __shared__ float s_f[4][4];
+  __shared__ int s_i[4];
+  const int row = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  float* lg = a.logits_out + (size_t)row * a.V;
+  uint32_t key0 = 0, key1 = 0;
+  if (a.mode == TMX_SAMPLE_TOP_P) threefry2x32(a.k0, a.k1, 0u, (uint32_t)*a.step, key0, key1);
+  const bool score = a.mode == TMX_SAMPLE_SCORE;
+  const int tpp = a.tpp > 0 ? a.tpp : 1;
+  const int target = score ? a.token_buffer[(size_t)(row / tpp) * a.buf_len + min(*a.step + row % tpp + 1, a.buf_len - 1)] : -1;
+  float mx = kNegBig, se = 0.f;
+  Best best = {-INFINITY, -INFINITY, 0x7FFFFFFF};
+  for (int v = threadIdx.x; v < a.V; v += 256) {
+    float logit = lg[v] * a.logit_scale;
+    lg[v] = logit;
+    if (v >= a.v_live) logit = -INFINITY;
+    for (int f = 0; f < a.n_forbidden; ++f)
+      if (a.forbidden[f] == v) logit = -INFINITY;
+    if (a.sort_keys) logit = rbf(logit);
+    float z = logit, key = logit;
+    if (score) {
+      z = score_clip(logit / a.temperature);
+      key = v == target ? 0.f : -INFINITY;
+    } else if (a.mode == TMX_SAMPLE_TOP_P) {
+      z = logit / a.temperature;
+      if (a.sort_keys) {
+        const uint32_t zb = __float_as_uint(logit + 0.0f) >> 16;
+        a.sort_keys[(size_t)row * a.V + v] = (uint16_t)((zb & 0x8000u) ? zb : (~zb & 0x7FFFu));
+        key = z;
+      } else {
+        uint32_t o0, o1;
+        threefry2x32(key0, key1, 0u, (uint32_t)row * (uint32_t)a.V + (uint32_t)v, o0, o1);
+        key = z + gumbel_from_bits(o0 ^ o1);
+      }
+    }
+    lse_merge(mx, se, z, 1.f);
+    Best c = {key, z, v};
+    best_merge(best, c);
+  }
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) {
+    const float mx2 = __shfl_xor(mx, off, 64), se2 = __shfl_xor(se, off, 64);
+    Best o = {__shfl_xor(best.key, off, 64), __shfl_xor(best.z, off, 64), __shfl_xor(best.idx, off, 64)};
+    lse_merge(mx, se, mx2, se2);
+    best_merge(best, o);
+  }
+  if (lane == 0) {
+    s_f[wave][0] = mx; s_f[wave][1] = se; s_f[wave][2] = best.key; s_f[wave][3] = best.z;
+    s_i[wave] = best.idx;
+  }
+  __syncthreads();
+  if (threadIdx.x) return;
+  for (int w = 1; w < 4; ++w) {
+    lse_merge(mx, se, s_f[w][0], s_f[w][1]);
+    Best o = {s_f[w][2], s_f[w][3], s_i[w]};
+    best_merge(best, o);
+  }
+  float* pf = a.part_f + (size_t)row * a.nwg * 4;
+  pf[0] = mx; pf[1] = se; pf[2] = best.key; pf[3] = best.z;
+  a.part_i[(size_t)row * a.nwg] = best.idx;
+}
+
 int head_logits(hipStream_t st, HeadArgs& a) {
+  if (a.logits_ready) {
+    if (!a.logits_out || a.V <= 0 || a.M <= 0) return TMX_ERR_SHAPE;
+    a.nwg = 1;
+    hipLaunchKernelGGL(head_select_f32_kernel, dim3(a.M), dim3(256), 0, st, a);
+    return check_launch();
+  }
   if (a.V % 32 || a.D % 64 || a.M <= 0 || a.M > TMX_MAX_FILL_ROWS) return TMX_ERR_SHAPE;
   a.nwg = (a.V + 127) / 128;
   // Rows go through the 32- or 64-row kernel in chunks of 64: one pass over the head matrix per chunk.

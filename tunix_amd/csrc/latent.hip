@@ -1,0 +1,523 @@
+// Latent attention: every token caches one latent vector c (normed) and one rotated key part shared by all heads;
+// a head's keys and values are linear in c, so its query is moved into the latent space (q~ = W_uk^T q, a batched
+// projection) and the attention runs on the cache rows themselves:
+//   score_j = (q~ . c_j + rot(q_r) . rot(k_r)_j) scale,   out~ = sum_j p_j c_j,   value = W_uv out~
+// All heads read the same row, once: keys are its rank_p + rot_p columns, values its first rank_p.
+//
+//   latent_rows_kernel    rotation of the queries, norm + rotation of the new cache row
+//   latent_attn_kernel    the walk over the cache on the matrix pipe (one or many tokens per sequence)
+//   latent_combine_kernel merge of the splits of a query row
+//   latent_attn_f32_kernel the same attention in f32 on the vector ALU
+#include "tmx_kernels.h"
+
+namespace tmx {
+
+__device__ __forceinline__ float act_get(const uint16_t* p) { return bf2f(*p); }
+__device__ __forceinline__ float act_get(const float* p) { return *p; }
+__device__ __forceinline__ void act_set(uint16_t* p, float v) { *p = f2bf(v); }
+__device__ __forceinline__ void act_set(float* p, float v) { *p = v; }
+
+// One workgroup per row of the fused projection.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_rows_kernel(LatentRowsArgs a) {
+  __shared__ float smem[4];
+  const int m = blockIdx.x, tid = threadIdx.x;
+  const int tpp = a.tpp > 0 ? a.tpp : 1;
+  const int seq = m / tpp, slot = min(*a.step + m % tpp, min(a.buf_len, a.C) - 1);
+  const int pos = min(max(a.positions[(size_t)seq * a.buf_len + slot], 0), a.max_positions - 1);
+  const int half = a.rot >> 1, ld = a.rank_p + a.rot_p;
+  const float2* tab = reinterpret_cast<const float2*>(a.table) + (size_t)pos * half;
+  const T* z = reinterpret_cast<const T*>(a.z) + (size_t)m * a.ldz;
+  T* q = reinterpret_cast<T*>(a.q) + (size_t)m * a.H * ld + a.rank_p;
+  float v[2] = {0.f, 0.f};  // the latent's values of this thread (rank <= 512)
+  if (a.off_kv >= 0) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      if (tid + 256 * i < a.rank) v[i] = act_get(z + a.off_kv + tid + 256 * i);
+  }
+  // rotated query part of every head; columns from the real width on are zero
+  for (int e = tid; e < a.H * half; e += 256) {
+    const int hd = e / half, i = e - hd * half;
+    const float u = act_get(z + a.off_qr + hd * a.rot + i), w = act_get(z + a.off_qr + hd * a.rot + half + i);
+    const float2 cs = tab[i];
+    act_set(q + (size_t)hd * ld + i, u * cs.x - w * cs.y);
+    act_set(q + (size_t)hd * ld + half + i, w * cs.x + u * cs.y);
+  }
+  const int pad = a.rot_p - a.rot;
+  for (int e = tid; e < a.H * pad; e += 256) act_set(q + (size_t)(e / pad) * ld + a.rot + e % pad, 0.f);
+  if (a.off_kv < 0) return;
+  T* row = reinterpret_cast<T*>(a.cache) + ((size_t)seq * a.C + slot) * ld;
+  const float ss = block_sum<4>(v[0] * v[0] + v[1] * v[1], smem);
+  const float inv = 1.f / sqrtf(ss / (float)a.rank + a.eps);
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int c = tid + 256 * i;
+    if (c < a.rank_p) act_set(row + c, c < a.rank ? v[i] * inv * a.norm_w[c] : 0.f);
+  }
+  if (tid < a.rot_p) {
+    float o = 0.f;
+    if (tid < a.rot) {
+      const T* kr = z + a.off_kv + a.rank;
+      const int i = tid < half ? tid : tid - half;
+      const float u = act_get(kr + i), w = act_get(kr + half + i);
+      const float2 cs = tab[i];
+      o = tid < half ? u * cs.x - w * cs.y : w * cs.x + u * cs.y;
+    }
+    act_set(row + a.rank_p + tid, o);
+  }
+}
+
+// ---------------------------------------------------------------------------
+// The walk.  Query rows of a sequence are its (token, head) pairs, 32 of them the columns of an MFMA tile: as in the
+// grouped-query kernels, scores^T [position, query] = rows . Q^T and out^T [column, query] += rows^T . P^T, with a
+// lane owning one query.  A block of 32 cache rows goes global -> LDS once (direct loads, 16-byte chunks XOR-swizzled
+// by row) and serves both products: as the A operand of the scores by rows, and transposed (ds_read_b64_tr_b16) as
+// the A operand of the output.  Probabilities enter the product as bf16 hi + lo.
+// The four waves of a workgroup are WQ groups of query rows x WP groups of positions x WC groups of output columns:
+//   SHARED (many query rows per sequence): WP = 1, all waves walk the same blocks;
+//   else (up to 32 query rows): WQ = 1, the position groups take different blocks and meet through LDS at the end.
+// WC = 2 at the full latent width, where the accumulators of 32 queries and the query fragments of one wave would not
+// fit its registers: both waves make the scores, each one half of the columns.
+// KVT: latent width / 32, RT: width of the rotated part / 64.
+template <int KVT, int RT, bool SHARED>
+struct LatentShape {
+  static constexpr int WC = KVT > 8 ? 2 : 1, WQ = SHARED ? 4 / WC : 1, WP = SHARED ? 1 : 4 / WC;
+  static constexpr int kLd = KVT * 32 + RT * 64;
+  static constexpr size_t kTile = (size_t)32 * kLd * 2;
+  static constexpr int kBufs = 2 * WP * kTile <= 160 * 1024 ? 2 : 1;  // tiles per position group
+  static constexpr size_t kTiles = kBufs * WP * kTile;
+  static constexpr size_t kMerge = SHARED ? 0 : (size_t)(WP / 2) * (KVT * 16 * 64 * 4 + WC * 2 * 32 * 4);
+  static constexpr size_t kBytes = kTiles > kMerge ? kTiles : kMerge;
+};
+
+// 16-byte chunk c of row r lies at chunk c ^ swz(r).  Rows whose stride is a multiple of the 64 banks are told apart
+// by four bits of the row; rows of an odd number of 128 bytes already alternate between the two halves of the banks
+// and take three.  Row bits 0, 1 (1) go to the high bits so that the four rows of a transposing read differ by
+// whole groups of four chunks.
+template <int CPR>
+__device__ __forceinline__ constexpr int latent_swz(int row) {
+  return CPR % 16 == 0 ? ((row & 3) << 2) | ((row >> 2) & 3) : (((row >> 1) & 1) << 2) | ((row >> 2) & 3);
+}
+
+template <int KVT, int RT, bool SHARED>
+__global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
+  using SH = LatentShape<KVT, RT, SHARED>;
+  extern __shared__ __align__(16) unsigned char la_smem[];
+  constexpr int LD = SH::kLd, CPR = LD / 8, KS = LD / 16, CP = KVT * 32;
+  constexpr int WC = SH::WC, WP = SH::WP, KC = KVT / WC;  // KC: column tiles of a wave
+  constexpr int kTile = 32 * LD;                          // elements
+  constexpr int WPW = 4 / WP;                             // waves per position group
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int h = lane >> 5, qi = lane & 31;
+  const int wc = wave % WC, wq = SHARED ? wave / WC : 0, wp = SHARED ? 0 : wave / WC;
+  const int wg = wave % WPW;  // wave within its position group
+  const int seq = blockIdx.y, split = blockIdx.z;
+  const int rows = a.tpp * a.H;  // query rows of a sequence
+  const int step0 = max(min(*a.step, min(a.C, a.buf_len) - a.tpp), 0);  // clamped: every slot read lies in the cache
+  const int q0 = blockIdx.x * (32 * SH::WQ);
+  const int qr = q0 + wq * 32 + qi, qr_l = qr < rows ? qr : rows - 1;
+  const int limit = step0 + qr_l / a.H;  // newest slot this query sees
+  const int q_end = min(q0 + 32 * SH::WQ, rows);
+  const int nblk_all = (step0 + (q_end - 1) / a.H + 32) >> 5;  // blocks up to the newest slot of the workgroup
+  const int bps = (nblk_all + a.nsplit - 1) / a.nsplit;
+  const int b_beg = split * bps, b_end = min(b_beg + bps, nblk_all);
+
+  const size_t qrow = (size_t)seq * rows + qr_l;
+  const uint16_t* qp = reinterpret_cast<const uint16_t*>(a.q) + qrow * LD + (LD / 2) * h;
+  u32x4_t qf[KS];
+#pragma unroll
+  for (int t = 0; t < KS; ++t) qf[t] = *reinterpret_cast<const u32x4_t*>(qp + 8 * t);
+
+  const __amdgpu_buffer_rsrc_t rc = make_rsrc(reinterpret_cast<const uint16_t*>(a.cache) + (size_t)seq * a.C * LD,
+                                              (uint32_t)a.C * LD * 2u);  // rows past the cache read zero
+  uint16_t* tiles = reinterpret_cast<uint16_t*>(la_smem) + wp * SH::kBufs * kTile;
+  auto dma = [&](int blk, uint16_t* tile) __attribute__((always_inline)) {
+    int ln = lane;
+    asm volatile("" : "+v"(ln));  // the offsets are formed at the transfer, not kept in registers over the loop
+#pragma unroll
+    for (int i = 0; i < CPR / 2 / WPW; ++i) {  // 1 KiB per load, the waves of the group share the tile
+      const int ld = wg + WPW * i;
+      const int g = ld * 64 + ln, row = g / CPR, slot = g - row * CPR;
+      load_row_to_lds(rc, tile + ld * 512, (row * CPR + (slot ^ latent_swz<CPR>(row))) * 16, blk * (32 * LD * 2));
+    }
+  };
+  const uint8_t* mrow = a.input_mask + (size_t)seq * a.buf_len;
+  auto mask_byte = [&](int blk) __attribute__((always_inline)) {
+    const int p = blk * 32 + qi;
+    return (h == 0 && p < a.buf_len) ? mrow[p] : (uint8_t)0;
+  };
+
+  f32x16_t o[KC];
+#pragma unroll
+  for (int c = 0; c < KC; ++c)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) o[c][r] = 0.f;
+  float m = -1e30f, l = 0.f;
+
+  auto block = [&](const uint16_t* kt, int blk, uint32_t mbits) __attribute__((always_inline)) {
+    f32x16_t sacc;
+#pragma unroll
+    for (int r = 0; r < 16; ++r) sacc[r] = 0.f;
+    {
+      const uint16_t* kb = kt + qi * LD;
+      const int sw = latent_swz<CPR>(qi);
+#pragma unroll
+      for (int t = 0; t < KS; ++t) {  // lane (position, h) multiplies the half h of its row
+        const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(kb + (((KS * h + t) ^ sw) << 3));
+        sacc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, __builtin_bit_cast(bf16x8_t, qf[t]), sacc, 0, 0, 0);
+      }
+    }
+    float sc[16], mn = m;
+#pragma unroll
+    for (int r = 0; r < 16; ++r) {
+      const int pl = acc_row(r, lane);
+      const bool ok = blk * 32 + pl <= limit && ((mbits >> pl) & 1u);
+      sc[r] = ok ? sacc[r] * a.scale : -1e30f;
+      mn = fmaxf(mn, sc[r]);
+    }
+    mn = fmaxf(mn, __shfl_xor(mn, 32, 64));
+    // the reference point of the exponentials moves only when a score has left it by more than 8: until then the
+    // probabilities stay below e^8 and the accumulators need no rescaling
+    if (__any(mn > m + 8.f)) {
+      const float alpha = __expf(m - mn);
+      m = mn;
+      l *= alpha;
+#pragma unroll
+      for (int c = 0; c < KC; ++c)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) o[c][r] *= alpha;
+    }
+    uint32_t pk[8], pl2[8];
+#pragma unroll
+    for (int r = 0; r < 16; r += 2) {
+      const float p0 = sc[r] > -1e29f ? __expf(sc[r] - m) : 0.f;
+      const float p1 = sc[r + 1] > -1e29f ? __expf(sc[r + 1] - m) : 0.f;
+      pk[r >> 1] = pack_bf2(p0, p1);
+      pl2[r >> 1] = pack_bf2(p0 - bf_lo(pk[r >> 1]), p1 - bf_hi(pk[r >> 1]));
+      l += p0 + p1;
+    }
+    // out^T += rows^T . P^T, 16 positions (accumulator registers 8 kb2 .. 8 kb2 + 7) per MFMA; the transposed
+    // fragment of lane (column 32 c + qi, h) is two runs of four consecutive rows (see gqa_tile_walk)
+    typedef short s16x4_t __attribute__((ext_vector_type(4)));
+    const int k4 = (lane & 15) >> 2, q4 = lane & 3, g2 = (lane >> 4) & 1;
+    const int lsw = (2 * g2 + (q4 >> 1)) ^ latent_swz<CPR>(4 * h + k4);
+    const uint16_t* vb = kt + (4 * h + k4) * LD + 4 * (q4 & 1) + wc * KC * 32;
+#pragma unroll
+    for (int kb2 = 0; kb2 < 2; ++kb2) {
+      const u32x4_t pf = {pk[4 * kb2], pk[4 * kb2 + 1], pk[4 * kb2 + 2], pk[4 * kb2 + 3]};
+      const u32x4_t pg = {pl2[4 * kb2], pl2[4 * kb2 + 1], pl2[4 * kb2 + 2], pl2[4 * kb2 + 3]};
+#pragma unroll
+      for (int c = 0; c < KC; ++c) {
+        s16x4_t run[2];
+#pragma unroll
+        for (int a2 = 0; a2 < 2; ++a2) {
+          const int row0 = 16 * kb2 + 8 * a2;
+          run[a2] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4_t*)(
+              vb + row0 * LD + ((lsw ^ (4 * c) ^ latent_swz<CPR>(row0)) << 3)));
+        }
+        uint32_t vw[4];
+        __builtin_memcpy(&vw[0], &run[0], 8);
+        __builtin_memcpy(&vw[2], &run[1], 8);
+        const u32x4_t vf = {vw[0], vw[1], vw[2], vw[3]};
+        o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, vf),
+                                                       __builtin_bit_cast(bf16x8_t, pf), o[c], 0, 0, 0);
+        o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, vf),
+                                                       __builtin_bit_cast(bf16x8_t, pg), o[c], 0, 0, 0);
+      }
+    }
+  };
+
+  // position group wp takes the blocks b_beg + wp, b_beg + wp + WP, ...; all groups run the same number of rounds
+  const int rounds = b_end > b_beg ? (b_end - b_beg + WP - 1) / WP : 0;
+  auto blk_of = [&](int round) { return b_beg + round * WP + wp; };
+  auto fetch = [&](int round, int buf) __attribute__((always_inline)) {
+    if (round < rounds && blk_of(round) < b_end) dma(blk_of(round), tiles + buf * kTile);
+  };
+  uint8_t mb = mask_byte(blk_of(0));
+  if (SH::kBufs == 2) fetch(0, 0);
+  for (int round = 0; round < rounds; ++round) {
+    const int buf = SH::kBufs == 2 ? round & 1 : 0;
+    if (SH::kBufs == 1) {
+      __syncthreads();  // the last round's reads are complete
+      fetch(round, 0);
+    }
+    const uint32_t mbits = (uint32_t)__ballot(mb != 0);
+    __builtin_amdgcn_s_waitcnt(0x0F70);  // this round's tile has landed
+    __syncthreads();
+    mb = mask_byte(blk_of(round + 1));
+    if (SH::kBufs == 2) fetch(round + 1, buf ^ 1);
+    if (blk_of(round) < b_end) block(tiles + buf * kTile, blk_of(round), mbits);
+  }
+  l += __shfl_xor(l, 32, 64);
+  if constexpr (WP > 1) {
+    // merge the position groups: the upper half of them hands its state to the lower half, until one is left
+    constexpr int kPart = KVT * 16 * 64;
+    float* mf = reinterpret_cast<float*>(la_smem);
+    float* ml = mf + (WP / 2) * kPart;  // [slot][column group][m, l][32]
+    auto put = [&](int s) __attribute__((always_inline)) {
+#pragma unroll
+      for (int c = 0; c < KC; ++c)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) mf[s * kPart + (((wc * KC + c) * 16 + r) << 6) + lane] = o[c][r];
+      if (h == 0) {
+        ml[(s * WC + wc) * 64 + qi] = m;
+        ml[(s * WC + wc) * 64 + 32 + qi] = l;
+      }
+    };
+    auto take = [&](int s) __attribute__((always_inline)) {
+      const float m2 = ml[(s * WC + wc) * 64 + qi], l2 = ml[(s * WC + wc) * 64 + 32 + qi];
+      const float mm = fmaxf(m, m2), w1 = __expf(m - mm), w2 = __expf(m2 - mm);
+#pragma unroll
+      for (int c = 0; c < KC; ++c)
+#pragma unroll
+        for (int r = 0; r < 16; ++r)
+          o[c][r] = o[c][r] * w1 + mf[s * kPart + (((wc * KC + c) * 16 + r) << 6) + lane] * w2;
+      l = l * w1 + l2 * w2;
+      m = mm;
+    };
+#pragma unroll
+    for (int n = WP / 2; n > 0; n >>= 1) {
+      __syncthreads();
+      if (wp >= n && wp < 2 * n) put(wp - n);
+      __syncthreads();
+      if (wp < n) take(wp);
+    }
+    if (wp != 0) return;
+  }
+  if (qr >= rows) return;
+  if (a.nsplit == 1) {
+    float w = 1.f;
+    if (a.sink) {  // one more term of the denominator, without a value
+      const float s = a.sink[qr % a.H], mm = fmaxf(m, s);
+      w = __expf(m - mm);
+      l = l * w + __expf(s - mm);
+    }
+    const float inv = l > 0.f ? w / l : 0.f;
+    uint16_t* dst = reinterpret_cast<uint16_t*>(a.out) + qrow * CP + wc * KC * 32;
+#pragma unroll
+    for (int c = 0; c < KC; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        uint2 v;
+        v.x = pack_bf2(o[c][4 * i] * inv, o[c][4 * i + 1] * inv);
+        v.y = pack_bf2(o[c][4 * i + 2] * inv, o[c][4 * i + 3] * inv);
+        *reinterpret_cast<uint2*>(dst + 32 * c + 8 * i + 4 * h) = v;
+      }
+    return;
+  }
+  float* pr = a.partial + (qrow * a.nsplit + split) * (CP + 2);
+#pragma unroll
+  for (int c = 0; c < KC; ++c)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float* d = pr + 32 * (wc * KC + c) + 8 * i + 4 * h;
+      *reinterpret_cast<f32x2_t*>(d) = f32x2_t{o[c][4 * i], o[c][4 * i + 1]};
+      *reinterpret_cast<f32x2_t*>(d + 2) = f32x2_t{o[c][4 * i + 2], o[c][4 * i + 3]};
+    }
+  if (h == 0 && wc == 0) {
+    pr[CP] = m;
+    pr[CP + 1] = l;
+  }
+}
+
+// One workgroup per query row: the softmax-weighted sum of its splits, then the sink.
+__global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnArgs a) {
+  const int CP = a.rank_p;
+  const size_t row = blockIdx.x;
+  const float* pr = a.partial + row * a.nsplit * (CP + 2);
+  float mm = a.sink ? a.sink[row % a.H] : -1e30f;
+  const float sink = mm;
+  for (int s = 0; s < a.nsplit; ++s) mm = fmaxf(mm, pr[(size_t)s * (CP + 2) + CP]);
+  float l = a.sink ? __expf(sink - mm) : 0.f;
+  for (int s = 0; s < a.nsplit; ++s) l += pr[(size_t)s * (CP + 2) + CP + 1] * __expf(pr[(size_t)s * (CP + 2) + CP] - mm);
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  for (int c = threadIdx.x * 2; c < CP; c += 512) {
+    f32x2_t v = {0.f, 0.f};
+#pragma unroll 4
+    for (int s = 0; s < a.nsplit; ++s) {
+      const float* p = pr + (size_t)s * (CP + 2);
+      const float w = __expf(p[CP] - mm);
+      const f32x2_t x = *reinterpret_cast<const f32x2_t*>(p + c);
+      v.x = fmaf(x.x, w, v.x);
+      v.y = fmaf(x.y, w, v.y);
+    }
+    *reinterpret_cast<uint32_t*>(reinterpret_cast<uint16_t*>(a.out) + row * CP + c) = pack_bf2(v.x * inv, v.y * inv);
+  }
+}
+
+// f32: one workgroup per (head, row); 256 positions at a time, a thread scores one of them and then owns columns of
+// the output.
+__global__ __launch_bounds__(256) void latent_attn_f32_kernel(LatentAttnArgs a) {
+  __shared__ __align__(16) float qs[TMX_MAX_LATENT_RANK + TMX_MAX_LATENT_ROT];
+  __shared__ float ps[256], red[4];
+  const int hd = blockIdx.x, m = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int seq = m / a.tpp, ld = a.rank_p + a.rot_p;
+  const int step0 = max(min(*a.step, min(a.C, a.buf_len) - a.tpp), 0);
+  const int limit = step0 + m % a.tpp;
+  const size_t qrow = (size_t)m * a.H + hd;
+  for (int i = tid; i < ld; i += 256) qs[i] = reinterpret_cast<const float*>(a.q)[qrow * ld + i];
+  const float* cache = reinterpret_cast<const float*>(a.cache) + (size_t)seq * a.C * ld;
+  const uint8_t* mrow = a.input_mask + (size_t)seq * a.buf_len;
+  float mx = a.sink ? a.sink[hd] : -1e30f, l = a.sink ? 1.f : 0.f;
+  float o[2] = {0.f, 0.f};
+  __syncthreads();
+  for (int p0 = 0; p0 <= limit; p0 += 256) {
+    const int p = p0 + tid;
+    const bool ok = p <= limit && mrow[p];
+    float s = -1e30f;
+    if (ok) {
+      const float4* row = reinterpret_cast<const float4*>(cache + (size_t)p * ld);
+      float d = 0.f;
+      for (int i = 0; i < ld / 4; ++i) {
+        const float4 k = row[i], qv = *reinterpret_cast<const float4*>(qs + 4 * i);
+        d = fmaf(k.x, qv.x, d); d = fmaf(k.y, qv.y, d); d = fmaf(k.z, qv.z, d); d = fmaf(k.w, qv.w, d);
+      }
+      s = d * a.scale;
+    }
+    float top = wave_max(s);
+    __syncthreads();  // the last chunk's ps and red are free
+    if (lane == 0) red[wave] = top;
+    __syncthreads();
+    const float mn = fmaxf(mx, fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])));
+    const float alpha = expf(mx - mn);
+    mx = mn;
+    const float pr = ok ? expf(s - mn) : 0.f;
+    ps[tid] = pr;
+    const float sum = block_sum<4>(pr, red);  // its barriers also publish ps
+    l = l * alpha + sum;
+    const int n = min(256, limit - p0 + 1);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int c = tid + 256 * i;
+      if (c >= a.rank_p) continue;
+      float v = o[i] * alpha;
+      for (int j = 0; j < n; ++j) v = fmaf(ps[j], cache[(size_t)(p0 + j) * ld + c], v);
+      o[i] = v;
+    }
+  }
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int c = tid + 256 * i;
+    if (c < a.rank_p) reinterpret_cast<float*>(a.out)[qrow * a.rank_p + c] = o[i] * inv;
+  }
+}
+
+// ---------------------------------------------------------------------------
+int latent_rows(hipStream_t st, int act, const LatentRowsArgs& a, int M) {
+  if (M <= 0 || a.H <= 0 || a.rot <= 0 || a.rot % 2 || a.rot > a.rot_p || a.rank > a.rank_p || a.rank <= 0 ||
+      !latent_attn_ok(a.rank_p, a.rot_p))
+    return TMX_ERR_SHAPE;
+  if (act == TMX_ACT_BF16) hipLaunchKernelGGL(latent_rows_kernel<uint16_t>, dim3(M), dim3(256), 0, st, a);
+  else if (act == TMX_ACT_F32) hipLaunchKernelGGL(latent_rows_kernel<float>, dim3(M), dim3(256), 0, st, a);
+  else return TMX_ERR_ARG;
+  return check_launch();
+}
+
+bool latent_attn_ok(int rank_p, int rot_p) {
+  return (rank_p == 64 || rank_p == 128 || rank_p == 256 || rank_p == 512) && (rot_p == 64 || rot_p == 128);
+}
+
+// A workgroup holds 64 or 128 query rows of a sequence, or 32 with its position groups on different blocks; the positions are split
+// until every CU has a workgroup (one fits a CU at the full latent width).
+struct LatentPlan { bool shared; int nsplit; };
+constexpr int kLatentWgs = 256, kLatentMaxSplits = 32;
+static int latent_block_rows(int rank_p, bool shared) { return !shared ? 32 : (rank_p > 256 ? 64 : 128); }
+static LatentPlan latent_plan(int n_seq, int T, int H, int rank_p, int C) {
+  LatentPlan p;
+  const int rows = T * H;
+  p.shared = rows > 32;
+  const int per = latent_block_rows(rank_p, p.shared);
+  const long wgs = (long)n_seq * ((rows + per - 1) / per);
+  long ns = kLatentWgs / wgs;
+  const int by_len = (C + 127) / 128;  // at least four blocks of 32 positions per split
+  if (ns > by_len) ns = by_len;
+  if (ns > kLatentMaxSplits) ns = kLatentMaxSplits;
+  p.nsplit = ns < 1 ? 1 : (int)ns;
+  return p;
+}
+
+size_t latent_attn_partial_bytes(int rows, int H, int rank_p) {
+  // nsplit > 1 only while nsplit * workgroups <= kLatentWgs, and a workgroup holds at most 128 query rows
+  size_t parts = (size_t)rows * H * kLatentMaxSplits;
+  if (parts > (size_t)kLatentWgs * 128) parts = (size_t)kLatentWgs * 128;
+  return parts * (rank_p + 2) * 4;
+}
+
+template <int KVT, int RT, bool SHARED>
+static int launch_latent(hipStream_t st, const LatentAttnArgs& a) {
+  using L = LatentShape<KVT, RT, SHARED>;
+  static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<KVT, RT, SHARED>),
+                                                     hipFuncAttributeMaxDynamicSharedMemorySize, (int)L::kBytes);
+  if (attr != hipSuccess) return TMX_ERR_LAUNCH;
+  const int per = 32 * L::WQ;
+  hipLaunchKernelGGL((latent_attn_kernel<KVT, RT, SHARED>), dim3((a.tpp * a.H + per - 1) / per, a.n_seq, a.nsplit),
+                     dim3(256), L::kBytes, st, a);
+  return check_launch();
+}
+template <int KVT>
+static int launch_latent_k(hipStream_t st, const LatentAttnArgs& a, bool shared) {
+  if (a.rot_p == 64) return shared ? launch_latent<KVT, 1, true>(st, a) : launch_latent<KVT, 1, false>(st, a);
+  return shared ? launch_latent<KVT, 2, true>(st, a) : launch_latent<KVT, 2, false>(st, a);
+}
+
+int latent_attention(hipStream_t st, int act, LatentAttnArgs a) {
+  if (a.n_seq <= 0 || a.n_seq > 65535 || a.tpp <= 0 || a.H <= 0 || a.C <= 0 || a.tpp > a.C ||
+      !latent_attn_ok(a.rank_p, a.rot_p))
+    return TMX_ERR_SHAPE;
+  if (act == TMX_ACT_F32) {
+    if ((long)a.n_seq * a.tpp > 65535) return TMX_ERR_SHAPE;
+    hipLaunchKernelGGL(latent_attn_f32_kernel, dim3(a.H, a.n_seq * a.tpp), dim3(256), 0, st, a);
+    return check_launch();
+  }
+  if (act != TMX_ACT_BF16) return TMX_ERR_ARG;
+  if ((size_t)a.C * (a.rank_p + a.rot_p) * 2 >= (1u << 31)) return TMX_ERR_SHAPE;
+  const LatentPlan p = latent_plan(a.n_seq, a.tpp, a.H, a.rank_p, a.C);
+  a.nsplit = p.nsplit;
+  if (a.nsplit > 1 && !a.partial) return TMX_ERR_ARG;
+  int rc;
+  switch (a.rank_p) {
+    case 64: rc = launch_latent_k<2>(st, a, p.shared); break;
+    case 128: rc = launch_latent_k<4>(st, a, p.shared); break;
+    case 256: rc = launch_latent_k<8>(st, a, p.shared); break;
+    default: rc = launch_latent_k<16>(st, a, p.shared); break;
+  }
+  if (rc != TMX_OK || a.nsplit == 1) return rc;
+  hipLaunchKernelGGL(latent_combine_kernel, dim3(a.n_seq * a.tpp * a.H), dim3(a.rank_p >= 512 ? 256 : (a.rank_p >= 256 ? 128 : 64)),
+                     0, st, a);
+  return check_launch();
+}
+
+}  // namespace tmx
+
+using namespace tmx;
+
+extern "C" int tmx_latent_rows(void* stream, int act, const void* z, int ldz, int off_qr, int off_kv,
+                               const float* norm_w, float eps, const float* table, int positions_max,
+                               const int32_t* positions, const int32_t* step, int buf_len, void* q, void* cache, int M,
+                               int T, int H, int rot, int rank, int rank_p, int rot_p, int C) {
+  if (!z || !table || !positions || !step || !q || (off_kv >= 0 && (!norm_w || !cache))) return TMX_ERR_ARG;
+  LatentRowsArgs a = {};
+  a.z = z; a.ldz = ldz; a.off_qr = off_qr; a.off_kv = off_kv; a.norm_w = norm_w; a.eps = eps; a.table = table;
+  a.max_positions = positions_max; a.positions = positions; a.step = step; a.buf_len = buf_len; a.tpp = T;
+  a.q = q; a.cache = cache; a.H = H; a.rot = rot; a.rank = rank; a.rank_p = rank_p; a.rot_p = rot_p; a.C = C;
+  return latent_rows((hipStream_t)stream, act, a, M);
+}
+
+extern "C" size_t tmx_latent_attention_workspace_bytes(int n_seq, int T, int H, int rank_p, int C) {
+  if (n_seq <= 0 || T <= 0 || H <= 0 || C <= 0) return 0;
+  const LatentPlan p = latent_plan(n_seq, T, H, rank_p, C);
+  return p.nsplit == 1 ? 0 : (size_t)n_seq * T * H * p.nsplit * (rank_p + 2) * 4;
+}
+
+extern "C" int tmx_latent_attention(void* stream, int act, const void* q, const void* cache, const float* sink,
+                                    const uint8_t* input_mask, const int32_t* step, int buf_len, void* out,
+                                    void* workspace, int n_seq, int T, int H, int rank_p, int rot_p, int C,
+                                    float scale) {
+  if (!q || !cache || !input_mask || !step || !out) return TMX_ERR_ARG;
+  LatentAttnArgs a = {};
+  a.q = q; a.cache = cache; a.sink = sink; a.input_mask = input_mask; a.step = step; a.buf_len = buf_len;
+  a.out = out; a.partial = (float*)workspace; a.n_seq = n_seq; a.tpp = T; a.H = H; a.rank_p = rank_p;
+  a.rot_p = rot_p; a.C = C; a.scale = scale;
+  return latent_attention((hipStream_t)stream, act, a);
+}

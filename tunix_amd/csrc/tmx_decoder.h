@@ -1,0 +1,48 @@
+// Shared by the translation units that enqueue a decode step.
+#pragma once
+#include <vector>
+
+#include "tmx_kernels.h"
+
+namespace tmx {
+
+inline size_t align256(size_t v) { return (v + 255) & ~(size_t)255; }
+
+// Optional per-kernel-class timing with HIP events (used by the benchmark only).
+struct Prof {
+  std::vector<hipEvent_t> ev[TMX_NUM_KERNEL_CLASSES];
+  void before(int k, hipStream_t st) { push(k, st); }
+  void after(int k, hipStream_t st) { push(k, st); }
+  void push(int k, hipStream_t st) {
+    hipEvent_t e;
+    if (hipEventCreate(&e) != hipSuccess) return;
+    (void)hipEventRecord(e, st);
+    ev[k].push_back(e);
+  }
+};
+
+#define TMX_TRY(kind, expr)            \
+  {                                    \
+    if (prof) prof->before(kind, st);  \
+    rc = (expr);                       \
+    if (prof) prof->after(kind, st);   \
+    if (rc != TMX_OK) return rc;       \
+  }
+
+// TMX_FAMILY_LATENT: workspace of a pass of `rows` rows (the first 256 bytes are the status block of every family).
+struct LatentWorkspace {
+  float* xs;            // residual streams [rows][S][Dp]
+  void *xn, *z, *q, *lat, *val, *y, *act;
+  float* attn_partial;
+  float* logits;        // f32 models: products of the head [rows][Vp]
+  void* head_partial;
+  size_t total;
+};
+LatentWorkspace latent_carve(const tmx_model_desc* m, int rows, char* base);
+int latent_check(const tmx_model_desc* m);
+// Embedding and every layer of one pass; with final_norm w.xn is the head's input afterwards.
+int latent_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_state* s, const LatentWorkspace& w,
+                  int n_seq, int T, bool final_norm, Prof* prof);
+inline int pad_to(int v, int k) { return (v + k - 1) / k * k; }
+
+}  // namespace tmx

@@ -198,6 +198,9 @@ struct HeadArgs {
   int row_base;  // score mode: x holds rows row_base .. row_base + M - 1 of the pass (chunks of <= 128 rows)
   int row_off;   // set by head_logits when it splits the rows over two launches: x, logits_out, sort_keys and the
                  // partials point at row row_off of the call, whose index the sort keys and the noise counter use
+  float logit_scale = 1.f;     // logits = bf16(product * logit_scale)
+  int v_live = 0x7FFFFFFF;     // vocabulary rows from here on are padding: never chosen, no probability
+  bool logits_ready = false;   // logits_out already holds the f32 products (f32 models): head_logits only selects
 };
 
 
@@ -267,6 +270,72 @@ struct SbAttnArgs {
   float eps;
   int family;                // rotation rounding: TMX_FAMILY_*
 };
+
+// Projection by a dense (unquantised) matrix, see tmx_dense_linear.
+struct DenseArgs {
+  const void* x;       // act [M][ldx], matrix h reads columns h x_head ..
+  int ldx, x_head;
+  const void* w;       // bf16: `heads` matrices in the tile layout of head_tiles_kernel; f32: [heads][N][K]
+  const float* bias;
+  const void* gate;    // TMX_DENSE_GATED
+  int ldg;
+  void* y;
+  int ldy, y_head;
+  int M, K, N, heads, epi;
+};
+
+// Mixing of the residual streams + the next sublayer's norm, see tmx_stream_rows; with `embed` set the streams are
+// first filled with embed[token] + pos_embed[position] of every row.
+struct StreamArgs {
+  float* xs;           // [M][S][Dp]
+  const void* y;       // act [M][Dp] or null
+  const float *mix, *out, *in, *norm_w;
+  void* xn;
+  int S, D, Dp, store;
+  float eps;
+  const uint16_t* embed;      // bf16 [vocab, Dp]
+  const uint16_t* pos_embed;  // bf16 [max_positions, Dp] or null
+  int vocab, max_positions;
+  const int32_t* token_buffer;
+  const int32_t* positions;
+  const int32_t* step;
+  int buf_len, tpp;
+};
+
+struct LatentRowsArgs {  // see tmx_latent_rows
+  const void* z;
+  int ldz, off_qr, off_kv;
+  const float* norm_w;
+  float eps;
+  const float* table;
+  int max_positions;
+  const int32_t* positions;
+  const int32_t* step;
+  int buf_len, tpp;
+  void* q;
+  void* cache;
+  int H, rot, rank, rank_p, rot_p, C;
+};
+
+struct LatentAttnArgs {  // see tmx_latent_attention
+  const void* q;
+  const void* cache;
+  const float* sink;
+  const uint8_t* input_mask;
+  const int32_t* step;
+  int buf_len;
+  void* out;
+  float* partial;  // [rows H][nsplit][rank_p + 2]
+  int n_seq, tpp, H, rank_p, rot_p, C, nsplit;
+  float scale;
+};
+
+int dense_linear(hipStream_t st, int act, const DenseArgs& a);
+int stream_rows(hipStream_t st, int act, const StreamArgs& a, int M);
+int latent_rows(hipStream_t st, int act, const LatentRowsArgs& a, int M);
+int latent_attention(hipStream_t st, int act, LatentAttnArgs a);
+bool latent_attn_ok(int rank_p, int rot_p);
+size_t latent_attn_partial_bytes(int rows, int H, int rank_p);  // room for every split of `rows` query rows
 
 int sb_linear(hipStream_t st, const SbLinearArgs& a, int pro, int epi);  // pro: 0 plain, 1 norm, 2 attention merge; epi: 0 plain, 1 residual, 2 SwiGLU
 bool sb_linear_ok(int M, int K, int N, int G, int rank, int rpad, bool norm);

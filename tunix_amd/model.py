@@ -14,7 +14,7 @@ import torch
 from tunix_amd import quant
 from tunix_amd import _lib
 
-FAMILY_LLAMA3, FAMILY_QWEN3 = 0, 1
+FAMILY_LLAMA3, FAMILY_QWEN3, FAMILY_LATENT = 0, 1, 2
 SAMPLE_GREEDY, SAMPLE_TOP_P, SAMPLE_SCORE = 0, 1, 2
 MAX_RPAD = 128
 
@@ -36,6 +36,34 @@ class ModelConfig:
   weight_tying: bool = False
   num_experts: Optional[int] = None
   num_experts_per_tok: Optional[int] = None
+
+  MAX_MOE_PAIRS = 8192  # routed (token, expert) pairs of one pass of a MoE model
+
+  def max_rows(self):
+    """Rows one pass can take: more than 128 need the 256-row projection blocks (every attention /
+    dense-MLP projection with K % 128 == 0); MoE models are bounded by the routed pairs per pass."""
+    ks = [self.embed_dim, self.num_heads * self.head_dim] + ([] if self.num_experts else [self.hidden_dim])
+    if not all(k % 128 == 0 for k in ks):
+      return 128
+    if self.num_experts:
+      return max(128, min(4096, self.MAX_MOE_PAIRS // self.num_experts_per_tok))
+    return 4096
+
+  max_rows_rule = '4096 when every projection has K % 128 == 0, MoE models 8192 / experts per token, else 128'
+  max_positions = None  # positions are not bounded by a table
+
+  def cache_shape(self, batch, cache_size):
+    """Shape of the cache tensor of `batch` sequences: [layers][k|v][B][C][Kh][H]."""
+    return (self.num_layers, 2, batch, cache_size, self.num_kv_heads, self.head_dim)
+
+  def cache_rows(self, cache, batch, cache_size):
+    """Views [B, C, ...] of a cache tensor, together all of it (a list of leading-axis views)."""
+    del batch, cache_size
+    return [cache[i, j] for i in range(self.num_layers) for j in range(2)]
+
+  @property
+  def logits_width(self):
+    return self.vocab_size
 
   @classmethod
   def from_reference(cls, cfg, family=None):
@@ -86,13 +114,35 @@ class LayerDesc(ctypes.Structure):
               ('gate_up', QLinearDesc), ('down', QLinearDesc), ('router_w', ctypes.c_void_p)]
 
 
+class DenseDesc(ctypes.Structure):
+  _fields_ = [('w', ctypes.c_void_p), ('bias', ctypes.c_void_p), ('K', ctypes.c_int), ('N', ctypes.c_int),
+              ('heads', ctypes.c_int)]
+
+
+class StreamsDesc(ctypes.Structure):
+  _fields_ = [('in_', ctypes.c_void_p), ('out', ctypes.c_void_p), ('mix', ctypes.c_void_p)]
+
+
+class LatentLayerDesc(ctypes.Structure):
+  _fields_ = [('norm1_w', ctypes.c_void_p), ('norm2_w', ctypes.c_void_p), ('hc1', StreamsDesc), ('hc2', StreamsDesc),
+              ('heads', ctypes.c_int), ('rot_dim', ctypes.c_int), ('kv_rank', ctypes.c_int), ('dim_p', ctypes.c_int),
+              ('rot_p', ctypes.c_int), ('rank_p', ctypes.c_int), ('vdim_p', ctypes.c_int), ('off_qr', ctypes.c_int),
+              ('off_kv', ctypes.c_int), ('off_gate', ctypes.c_int), ('kv_layer', ctypes.c_int),
+              ('scale', ctypes.c_float), ('in_', DenseDesc), ('uk', DenseDesc), ('uv', DenseDesc), ('o', DenseDesc),
+              ('kv_norm_w', ctypes.c_void_p), ('table', ctypes.c_void_p), ('sink', ctypes.c_void_p),
+              ('gate_up', DenseDesc), ('down', DenseDesc)]
+
+
 class ModelDesc(ctypes.Structure):
   _fields_ = [('family', ctypes.c_int), ('num_layers', ctypes.c_int), ('vocab_size', ctypes.c_int),
               ('embed_dim', ctypes.c_int), ('hidden_dim', ctypes.c_int), ('num_heads', ctypes.c_int),
               ('num_kv_heads', ctypes.c_int), ('head_dim', ctypes.c_int), ('num_experts', ctypes.c_int),
               ('experts_per_tok', ctypes.c_int), ('rope_theta', ctypes.c_float),
               ('norm_eps', ctypes.c_float), ('embed', ctypes.c_void_p), ('final_norm_w', ctypes.c_void_p),
-              ('head', ctypes.c_void_p), ('layers', ctypes.POINTER(LayerDesc)), ('head_tiles', ctypes.c_void_p)]
+              ('head', ctypes.c_void_p), ('layers', ctypes.POINTER(LayerDesc)), ('head_tiles', ctypes.c_void_p),
+              ('latent_layers', ctypes.POINTER(LatentLayerDesc)), ('act', ctypes.c_int), ('streams', ctypes.c_int),
+              ('max_positions', ctypes.c_int), ('pos_embed', ctypes.c_void_p), ('final_in', ctypes.c_void_p),
+              ('logit_scale', ctypes.c_float)]
 
 
 class DecodeState(ctypes.Structure):
@@ -283,9 +333,7 @@ class QLoRAModel:
   def init_cache(self, batch_size, cache_size, dtype=torch.bfloat16):
     """One allocation [layers][k|v][B][C][Kh][H]; layer i's 'k' is cache[i, 0].
     (tunix/generate/sampler.py:171-202, qwen3/model.py:1359-1373.)"""
-    c = self.config
-    return torch.zeros(c.num_layers, 2, batch_size, cache_size, c.num_kv_heads, c.head_dim,
-                       dtype=dtype, device=self.device)
+    return torch.zeros(self.config.cache_shape(batch_size, cache_size), dtype=dtype, device=self.device)
 
   def lora_state(self):
     """Flat dict of the LoRA tensors (the nnx.LoRAParam leaves of the reference)."""

@@ -165,6 +165,11 @@ class Sampler:
   def dtype(self):
     return self._transformer.dtype
 
+  def _check_positions(self, length):
+    limit = self._transformer.config.max_positions
+    if limit is not None and length > limit:
+      raise ValueError(f'a sequence of {length} tokens exceeds the {limit} positions of the model')
+
   def tokenize(self, input_string):
     ids = self.tokenizer.encode(input_string)
     bos = [self.tokenizer.bos_id()] if self.tokenizer.bos_id() else []
@@ -209,7 +214,7 @@ class Sampler:
     positions = utils.build_positions_from_mask(input_mask)
     share = shared_prompt_groups(ids, input_mask[:, :p]) if self.share_prompt_kv else (1, 0, 0)
     c = self._transformer.config
-    need = (c.num_layers, 2, b, self.cache_config.cache_size, c.num_kv_heads, c.head_dim)
+    need = c.cache_shape(b, self.cache_config.cache_size)
     if self._cache is None or tuple(self._cache.shape) != need:
       self._cache = None
       self._cache = self._transformer.init_cache(b, self.cache_config.cache_size)
@@ -237,7 +242,7 @@ class Sampler:
         'forbidden': torch.tensor(list(forbidden_token_ids), dtype=torch.int32, device=dev)
                      if forbidden_token_ids else None,
         'eos': torch.tensor(np.asarray(self.eos_ids).reshape(-1), dtype=torch.int32, device=dev),
-        'logits': torch.zeros(b, c.vocab_size, dtype=torch.float32, device=dev) if include_logits else None,
+        'logits': torch.zeros(b, c.logits_width, dtype=torch.float32, device=dev) if include_logits else None,
     }
     return st
 
@@ -247,7 +252,7 @@ class Sampler:
     if rows > self._max_rows():
       raise ValueError(
           f'{b} sequences x {max(tokens_per_pass, 1)} tokens per pass: this model takes at most {self._max_rows()} rows '
-          '(4096 when every projection has K % 128 == 0, MoE models 8192 / experts per token, else 128)')
+          f'({self._transformer.config.max_rows_rule})')
     ws_bytes = self._lib.tmx_decode_workspace_bytes(
         ctypes.byref(self._transformer.desc()), b * tokens_per_pass, self.cache_config.cache_size)
     if self._workspace is None or self._workspace.numel() < ws_bytes:
@@ -273,7 +278,7 @@ class Sampler:
     s.workspace, s.workspace_bytes = self._workspace.data_ptr(), self._workspace.numel()
     if s.sampling_mode == SAMPLE_TOP_P and (s.top_p < 1.0 or s.top_k > 0):
       # the sorting branch of sample_top_p needs room for one sort key per logit
-      nb = self._lib.tmx_nucleus_workspace_bytes(b, self._transformer.config.vocab_size)
+      nb = self._lib.tmx_nucleus_workspace_bytes(b, self._transformer.config.logits_width)
       if nb == 0:
         raise _lib.TmxError('tmx_nucleus_workspace_bytes returned 0 (no device, or batch x vocab too large)')
       if self._nucleus_ws is None or self._nucleus_ws.numel() < nb:
@@ -284,19 +289,10 @@ class Sampler:
   MAX_ROWS = 128        # rows of one pass that chooses tokens (sequences x tokens per pass)
   MAX_FILL_ROWS = 4096  # rows of one cache-fill or scoring pass of a dense model (256-row projection blocks)
 
-  MAX_MOE_PAIRS = 8192  # routed (token, expert) pairs of one pass of a MoE model
   MAX_PASSES_IN_FLIGHT = 64  # passes a walk enqueues before it waits for the stream
 
   def _max_rows(self):
-    """Rows one pass can take: more than 128 need the 256-row projection blocks (every attention /
-    dense-MLP projection with K % 128 == 0); MoE models are bounded by the routed pairs per pass."""
-    cfg = self._transformer.config
-    ks = [cfg.embed_dim, cfg.num_heads * cfg.head_dim] + ([] if cfg.num_experts else [cfg.hidden_dim])
-    if not all(k % 128 == 0 for k in ks):
-      return 128
-    if cfg.num_experts:
-      return max(128, min(4096, self.MAX_MOE_PAIRS // cfg.num_experts_per_tok))
-    return 4096
+    return self._transformer.config.max_rows()
 
   def _many_rows_ok(self):
     return self._max_rows() > 128
@@ -330,6 +326,33 @@ class Sampler:
         # thousands of short passes otherwise leaves tens of thousands of dispatches pending at once
         torch.cuda.current_stream().synchronize()
 
+  def walk_logits(self, st, n_tokens, wanted):
+    """Advances every sequence by n_tokens known tokens like `walk`, and returns the logits at the wanted places,
+    f32 [len(wanted), vocab] on the device.  wanted: (row, offset) pairs, offset counted from the first token walked.
+    Passes in which nothing is wanted skip the head; the others run it for all of their rows (scoring mode: no token
+    is chosen)."""
+    c = self._transformer.config
+    b = st['token_buffer'].shape[0]
+    per = min(128, max(1, self._fill_rows() // b))
+    out = torch.empty(len(wanted), c.vocab_size, dtype=torch.float32, device=self._transformer.device)
+    keep = st['sampling_mode'], st['logits']
+    passes = 0
+    for beg in range(0, n_tokens, per):
+      t = min(per, n_tokens - beg)
+      here = [(k, row * t + off - beg) for k, (row, off) in enumerate(wanted) if beg <= off < beg + t]
+      if here:
+        st['sampling_mode'], st['logits'] = 'score', torch.empty(b * t, c.logits_width, dtype=torch.float32,
+                                                                 device=self._transformer.device)
+      self.run_steps(st, 1, sample=bool(here), tokens_per_pass=t)
+      if here:
+        dst, src = (torch.tensor(i, device=out.device) for i in zip(*here))
+        out[dst] = st['logits'][src, :c.vocab_size]
+      st['sampling_mode'], st['logits'] = keep
+      passes += 1
+      if passes % self.MAX_PASSES_IN_FLIGHT == 0:
+        torch.cuda.current_stream().synchronize()
+    return out
+
   def _walk_group_leaders(self, st, n):
     """Cache fill over the first n columns, which every group of st['share_group'] consecutive rows has in
     common (the samples of one prompt): the first row of every group is walked, in a cache of its own, and
@@ -340,10 +363,11 @@ class Sampler:
     dev = self._transformer.device
     lead = torch.arange(0, b, g, device=dev)
     c = self._transformer.config
-    need = (c.num_layers, 2, b // g, self.cache_config.cache_size, c.num_kv_heads, c.head_dim)
+    size = self.cache_config.cache_size
+    need = c.cache_shape(b // g, size)
     if getattr(self, '_lead_cache', None) is None or tuple(self._lead_cache.shape) != need:
       self._lead_cache = None
-      self._lead_cache = self._transformer.init_cache(b // g, self.cache_config.cache_size)
+      self._lead_cache = self._transformer.init_cache(b // g, size)
     sub = dict(st)
     sub.update({
         'token_buffer': st['token_buffer'][lead].contiguous(), 'positions': st['positions'][lead].contiguous(),
@@ -351,8 +375,9 @@ class Sampler:
         'logprobs': None, 'logits': None, 'step': torch.zeros(1, dtype=torch.int32, device=dev),
         'cache': self._lead_cache, 'share_group': 1, 'share_len': 0, 'share_common': 0, 'fresh': False})
     self.walk(sub, n)
-    for r in range(g):  # rows r, r + g, ... of the cache <- the leaders' rows (strided copies, no temporary)
-      st['cache'][:, :, r::g, :n].copy_(self._lead_cache[:, :, :, :n])
+    for dst, src in zip(c.cache_rows(st['cache'], b, size), c.cache_rows(self._lead_cache, b // g, size)):
+      for r in range(g):  # rows r, r + g, ... of the cache <- the leaders' rows (strided copies, no temporary)
+        dst[r::g, :n].copy_(src[:, :n])
     st['step'].fill_(n)
 
   def run_steps(self, st, n_steps, sample=True, graph=False, tokens_per_pass=1):
@@ -402,6 +427,7 @@ class Sampler:
     valid = (ids != pad) if token_mask is None else np.asarray(token_mask).astype(bool)
     if valid.shape != ids.shape:
       raise ValueError('token_mask must match the full prompt/completion shape')
+    self._check_positions(int(valid.sum(axis=1).max()))
     self.eos_ids = np.array([-1])
     st = self.init_sample_state(ids, total, False, None, temperature if temperature not in (0.0, 1.0) else 1.0,
                                 1.0, None, 0, include_logprobs=True)
@@ -445,6 +471,7 @@ class Sampler:
     if total > self.cache_config.cache_size:
       raise ValueError(f'Total sampling steps {total} must be less than the cache size'
                        f' {self.cache_config.cache_size}.')
+    self._check_positions(int(prompt_lengths.max()) + max_generation_steps)
     st = self.init_sample_state(
         all_input_ids, total, return_logits, forbidden, temperature, top_p, top_k, seed, beam_size,
         include_logprobs=return_logprobs, prompt_lengths=prompt_lengths if exact_input else None)
@@ -459,7 +486,7 @@ class Sampler:
         self.run_steps(st, n, sample=True, graph=self.use_graph)
         remaining -= n
         if return_logits:
-          logits_steps.append(st['logits'].clone())
+          logits_steps.append(st['logits'][:, :self._transformer.config.vocab_size].clone())
         if remaining > 0 and bool(st['done'].all().item()):
           break
     self.check_device_status(st)
