@@ -38,7 +38,15 @@ LABELS = {'llama3.1-8b-grpo': '8B', 'llama3.2-1b-b1': '1B single-sequence', 'toy
           'qwen3-8b-b128': 'Qwen3-8B 128-sequence', 'qwen3-30b-a3b-moe': 'Qwen3-30B-A3B MoE'}
 
 CLASS_NAMES = ['row_norm', 'qkv_linear', 'rope_kvwrite', 'attention', 'o_linear', 'gate_up_linear',
-               'swiglu', 'down_linear', 'head_sample', 'advance_step', 'empty_launch', 'router']
+               'swiglu', 'down_linear', 'head_sample', 'advance_step', 'empty_launch', 'router', 'latent_q', 'latent_v']
+
+# --latent: layers of the dense latent-attention design at sizes of real models, each beside the quantised model of
+# equal width and feed-forward: (width, ff, heads, dim, rot_dim, vdim, kv_rank, streams, layers, vocab)
+LATENT_SIZES = {
+    '2k': (2048, 8192, 16, 128, 64, 128, 512, 4, 8, 128256),
+    '4k': (4096, 14336, 32, 128, 64, 128, 512, 4, 8, 128256),
+    '4k-r256': (4096, 14336, 32, 64, 32, 64, 256, 2, 8, 128256),
+}
 
 
 def linear_bytes(pl, batch, frac=1.0):
@@ -108,6 +116,159 @@ def cpu_baseline(workload, n_layers=2):
   }
 
 
+class IdTok:  # ids only: the benchmark feeds token ids and never decodes text
+  def encode(self, s): return [int(t) for t in s.split()]
+  def decode(self, ids): return ''
+  def pad_id(self): return 0
+  def bos_id(self): return 1
+  def eos_id(self): return -1
+
+
+def class_work(model, rows, keys, decode):
+  """Per launch class: (algorithmic bytes, flops) of one launch over `rows` rows that see `keys` cache rows on average
+  (decode: every row reads its own sequence's rows; else the rows of a pass share theirs)."""
+  c = model.config
+  out = {}
+  layer = model.layers[0]
+  if hasattr(c, 'layers'):
+    l = c.layers[0]
+    n = c.streams
+    out['row_norm'] = (rows * c.embed_dim * (2 * n * 4 + 4), rows * c.embed_dim * 2 * n * (n + 2))
+    def dense(k, n_out, heads=1):
+      return 2.0 * heads * k * n_out + 2.0 * rows * heads * (k + n_out), 2.0 * rows * heads * k * n_out
+    own = l.heads * (l.dim + l.rot_dim) + l.kv_rank + l.rot_dim + (l.heads * l.vdim if l.gate else 0)
+    width = l.kv_rank + l.rot_dim
+    out['qkv_linear'] = dense(c.embed_dim, own)
+    out['rope_kvwrite'] = (rows * 4.0 * (l.heads * l.rot_dim + width), 0)
+    out['latent_q'] = dense(l.dim, l.kv_rank, l.heads)
+    out['latent_v'] = dense(l.kv_rank, l.vdim, l.heads)
+    out['attention'] = ((rows * keys if decode else keys) * width * 2.0 + rows * l.heads * 2.0 * (width + l.kv_rank),
+                        2.0 * rows * keys * l.heads * (width + l.kv_rank))
+    out['o_linear'] = dense(l.heads * l.vdim, c.embed_dim)
+    g, d = dense(c.embed_dim, 2 * l.ff), dense(l.ff, c.embed_dim)
+    out['gate_up_linear'], out['down_linear'] = (g[0] - 2.0 * rows * l.ff, g[1]), d
+    out['head_sample'] = (2.0 * c.vocab_size * c.embed_dim, 2.0 * rows * c.vocab_size * c.embed_dim)
+    return out
+  def quant(pl):
+    f = 2.0 * rows * pl.k * pl.n + (2.0 * rows * pl.rank * (pl.k * len(pl.seg_cols) + pl.n) if pl.lora_a_t is not None else 0)
+    return float(linear_bytes(pl, rows)), f
+  for name, key in (('qkv_linear', 'qkv'), ('o_linear', 'o'), ('gate_up_linear', 'gate_up'), ('down_linear', 'down')):
+    out[name] = quant(layer[key])
+  out['row_norm'] = (rows * c.embed_dim * 2.0 * 4, 0)
+  out['rope_kvwrite'] = (rows * 4.0 * (c.num_heads + 2 * c.num_kv_heads) * c.head_dim, 0)
+  kv = c.num_kv_heads * c.head_dim * 4.0
+  out['attention'] = ((rows * keys if decode else keys) * kv + rows * 4.0 * c.num_heads * c.head_dim,
+                      4.0 * rows * keys * c.num_heads * c.head_dim)
+  out['head_sample'] = (2.0 * c.vocab_size * c.embed_dim, 2.0 * rows * c.vocab_size * c.embed_dim)
+  return out
+
+
+def latent_bench(size, batches, prompt, steps):
+  """Prefill and decode throughput of the latent-attention design beside the closest quantised model, with the
+  distance of every launch class from its roofline (measured event time over the larger of bytes / 8 TB/s and
+  flops / 2.5 PFLOP/s).  Prints one JSON line."""
+  import torch
+  from tunix_amd import _lib
+  from tunix_amd.configs import CacheConfig
+  from tunix_amd.latent import LatentConfig, LatentModel
+  from tunix_amd.model import ModelConfig, QLoRAModel
+  from tunix_amd.sampler import Sampler
+  d, ff, heads, dim, rot, vdim, rank, streams, layers, vocab = LATENT_SIZES[size]
+  torch.cuda.set_device(0)
+  lib = _lib.lib()
+  rng = np.random.default_rng(0)
+
+  def build(kind):
+    if kind == 'kagapel':
+      return LatentModel.random_init(LatentConfig.uniform(layers, vocab, d, ff, heads, dim, rot, vdim, rank, streams))
+    cfg = ModelConfig('llama3', layers, vocab, d, ff, d // 128, 128, 8, 500_000, 1e-5, False)
+    return QLoRAModel.random_init(cfg, seed=0, group=64, lora_rank=16, lora_alpha=32.0)
+
+  def profiled(s, st, t, n, sample):
+    ms, cnt = np.zeros(len(CLASS_NAMES), np.float32), np.zeros(len(CLASS_NAMES), np.int32)
+    tot, tc = np.zeros_like(ms), np.zeros_like(cnt)
+    for _ in range(n):
+      cs = s._c_state(st, t)
+      _lib.check(lib.tmx_decode_steps_profiled(ctypes.byref(s.transformer.desc()), ctypes.byref(cs), _lib.stream(), 1, sample,
+                                               ms.ctypes.data_as(ctypes.c_void_p), cnt.ctypes.data_as(ctypes.c_void_p)),
+                 'tmx_decode_steps_profiled')
+      tot += ms
+      tc += cnt
+    return {k: (float(tot[i] / tc[i]) * 1e-3, int(tc[i]) // n) for i, k in enumerate(CLASS_NAMES) if tc[i]}
+
+  def distances(times, work):
+    out = {}
+    for k, (sec, n) in times.items():
+      if k not in work:
+        continue
+      byts, flops = work[k]
+      bound = max(byts / 8e12, flops / 2.5e15)
+      out[k] = {'us': round(sec * 1e6, 2), 'launches': n, 'bound': 'mfma' if flops / 2.5e15 > byts / 8e12 else 'hbm',
+                'frac': round(bound / sec, 4)}
+    return out
+
+  result = {'metric': f'prefill and decode tokens/s, latent-attention design, {size} layers', 'unit': 'tokens/s',
+            'n_gpus': 1, 'higher_is_better': True, 'data': 'synthetic (random-init weights, uniform-random token ids)',
+            'config': {'width': d, 'ff': ff, 'heads': heads, 'dim': dim, 'rot_dim': rot, 'vdim': vdim, 'kv_rank': rank,
+                       'streams': streams, 'layers': layers, 'vocab': vocab, 'prompt': prompt, 'decode_steps': steps}}
+  for kind in ('kagapel', 'llama3-int4'):
+    model = build(kind)
+    c = model.config
+    total = prompt + steps + 40
+    s = Sampler(model, IdTok(), CacheConfig(total, c.num_layers, c.num_kv_heads, c.head_dim))
+    s.eos_ids = np.array([-1])
+    s.share_prompt_kv = False
+    wbytes, hbytes = model.weight_bytes()
+    rec = {'weight_bytes_per_layer': wbytes // layers}
+    for b in batches:
+      ids = rng.integers(3, vocab, (b, prompt)).astype(np.int32)
+      def fresh():
+        return s.init_sample_state(ids, total, False, None, 0.0, None, None, 0, prompt_lengths=np.full(b, prompt))
+      def timed(fn):
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        fn()
+        torch.cuda.synchronize()
+        return time.perf_counter() - t0
+      st = fresh()
+      s.walk(st, prompt - 1)
+      st = fresh()
+      fill = timed(lambda: s.walk(st, prompt - 1))
+      s.run_steps(st, 8)
+      dec = timed(lambda: s.run_steps(st, steps))
+      s.check_device_status(st)
+      r = {'prefill_tokens_per_s': round(b * (prompt - 1) / fill), 'prefill_ms': round(fill * 1e3, 3),
+           'decode_tokens_per_s': round(b * steps / dec), 'decode_ms_per_step': round(dec / steps * 1e3, 4)}
+      ctx = int(st['step'].item()) + 4
+      r['decode_kernels'] = distances(profiled(s, st, 1, 8, 1), class_work(model, b, ctx, True))
+      # one pass of the prompt walk, its tokens in the middle of the prompt
+      per = min(128, max(1, s._fill_rows() // b), prompt // 2)
+      st = fresh()
+      s.walk(st, prompt // 2)
+      work = class_work(model, b * per, prompt // 2 + per / 2.0, False)
+      by, fl = work['attention']
+      kb = (prompt // 2 + per) * (c.cache_bytes_per_token() / c.num_layers if hasattr(c, 'layers') else c.num_kv_heads * c.head_dim * 4.0)
+      work['attention'] = (b * kb, fl)
+      r['prefill_kernels'] = distances(profiled(s, st, per, 1, 0), work)
+      r['prefill_rows_per_pass'] = b * per
+      rec[f'batch_{b}'] = r
+    result[kind] = rec
+    del model, s, st
+    torch.cuda.empty_cache()
+  result['value'] = result['kagapel'][f'batch_{batches[-1]}']['decode_tokens_per_s']
+  # how much farther from its roofline a launch class of the design is than the like class of the closest model
+  rel = {}
+  for b in batches:
+    for phase in ('decode_kernels', 'prefill_kernels'):
+      new, old = (result[k][f'batch_{b}'][phase] for k in ('kagapel', 'llama3-int4'))
+      for k, v in new.items():
+        like = {'latent_q': 'o_linear', 'latent_v': 'o_linear'}.get(k, k)
+        if like in old:
+          rel.setdefault(k, {})[f'{phase[:7].rstrip("_")}_{b}'] = round(old[like]['frac'] / v['frac'], 2)
+  result['distance_ratio'] = rel
+  print(json.dumps(result))
+
+
 def pmc_summary(path, counter, match=None, top=16):
   """Prints, for every kernel symbol of a rocprofv3 counter-collection CSV, the number of
   dispatches and the mean / max of `counter` over them (template arguments kept, argument
@@ -149,7 +310,14 @@ def main():
                        'cannot hold tens of thousands of pending dispatches)')
   ap.add_argument('--pmc-calibrate', action='store_true',
                   help='also run one 1 GiB device copy (a kernel of known traffic) to scale PMC counters')
+  ap.add_argument('--latent', choices=sorted(LATENT_SIZES), default=None,
+                  help='prefill and decode throughput of the latent-attention design at this size beside the closest '
+                       'quantised model: a separate JSON line, not the headline metric')
+  ap.add_argument('--latent-batches', type=int, nargs='+', default=[1, 16, 64])
   args = ap.parse_args()
+  if args.latent:
+    latent_bench(args.latent, args.latent_batches, 512, min(args.steps, 64))
+    return
   if args.pmc_summary:
     pmc_summary(args.pmc_summary[0], args.pmc_summary[1], args.match)
     return
@@ -179,14 +347,7 @@ def main():
                                  lora_targets=targets)
   cache_size = prompt + new
 
-  class _Tok:  # ids only: the benchmark feeds token ids and never decodes text
-    def encode(self, s): return [int(t) for t in s.split()]
-    def decode(self, ids): return ''
-    def pad_id(self): return 0
-    def bos_id(self): return 1
-    def eos_id(self): return -1
-
-  sampler = Sampler(model, _Tok(), CacheConfig(cache_size, cfg.num_layers, cfg.num_kv_heads, cfg.head_dim))
+  sampler = Sampler(model, IdTok(), CacheConfig(cache_size, cfg.num_layers, cfg.num_kv_heads, cfg.head_dim))
   sampler.eos_ids = np.array([-1])  # unreachable: every row runs the full length
   sampler.share_prompt_kv = not args.no_kv_sharing
   rng = np.random.default_rng(0)

@@ -14,7 +14,8 @@ import sys
 sys.path.insert(0, os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 
 from tunix_amd import _lib
-from tunix_amd.model import DecodeState, LayerDesc, ModelDesc, QLinearDesc
+from tunix_amd.model import (DecodeState, DenseDesc, FAMILY_LATENT, LatentLayerDesc, LayerDesc, ModelDesc, QLinearDesc,
+                             StreamsDesc)
 
 FAKE = 0x1000  # a non-null "device pointer": never dereferenced on the host
 
@@ -59,6 +60,62 @@ def model_desc(family, layers, vocab, dm, f, n, kh, h, experts, per_tok, group, 
   return d, arr
 
 
+def latent_desc(act, layers, vocab, d, ff, heads, dim_p, rot, rank, rank_p, vdim_p, streams):
+  """A TMX_FAMILY_LATENT model: every other layer reads the latents of the one before it."""
+  arr = (LatentLayerDesc * layers)()
+  dp, rot_p = (d + 63) // 64 * 64, 64
+  up32 = lambda v: (v + 31) // 32 * 32
+  hc = StreamsDesc(FAKE, FAKE, FAKE)
+  for i in range(layers):
+    a = arr[i]
+    a.norm1_w = a.norm2_w = a.table = FAKE
+    a.hc1 = a.hc2 = hc
+    a.heads, a.rot_dim, a.kv_rank, a.dim_p, a.rot_p, a.rank_p, a.vdim_p = heads, rot, rank, dim_p, rot_p, rank_p, vdim_p
+    a.scale = 0.1
+    a.off_qr = heads * dim_p
+    n = a.off_qr + up32(heads * rot)
+    a.off_kv = a.off_gate = -1
+    a.kv_layer = i - i % 2
+    if i % 2 == 0:
+      a.off_kv, a.kv_norm_w = n, FAKE
+      n += up32(rank + rot)
+    else:
+      a.off_gate = n
+      n += heads * vdim_p
+    a.in_ = DenseDesc(FAKE, None, dp, n, 1)
+    a.uk, a.uv = DenseDesc(FAKE, None, dim_p, rank_p, heads), DenseDesc(FAKE, None, rank_p, vdim_p, heads)
+    a.o = DenseDesc(FAKE, None, heads * vdim_p, dp, 1)
+    if i != 1:
+      a.gate_up, a.down = DenseDesc(FAKE, FAKE, dp, 2 * ff, 1), DenseDesc(FAKE, FAKE, ff, dp, 1)
+  m = ModelDesc()
+  m.family, m.num_layers, m.vocab_size, m.embed_dim, m.norm_eps = FAMILY_LATENT, layers, vocab, d, 1e-5
+  m.embed = m.pos_embed = m.final_norm_w = m.head = m.final_in = FAKE
+  m.latent_layers = ctypes.cast(arr, ctypes.POINTER(LatentLayerDesc))
+  m.act, m.streams, m.max_positions, m.logit_scale = act, streams, 64, 1.0
+  return m, arr
+
+
+def latent_plans(lib):
+  for shape in ((4, 1000, 200, 320, 5, 64, 10, 100, 128, 64, 3), (3, 128256, 4096, 14336, 32, 128, 64, 512, 512, 128, 4)):
+    for act in (0, 1):
+      m, arr = latent_desc(act, *shape)
+      for batch in (1, 32, 129, 4096):
+        nb = lib.tmx_decode_workspace_bytes(ctypes.byref(m), batch, 640)
+        assert nb > 256, (shape, act, batch)
+        st = DecodeState()
+        st.batch, st.buf_len, st.cache_size = batch, 640, 640
+        st.token_buffer = st.positions = st.input_mask = st.done = st.step = st.kv_cache = st.workspace = FAKE
+        st.workspace_bytes = nb - 1
+        assert lib.tmx_decode_steps(ctypes.byref(m), ctypes.byref(st), None, 1, 1) == -2
+      arr[1].kv_layer = 1  # no latents of its own and no earlier layer to take them from
+      assert lib.tmx_decode_workspace_bytes(ctypes.byref(m), 1, 640) == 0
+      assert lib.tmx_decode_steps(ctypes.byref(m), ctypes.byref(st), None, 1, 1) == -1
+  for n_seq in (1, 64, 4096):
+    for t in (1, 7, 128):
+      for h in (1, 32, 128):
+        lib.tmx_latent_attention_workspace_bytes(n_seq, t, h, 512, 4096)
+
+
 def main():
   lib = _lib.lib()
   assert os.path.basename(_lib.LIB_PATH) == 'libtmx_hostsan.so', _lib.LIB_PATH
@@ -97,6 +154,7 @@ def main():
       lib.tmx_gqa_decode_workspace_bytes(b, n, kh, h, 1536)
       lib.tmx_head_sample_workspace_bytes(b, c[2])
       lib.tmx_nucleus_workspace_bytes(b, c[2])
+  latent_plans(lib)
   assert lib.tmx_int4_dequant(None, None, None, None, 64, 32, 64) == -1
   assert lib.tmx_int4_dequant(None, FAKE, FAKE, FAKE, 65, 32, 64) == -2
   assert lib.tmx_qlora_linear_planes(None, FAKE, FAKE, FAKE, None, FAKE, None, 4, 100, 32, 64, 0, 1) == -2

@@ -16,6 +16,10 @@ HIPCC_FLAGS = [
     '-Xclang', '-target-feature', '-Xclang', '-packed-fp32-ops',
 ]
 
+# per source: the walk over latent cache rows keeps its accumulators in ordinary registers (in accumulation registers
+# they would be copied out and back around every rescaling)
+EXTRA_FLAGS = {'latent.hip': ['-mllvm', '-amdgpu-mfma-vgpr-form=1']}
+
 
 def sources():
   return sorted(os.path.join(CSRC, f) for f in os.listdir(CSRC) if f.endswith('.hip'))
@@ -48,7 +52,7 @@ def build(verbose=False, jobs=6, host_sanitizers=False):
   srcs = sources()
   objs = [os.path.join(obj_dir, os.path.basename(s)[:-4] + '.o') for s in srcs]
   with concurrent.futures.ThreadPoolExecutor(max_workers=jobs) as ex:
-    outs = list(ex.map(lambda so: _run([hipcc] + HIPCC_FLAGS + extra + inc + ['-c', so[0], '-o', so[1]]),
+    outs = list(ex.map(lambda so: _run([hipcc] + HIPCC_FLAGS + EXTRA_FLAGS.get(os.path.basename(so[0]), []) + extra + inc + ['-c', so[0], '-o', so[1]]),
                        zip(srcs, objs)))
   part = lib_path + '.part'
   link = [hipcc, '--offload-arch=gfx950', '-shared', '-fPIC', '-o', part]

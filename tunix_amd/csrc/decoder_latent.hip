@@ -13,8 +13,8 @@ LatentWorkspace latent_carve(const tmx_model_desc* m, int rows, char* base) {
   LatentWorkspace w = {};
   size_t off = 0;
   auto take = [&](size_t bytes) { char* p = (base && bytes) ? base + off : nullptr; off += align256(bytes); return p; };
-  const size_t B = rows, Dp = pad_to(m->embed_dim, 64), e = act_bytes(m);
-  size_t z = 0, q = 0, lat = 0, val = 0, act = 0, part = 0;
+  const size_t B = rows, Bt = pad_to(rows, 32), Dp = pad_to(m->embed_dim, 64), e = act_bytes(m);
+  size_t z = 0, q = 0, lat = 0, val = 0, act = 0, part = 0, splits = 1;
   auto up = [](size_t& d, size_t v) { if (v > d) d = v; };
   for (int i = 0; i < m->num_layers; ++i) {
     const tmx_latent_layer_desc& l = m->latent_layers[i];
@@ -22,19 +22,24 @@ LatentWorkspace latent_carve(const tmx_model_desc* m, int rows, char* base) {
     up(q, (size_t)l.heads * (l.rank_p + l.rot_p));
     up(lat, (size_t)l.heads * l.rank_p);
     up(val, (size_t)l.heads * l.vdim_p);
-    if (l.gate_up.w) up(act, l.gate_up.N / 2);
+    up(splits, dense_num_splits(m->act, rows, l.o.K, l.o.N));
+    if (l.gate_up.w) {
+      up(act, l.gate_up.N / 2);
+      up(splits, dense_num_splits(m->act, rows, l.down.K, l.down.N));
+    }
     if (m->act == TMX_ACT_BF16) up(part, latent_attn_partial_bytes(rows, l.heads, l.rank_p));
   }
   take(256);  // status block
   w.xs = (float*)take(B * m->streams * Dp * 4);
-  w.xn = take(B * Dp * e);
+  w.xn = take(Bt * Dp * e);
   w.z = take(B * z * e);
   w.q = take(B * q * e);
   w.lat = take(B * lat * e);
-  w.val = take(B * val * e);
+  w.val = take(Bt * val * e);
   w.y = take(B * Dp * e);
-  w.act = take(B * act * e);
+  w.act = take(Bt * act * e);
   w.attn_partial = (float*)take(part);
+  w.y_part = (float*)take(splits > 1 ? splits * B * Dp * 4 : 0);
   const size_t Vp = pad_to(m->vocab_size, 32);
   w.logits = (float*)take(m->act == TMX_ACT_F32 ? B * Vp * 4 : 0);
   w.head_partial = take(head_partial_bytes(rows, (int)Vp));
@@ -86,23 +91,36 @@ int latent_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_stat
   const int M = n_seq * T, C = s->cache_size, L = s->buf_len, Dp = pad_to(m->embed_dim, 64), act = m->act;
   const size_t e = act_bytes(m);
   int rc;
-  auto dense = [&](const tmx_dense_desc& d, const void* x, int ldx, int x_head, void* y, int ldy, int y_head, int epi,
-                   const void* gate, int ldg) {
+  // up to 128 bf16 rows: the inputs of the plain projections travel in the order the matrix pipe reads them
+  const bool tiled = act == TMX_ACT_BF16 && M <= 128;
+  auto args = [&](const tmx_dense_desc& d, const void* x, int ldx, int x_head, void* y, int ldy, int y_head, int epi) {
     DenseArgs a = {};
     a.x = x; a.ldx = ldx; a.x_head = x_head;
-    a.w = d.w; a.bias = d.bias; a.gate = gate; a.ldg = ldg;
+    a.w = d.w; a.bias = d.bias;
     a.y = y; a.ldy = ldy; a.y_head = y_head;
     a.M = M; a.K = d.K; a.N = d.N; a.heads = d.heads; a.epi = epi;
+    return a;
+  };
+  // a sublayer's last projection, whose result the next stream row kernel adds: w.y, or planes in w.y_part
+  int y_splits = 1;
+  auto into_streams = [&](const tmx_dense_desc& d, const void* x) {
+    DenseArgs a = args(d, x, d.K, 0, w.y, Dp, 0, TMX_DENSE_PLAIN);
+    a.x_tiled = tiled;
+    a.nsplit = y_splits = dense_num_splits(act, M, d.K, d.N);
+    a.y_part = w.y_part;
     return dense_linear(st, act, a);
   };
   // The boundary behind sublayer `prev` (null: the embedding) and in front of the next one.
   const tmx_streams_desc* prev = nullptr;
-  auto boundary = [&](const float* in, const float* norm_w, bool store) {
+  auto boundary = [&](const float* in, const float* norm_w, bool head) {
     StreamArgs a = {};
     a.xs = w.xs; a.in = in; a.norm_w = norm_w; a.xn = w.xn;
-    a.S = m->streams; a.D = m->embed_dim; a.Dp = Dp; a.eps = m->norm_eps; a.store = store;
+    a.S = m->streams; a.D = m->embed_dim; a.Dp = Dp; a.eps = m->norm_eps; a.store = !head;
+    a.xn_tiled = tiled && !head;
     if (prev) {
-      a.y = w.y; a.mix = prev->mix; a.out = prev->out;
+      if (y_splits > 1) { a.y_part = w.y_part; a.nsplit = y_splits; }
+      else a.y = w.y;
+      a.mix = prev->mix; a.out = prev->out;
     } else {
       a.embed = (const uint16_t*)m->embed; a.pos_embed = (const uint16_t*)m->pos_embed;
       a.vocab = m->vocab_size; a.max_positions = m->max_positions;
@@ -126,8 +144,12 @@ int latent_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_stat
   for (int i = 0; i < m->num_layers; ++i) {
     const tmx_latent_layer_desc& l = m->latent_layers[i];
     const int ld = l.rank_p + l.rot_p, H = l.heads;
-    TMX_TRY(TMX_K_ROWNORM, boundary(l.hc1.in, l.norm1_w, true));
-    TMX_TRY(TMX_K_QKV, dense(l.in, w.xn, Dp, 0, w.z, l.in.N, 0, TMX_DENSE_PLAIN, nullptr, 0));
+    TMX_TRY(TMX_K_ROWNORM, boundary(l.hc1.in, l.norm1_w, false));
+    {
+      DenseArgs a = args(l.in, w.xn, Dp, 0, w.z, l.in.N, 0, TMX_DENSE_PLAIN);
+      a.x_tiled = tiled;
+      TMX_TRY(TMX_K_QKV, dense_linear(st, act, a));
+    }
     {
       LatentRowsArgs a = {};
       a.z = w.z; a.ldz = l.in.N; a.off_qr = l.off_qr; a.off_kv = l.off_kv;
@@ -138,7 +160,7 @@ int latent_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_stat
       a.H = H; a.rot = l.rot_dim; a.rank = l.kv_rank; a.rank_p = l.rank_p; a.rot_p = l.rot_p; a.C = C;
       TMX_TRY(TMX_K_ROPE, latent_rows(st, act, a, M));
     }
-    TMX_TRY(TMX_K_LATENT_Q, dense(l.uk, w.z, l.in.N, l.dim_p, w.q, H * ld, ld, TMX_DENSE_PLAIN, nullptr, 0));
+    TMX_TRY(TMX_K_LATENT_Q, dense_linear(st, act, args(l.uk, w.z, l.in.N, l.dim_p, w.q, H * ld, ld, TMX_DENSE_PLAIN)));
     {
       LatentAttnArgs a = {};
       a.q = w.q; a.cache = cache[i]; a.sink = l.sink;
@@ -147,21 +169,30 @@ int latent_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_stat
       a.n_seq = n_seq; a.tpp = T; a.H = H; a.rank_p = l.rank_p; a.rot_p = l.rot_p; a.C = C; a.scale = l.scale;
       TMX_TRY(TMX_K_ATTN, latent_attention(st, act, a));
     }
-    const char* gate = l.off_gate >= 0 ? (const char*)w.z + (size_t)l.off_gate * e : nullptr;
-    TMX_TRY(TMX_K_LATENT_V, dense(l.uv, w.lat, H * l.rank_p, l.rank_p, w.val, H * l.vdim_p, l.vdim_p,
-                                  gate ? TMX_DENSE_GATED : TMX_DENSE_PLAIN, gate, l.in.N));
-    TMX_TRY(TMX_K_O, dense(l.o, w.val, H * l.vdim_p, 0, w.y, Dp, 0, TMX_DENSE_PLAIN, nullptr, 0));
+    {
+      DenseArgs a = args(l.uv, w.lat, H * l.rank_p, l.rank_p, w.val, H * l.vdim_p, l.vdim_p, TMX_DENSE_PLAIN);
+      if (l.off_gate >= 0) {
+        a.epi = TMX_DENSE_GATED;
+        a.gate = (const char*)w.z + (size_t)l.off_gate * e;
+        a.ldg = l.in.N;
+      }
+      a.y_tiled = tiled;
+      TMX_TRY(TMX_K_LATENT_V, dense_linear(st, act, a));
+    }
+    TMX_TRY(TMX_K_O, into_streams(l.o, w.val));
     prev = &l.hc1;
     if (l.gate_up.w) {
       const int Fp = l.gate_up.N / 2;
-      TMX_TRY(TMX_K_ROWNORM, boundary(l.hc2.in, l.norm2_w, true));
-      TMX_TRY(TMX_K_GATE_UP, dense(l.gate_up, w.xn, Dp, 0, w.act, Fp, 0, TMX_DENSE_SWIGLU, nullptr, 0));
-      TMX_TRY(TMX_K_DOWN, dense(l.down, w.act, Fp, 0, w.y, Dp, 0, TMX_DENSE_PLAIN, nullptr, 0));
+      TMX_TRY(TMX_K_ROWNORM, boundary(l.hc2.in, l.norm2_w, false));
+      DenseArgs a = args(l.gate_up, w.xn, Dp, 0, w.act, Fp, 0, TMX_DENSE_SWIGLU);
+      a.x_tiled = a.y_tiled = tiled;
+      TMX_TRY(TMX_K_GATE_UP, dense_linear(st, act, a));
+      TMX_TRY(TMX_K_DOWN, into_streams(l.down, w.act));
       prev = &l.hc2;
     }
     if (prof) TMX_TRY(TMX_K_EMPTY, empty_launch(st));
   }
-  if (final_norm) TMX_TRY(TMX_K_ROWNORM, boundary(m->final_in, (const float*)m->final_norm_w, false));
+  if (final_norm) TMX_TRY(TMX_K_ROWNORM, boundary(m->final_in, (const float*)m->final_norm_w, true));
   return TMX_OK;
 }
 

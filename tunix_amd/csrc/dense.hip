@@ -17,7 +17,8 @@ __device__ __forceinline__ float sigmoid(float z) { return 1.f / (1.f + expf(-z)
 
 // MT: 32-row tiles of x; WK: waves that share K (8 / WK column tiles per workgroup); NT = 2: SwiGLU pairs (a gate
 // tile and the up tile N / 64 tiles further).
-template <int MT, int WK, int NT>
+// XT: x is tiled (act_tile_off): a wave's load is 1 KiB of consecutive bytes instead of 16-byte pieces of 32 rows.
+template <int MT, int WK, int NT, bool XT>
 __global__ __launch_bounds__(512, 2) void dense_small_kernel(DenseArgs a) {
   constexpr int WN = 8 / WK;
   __shared__ float red[WK > 1 ? 2 : 1][WK > 1 ? 8 * 1024 : 1];
@@ -25,7 +26,9 @@ __global__ __launch_bounds__(512, 2) void dense_small_kernel(DenseArgs a) {
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int h = lane >> 5, nl = lane & 31;
   const int wn = wave / WK, wk = wave % WK;
-  const int KT = a.K >> 6, klast = KT - 1;
+  const int KT = a.K >> 6;
+  const int kts = (KT + a.nsplit - 1) / a.nsplit, slice = blockIdx.z;
+  const int k_beg = slice * kts, k_end = k_beg + kts < KT ? k_beg + kts : KT, klast = k_end - 1;
   const int pair = a.N >> 6;  // tiles from a gate tile to its up tile
   const int tiles = NT == 2 ? pair : a.N >> 5;
   const int tile = blockIdx.x * WN + wn;
@@ -38,8 +41,14 @@ __global__ __launch_bounds__(512, 2) void dense_small_kernel(DenseArgs a) {
   const uint16_t* xsrc[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
-    const int row = m * 32 + nl < a.M ? m * 32 + nl : a.M - 1;
-    xsrc[m] = reinterpret_cast<const uint16_t*>(a.x) + (size_t)row * a.ldx + head * a.x_head + h * 32;
+    if (XT) {
+      // (row tiles past the last one repeat it)
+      const int mt = m * 32 < a.M ? m : (a.M - 1) >> 5;
+      xsrc[m] = reinterpret_cast<const uint16_t*>(a.x) + (size_t)mt * KT * 2048 + lane * 8;
+    } else {
+      const int row = m * 32 + nl < a.M ? m * 32 + nl : a.M - 1;
+      xsrc[m] = reinterpret_cast<const uint16_t*>(a.x) + (size_t)row * a.ldx + head * a.x_head + h * 32;
+    }
   }
   f32x16_t acc[NT][MT];
 #pragma unroll
@@ -61,7 +70,8 @@ __global__ __launch_bounds__(512, 2) void dense_small_kernel(DenseArgs a) {
 #pragma unroll
     for (int m = 0; m < MT; ++m)
 #pragma unroll
-      for (int t = 0; t < 4; ++t) xr[p][m][t] = *reinterpret_cast<const u32x4_t*>(xsrc[m] + (size_t)kt * 64 + t * 8);
+      for (int t = 0; t < 4; ++t)
+        xr[p][m][t] = *reinterpret_cast<const u32x4_t*>(xsrc[m] + (XT ? (size_t)kt * 2048 + t * 512 : (size_t)kt * 64 + t * 8));
   };
   auto use = [&](auto pc) __attribute__((always_inline)) {
     constexpr int p = decltype(pc)::value;
@@ -74,26 +84,31 @@ __global__ __launch_bounds__(512, 2) void dense_small_kernel(DenseArgs a) {
           acc[n][m] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, xr[p][m][t]),
                                                               __builtin_bit_cast(bf16x8_t, wr[p][n][t]), acc[n][m], 0, 0, 0);
   };
-  static_for<P>([&](auto pc) __attribute__((always_inline)) { load(wk + decltype(pc)::value * WK, pc); });
-  for (int kt = wk; kt < KT; kt += P * WK)
+  static_for<P>([&](auto pc) __attribute__((always_inline)) { load(k_beg + wk + decltype(pc)::value * WK, pc); });
+  for (int kt = k_beg + wk; kt < k_end; kt += P * WK)
     static_for<P>([&](auto pc) __attribute__((always_inline)) {
       const int k = kt + decltype(pc)::value * WK;
-      if (k < KT) {
+      if (k < k_end) {
         use(pc);
         load(k + P * WK, pc);
       }
     });
 
-  const float b0 = a.bias ? a.bias[tl * 32 + nl] : 0.f;
+  const float b0 = a.bias && slice == 0 ? a.bias[tl * 32 + nl] : 0.f;
   const float b1 = (NT == 2 && a.bias) ? a.bias[(tl + pair) * 32 + nl] : 0.f;
   auto finish = [&](int m, int r, const float* s) __attribute__((always_inline)) {
     const int row = m * 32 + acc_row(r, lane), col = tile * 32 + nl;
     if (row >= a.M || tile >= tiles) return;
     float v = s[0] + b0;
+    if (NT == 1 && a.nsplit > 1) {
+      a.y_part[((size_t)slice * a.M + row) * a.N + col] = v;
+      return;
+    }
     if (NT == 2) v = silu(v) * (s[NT - 1] + b1);
     if (a.epi == TMX_DENSE_GATED)
       v *= sigmoid(bf2f(reinterpret_cast<const uint16_t*>(a.gate)[(size_t)row * a.ldg + head * a.y_head + col]));
-    reinterpret_cast<uint16_t*>(a.y)[(size_t)row * a.ldy + head * a.y_head + col] = f2bf(v);
+    const int yc = head * a.y_head + col;
+    reinterpret_cast<uint16_t*>(a.y)[a.y_tiled ? act_tile_off(row, yc, a.ldy) : (size_t)row * a.ldy + yc] = f2bf(v);
   };
   if constexpr (WK == 1) {
     static_for<MT>([&](auto mc) __attribute__((always_inline)) {
@@ -144,6 +159,7 @@ struct DenseWide {
 
 template <int MT, int TS>
 __global__ __launch_bounds__(512, 1) void dense_wide_kernel(DenseArgs a, int row_blocks, int col_blocks) {
+  // (nsplit > 1: blockIdx.z is the slice of K, of KT / nsplit k-tiles)
   extern __shared__ __align__(16) unsigned char dw_smem[];
   constexpr int kSlab = MT * TS * 4096, kPieces = MT * TS * 4 / 8;  // 1 KiB pieces per wave and step
   const int tid = threadIdx.x, lane = tid & 63;
@@ -155,7 +171,7 @@ __global__ __launch_bounds__(512, 1) void dense_wide_kernel(DenseArgs a, int row
   const bool swiglu = a.epi == TMX_DENSE_SWIGLU;
   const int KT = a.K >> 6, ntiles = a.N >> 5, pair = a.N >> 6;
   const int row = rb * 256 + wave * 32 + nl, row_l = row < a.M ? row : a.M - 1;
-  const int nsteps = KT / TS, last_step = nsteps - 1;
+  const int slice = blockIdx.z, nsteps = KT / TS / a.nsplit, first = slice * nsteps, last_step = first + nsteps - 1;
   // column tile of fragment m: MT consecutive ones, or MT / 2 gate tiles and their up tiles
   const int tile0 = swiglu ? cb * (MT / 2) : cb * MT;
   const int live_end = swiglu ? pair : ntiles;
@@ -222,11 +238,11 @@ __global__ __launch_bounds__(512, 1) void dense_wide_kernel(DenseArgs a, int row
     });
   };
 
-  dma_w(0, 0);
-  static_for<4 * TS>([&](auto gc) __attribute__((always_inline)) { load_b(0, gc); });
+  dma_w(first, 0);
+  static_for<4 * TS>([&](auto gc) __attribute__((always_inline)) { load_b(first, gc); });
   wait_slab();
-  for (int step = 0; step < nsteps; ++step) {
-    const int buf = step & 1;
+  for (int step = first; step <= last_step; ++step) {
+    const int buf = (step - first) & 1;
     dma_w(step + 1, buf ^ 1);
     __builtin_amdgcn_sched_barrier(0);
     step_math(step, buf);
@@ -264,7 +280,11 @@ __global__ __launch_bounds__(512, 1) void dense_wide_kernel(DenseArgs a, int row
     if (t >= ntiles) return;
     float v[4];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] = acc[m][4 * q + e] + (a.bias ? a.bias[col + e] : 0.f);
+    for (int e = 0; e < 4; ++e) v[e] = acc[m][4 * q + e] + (a.bias && slice == 0 ? a.bias[col + e] : 0.f);
+    if (a.nsplit > 1) {
+      *reinterpret_cast<f32x4_t*>(a.y_part + ((size_t)slice * a.M + row) * a.N + col) = f32x4_t{v[0], v[1], v[2], v[3]};
+      return;
+    }
     if (grow) {
       const uint2 g = *reinterpret_cast<const uint2*>(grow + col);
       v[0] *= sigmoid(bf_lo(g.x)); v[1] *= sigmoid(bf_hi(g.x));
@@ -331,19 +351,40 @@ __global__ __launch_bounds__(256) void dense_f32_kernel(DenseArgs a) {
 }
 
 // ---------------------------------------------------------------------------
-template <int MT, int WK, int NT>
+template <int MT, int WK, int NT, bool XT>
 static int launch_small(hipStream_t st, const DenseArgs& a) {
   const int tiles = NT == 2 ? a.N / 64 : a.N / 32, wn = 8 / WK;
-  hipLaunchKernelGGL((dense_small_kernel<MT, WK, NT>), dim3((tiles + wn - 1) / wn, a.heads), dim3(512), 0, st, a);
+  hipLaunchKernelGGL((dense_small_kernel<MT, WK, NT, XT>), dim3((tiles + wn - 1) / wn, a.heads, a.nsplit), dim3(512), 0, st, a);
   return check_launch();
 }
-template <int MT, int NT>
+template <int MT, int NT, bool XT>
 static int launch_small_k(hipStream_t st, const DenseArgs& a) {
-  const int KT = a.K >> 6;
-  if (KT >= 5) return launch_small<MT, 8, NT>(st, a);
-  if (KT >= 2) return launch_small<MT, 2, NT>(st, a);
-  return launch_small<MT, 1, NT>(st, a);
+  const int KT = (a.K >> 6) / a.nsplit;
+  if (KT >= 8) return launch_small<MT, 8, NT, XT>(st, a);
+  if (KT >= 4) return launch_small<MT, 4, NT, XT>(st, a);
+  if (KT >= 2) return launch_small<MT, 2, NT, XT>(st, a);
+  return launch_small<MT, 1, NT, XT>(st, a);
 }
+template <int MT, int NT>
+static int launch_small_x(hipStream_t st, const DenseArgs& a) {
+  return a.x_tiled ? launch_small_k<MT, NT, true>(st, a) : launch_small_k<MT, NT, false>(st, a);
+}
+
+int dense_num_splits(int act, int M, int K, int N) {
+  if (act != TMX_ACT_BF16) return 1;
+  const int KT = K >> 6, cus = device_cus();
+  int ns = 1;
+  if (M <= 128) {
+    // two workgroups per CU, at least two k-tiles per wave
+    while (ns < 4 && (N / 32) * ns * 2 <= 2 * cus && KT / (2 * ns) >= 16) ns *= 2;
+    return ns;
+  }
+  // 256 x 256 blocks while they do not fill the CUs
+  const long wgs = (long)((M + 255) / 256) * ((N + 255) / 256);
+  while (ns < 4 && wgs * ns * 2 <= cus && KT % (4 * ns) == 0 && KT / (2 * ns) >= 8) ns *= 2;
+  return ns;
+}
+
 template <int MT, int TS>
 static int launch_wide(hipStream_t st, const DenseArgs& a) {
   static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&dense_wide_kernel<MT, TS>),
@@ -351,15 +392,20 @@ static int launch_wide(hipStream_t st, const DenseArgs& a) {
   if (attr != hipSuccess) return TMX_ERR_LAUNCH;
   const int per = a.epi == TMX_DENSE_SWIGLU ? MT / 2 : MT, tiles = a.epi == TMX_DENSE_SWIGLU ? a.N / 64 : a.N / 32;
   const int rb = (a.M + 255) / 256, cb = (tiles + per - 1) / per;
-  hipLaunchKernelGGL((dense_wide_kernel<MT, TS>), dim3(rb * cb, a.heads), dim3(512), (DenseWide<MT, TS>::LDS), st, a, rb, cb);
+  hipLaunchKernelGGL((dense_wide_kernel<MT, TS>), dim3(rb * cb, a.heads, a.nsplit), dim3(512), (DenseWide<MT, TS>::LDS), st, a, rb, cb);
   return check_launch();
 }
 
-int dense_linear(hipStream_t st, int act, const DenseArgs& a) {
+int dense_linear(hipStream_t st, int act, const DenseArgs& args) {
+  DenseArgs a = args;
+  if (a.nsplit < 1) a.nsplit = 1;
   const bool swiglu = a.epi == TMX_DENSE_SWIGLU;
   if (a.M <= 0 || a.K <= 0 || a.N <= 0 || a.heads <= 0 || a.heads > 65535 || a.K % 64 || a.N % 32) return TMX_ERR_SHAPE;
   if (swiglu && (a.N % 64 || a.heads != 1)) return TMX_ERR_SHAPE;
   if (a.heads != 1 && a.bias) return TMX_ERR_ARG;
+  if (a.nsplit > 1 && (!a.y_part || a.heads != 1 || a.epi != TMX_DENSE_PLAIN || act != TMX_ACT_BF16)) return TMX_ERR_ARG;
+  if ((a.x_tiled || a.y_tiled) && (act != TMX_ACT_BF16 || a.M > 128 || (a.x_tiled && a.heads != 1) || (a.y_tiled && a.ldy % 64)))
+    return TMX_ERR_ARG;
   if (act == TMX_ACT_F32) {
     if (a.ldx % 4 || a.x_head % 4) return TMX_ERR_SHAPE;
     const int cols = swiglu ? a.N / 2 : a.N;
@@ -372,20 +418,21 @@ int dense_linear(hipStream_t st, int act, const DenseArgs& a) {
   if (a.ldx % 8 || a.x_head % 8 || a.ldy % 4 || a.y_head % 4 || a.ldg % 4) return TMX_ERR_SHAPE;
   if (a.M <= 128) {
     if (swiglu) {
-      if (a.M <= 32) return launch_small_k<1, 2>(st, a);
-      if (a.M <= 64) return launch_small_k<2, 2>(st, a);
-      return launch_small_k<4, 2>(st, a);
+      if (a.M <= 32) return launch_small_x<1, 2>(st, a);
+      if (a.M <= 64) return launch_small_x<2, 2>(st, a);
+      return launch_small_x<4, 2>(st, a);
     }
-    if (a.M <= 32) return launch_small_k<1, 1>(st, a);
-    if (a.M <= 64) return launch_small_k<2, 1>(st, a);
-    return launch_small_k<4, 1>(st, a);
+    if (a.M <= 32) return launch_small_x<1, 1>(st, a);
+    if (a.M <= 64) return launch_small_x<2, 1>(st, a);
+    return launch_small_x<4, 1>(st, a);
   }
   // buffer descriptors hold byte offsets of 31 bits
   if ((size_t)a.N * a.K * 2 >= (1u << 31) || (size_t)a.M * a.ldx * 2 >= (1u << 31)) return TMX_ERR_SHAPE;
   const int tiles = swiglu ? a.N / 64 : a.N / 32, per8 = swiglu ? 4 : 8;
-  const long wgs = (long)((a.M + 255) / 256) * ((tiles + per8 - 1) / per8) * a.heads;
+  const long wgs = (long)((a.M + 255) / 256) * ((tiles + per8 - 1) / per8) * a.heads * a.nsplit;
   const bool wide8 = wgs >= device_cus() && tiles > per8 / 2;
-  if ((a.K >> 6) % 2 == 0) return wide8 ? launch_wide<8, 2>(st, a) : launch_wide<4, 2>(st, a);
+  if ((a.K >> 6) % (2 * a.nsplit) == 0) return wide8 ? launch_wide<8, 2>(st, a) : launch_wide<4, 2>(st, a);
+  if ((a.K >> 6) % a.nsplit) return TMX_ERR_SHAPE;
   return wide8 ? launch_wide<8, 1>(st, a) : launch_wide<4, 1>(st, a);
 }
 

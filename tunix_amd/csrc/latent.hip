@@ -113,32 +113,23 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
   const int wg = wave % WPW;  // wave within its position group
   const int seq = blockIdx.y, split = blockIdx.z;
   const int rows = a.tpp * a.H;  // query rows of a sequence
-  const int step0 = max(min(*a.step, min(a.C, a.buf_len) - a.tpp), 0);  // clamped: every slot read lies in the cache
   const int q0 = blockIdx.x * (32 * SH::WQ);
   const int qr = q0 + wq * 32 + qi, qr_l = qr < rows ? qr : rows - 1;
-  const int limit = step0 + qr_l / a.H;  // newest slot this query sees
-  const int q_end = min(q0 + 32 * SH::WQ, rows);
-  const int nblk_all = (step0 + (q_end - 1) / a.H + 32) >> 5;  // blocks up to the newest slot of the workgroup
-  const int bps = (nblk_all + a.nsplit - 1) / a.nsplit;
-  const int b_beg = split * bps, b_end = min(b_beg + bps, nblk_all);
-
   const size_t qrow = (size_t)seq * rows + qr_l;
-  const uint16_t* qp = reinterpret_cast<const uint16_t*>(a.q) + qrow * LD + (LD / 2) * h;
-  u32x4_t qf[KS];
-#pragma unroll
-  for (int t = 0; t < KS; ++t) qf[t] = *reinterpret_cast<const u32x4_t*>(qp + 8 * t);
 
   const __amdgpu_buffer_rsrc_t rc = make_rsrc(reinterpret_cast<const uint16_t*>(a.cache) + (size_t)seq * a.C * LD,
                                               (uint32_t)a.C * LD * 2u);  // rows past the cache read zero
   uint16_t* tiles = reinterpret_cast<uint16_t*>(la_smem) + wp * SH::kBufs * kTile;
-  auto dma = [&](int blk, uint16_t* tile) __attribute__((always_inline)) {
+  // 32 rows of LD columns into a tile, 1 KiB per load, shared by n waves of which this is number i0
+  auto dma = [&](__amdgpu_buffer_rsrc_t src, int row0, uint16_t* tile, int i0, auto nc) __attribute__((always_inline)) {
+    constexpr int n = decltype(nc)::value;
     int ln = lane;
     asm volatile("" : "+v"(ln));  // the offsets are formed at the transfer, not kept in registers over the loop
 #pragma unroll
-    for (int i = 0; i < CPR / 2 / WPW; ++i) {  // 1 KiB per load, the waves of the group share the tile
-      const int ld = wg + WPW * i;
+    for (int i = 0; i < CPR / 2 / n; ++i) {
+      const int ld = i0 + n * i;
       const int g = ld * 64 + ln, row = g / CPR, slot = g - row * CPR;
-      load_row_to_lds(rc, tile + ld * 512, (row * CPR + (slot ^ latent_swz<CPR>(row))) * 16, blk * (32 * LD * 2));
+      load_row_to_lds(src, tile + ld * 512, (row * CPR + (slot ^ latent_swz<CPR>(row))) * 16, row0 * (LD * 2));
     }
   };
   const uint8_t* mrow = a.input_mask + (size_t)seq * a.buf_len;
@@ -154,26 +145,90 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
     for (int r = 0; r < 16; ++r) o[c][r] = 0.f;
   float m = -1e30f, l = 0.f;
 
+  // Blocks are dealt out in turn to the position groups of all splits: the first one does not depend on *step, so its
+  // transfer starts at once.  All groups of a workgroup run the same number of rounds.
+  const int blk0 = split * WP + wp, stride = a.nsplit * WP;
+  auto blk_of = [&](int round) { return blk0 + round * stride; };
+  auto fetch = [&](int round, int buf) __attribute__((always_inline)) {
+    dma(rc, blk_of(round) * 32, tiles + buf * kTile, wg, IC<WPW>{});
+  };
+  // The query fragments come through LDS as well (read from memory they would be 16-byte pieces of 32 rows per load):
+  // the query groups of the workgroup, two at a time, through the tiles that are not in use yet.
+  u32x4_t qf[KS];
+  {
+    constexpr bool early = !SHARED && SH::kBufs == 2;  // the first tile of every position group is in buffer 0
+    const __amdgpu_buffer_rsrc_t rq = make_rsrc(reinterpret_cast<const uint16_t*>(a.q) + (size_t)seq * rows * LD, (uint32_t)rows * LD * 2u);
+    uint16_t* const lds = reinterpret_cast<uint16_t*>(la_smem);
+    if (early) fetch(0, 0);
+    constexpr int kStage = SHARED ? 2 : 1;  // query groups per turn
+#pragma unroll
+    for (int g = 0; g < SH::WQ; g += kStage) {
+#pragma unroll
+      for (int e = 0; e < kStage; ++e) dma(rq, q0 + (g + e) * 32, lds + (early ? 1 : e) * kTile, wave, IC<4>{});
+      __builtin_amdgcn_s_waitcnt(0x0F70);
+      __syncthreads();
+      if (wq >= g && wq < g + kStage) {
+        const uint16_t* qb = lds + (early ? 1 : wq - g) * kTile + qi * LD;
+#pragma unroll
+        for (int t = 0; t < KS; ++t)
+          qf[t] = *reinterpret_cast<const u32x4_t*>(qb + (((KS * h + t) ^ latent_swz<CPR>(qi)) << 3));
+      }
+      __syncthreads();
+    }
+    if (!early && SH::kBufs == 2) fetch(0, 0);
+  }
+  const int step0 = max(min(*a.step, min(a.C, a.buf_len) - a.tpp), 0);  // clamped: every slot read lies in the cache
+  const int limit = step0 + qr_l / a.H;                               // newest slot this query sees
+  const int b_end = (step0 + (min(q0 + 32 * SH::WQ, rows) - 1) / a.H + 32) >> 5;  // blocks up to the workgroup's newest slot
+  const int rounds = b_end > split * WP ? (b_end - split * WP + stride - 1) / stride : 0;
+  uint8_t mb = mask_byte(blk_of(0));
+  // transposed fragments of the output product: lane (column 32 c + qi, h) takes two runs of four consecutive rows
+  // (see gqa_tile_walk)
+  const int k4 = (lane & 15) >> 2, q4 = lane & 3, g2 = (lane >> 4) & 1;
+  const uint32_t lsw = ((2 * g2 + (q4 >> 1)) ^ latent_swz<CPR>(4 * h + k4)) * 16;
+  const uint32_t vbase = ((4 * h + k4) * LD + 4 * (q4 & 1) + wc * KC * 32) * 2;
+  const int kbase = qi * LD;
   auto block = [&](const uint16_t* kt, int blk, uint32_t mbits) __attribute__((always_inline)) {
+    constexpr int R = 4;  // LDS fragments in flight
+    const int sw = latent_swz<CPR>(qi);
+    bf16x8_t kf[R];
+    auto load_k = [&](auto tc) __attribute__((always_inline)) {
+      constexpr int t = decltype(tc)::value;
+      kf[t % R] = *reinterpret_cast<const bf16x8_t*>(kt + kbase + (((KS * h + t) ^ sw) << 3));
+    };
+    // (the reads are spelled in assembly: for the builtin the compiler waits for every direct-to-LDS load in flight,
+    // i.e. for the next tile; the waits below count them instead)
+    const uint32_t vb = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const uint16_t*)kt + vbase;
+    u32x2_t vf[R][2];
+    auto load_v = [&](auto fc) __attribute__((always_inline)) {
+      constexpr int f = decltype(fc)::value, kb2 = f / KC, c = f % KC;
+      static_for<2>([&](auto ac) __attribute__((always_inline)) {
+        constexpr int a2 = decltype(ac)::value, row0 = 16 * kb2 + 8 * a2;
+        const uint32_t ad = vb + (lsw ^ (uint32_t)(((4 * c) ^ latent_swz<CPR>(row0)) * 16));
+        u32x2_t& dst = vf[f % R][a2];
+        asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(dst) : "v"(ad), "i"(row0 * LD * 2));
+      });
+    };
     f32x16_t sacc;
 #pragma unroll
     for (int r = 0; r < 16; ++r) sacc[r] = 0.f;
-    {
-      const uint16_t* kb = kt + qi * LD;
-      const int sw = latent_swz<CPR>(qi);
-#pragma unroll
-      for (int t = 0; t < KS; ++t) {  // lane (position, h) multiplies the half h of its row
-        const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(kb + (((KS * h + t) ^ sw) << 3));
-        sacc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, __builtin_bit_cast(bf16x8_t, qf[t]), sacc, 0, 0, 0);
-      }
-    }
-    float sc[16], mn = m;
+    static_for<R>([&](auto tc) __attribute__((always_inline)) { load_k(tc); });
+    __builtin_amdgcn_sched_barrier(0);
+    static_for<KS>([&](auto tc) __attribute__((always_inline)) {  // lane (position, h) multiplies the half h of its row
+      constexpr int t = decltype(tc)::value;
+      sacc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[t % R], __builtin_bit_cast(bf16x8_t, qf[t]), sacc, 0, 0, 0);
+      if constexpr (t + R < KS) load_k(IC<t + R>{});
+      __builtin_amdgcn_sched_barrier(0);
+    });
+    static_for<R>([&](auto fc) __attribute__((always_inline)) { load_v(fc); });  // they do not wait for the softmax
+    __builtin_amdgcn_sched_barrier(0);
+    float mn = m;
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int pl = acc_row(r, lane);
       const bool ok = blk * 32 + pl <= limit && ((mbits >> pl) & 1u);
-      sc[r] = ok ? sacc[r] * a.scale : -1e30f;
-      mn = fmaxf(mn, sc[r]);
+      sacc[r] = ok ? sacc[r] * a.scale : -1e30f;
+      mn = fmaxf(mn, sacc[r]);
     }
     mn = fmaxf(mn, __shfl_xor(mn, 32, 64));
     // the reference point of the exponentials moves only when a score has left it by more than 8: until then the
@@ -190,62 +245,41 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
     uint32_t pk[8], pl2[8];
 #pragma unroll
     for (int r = 0; r < 16; r += 2) {
-      const float p0 = sc[r] > -1e29f ? __expf(sc[r] - m) : 0.f;
-      const float p1 = sc[r + 1] > -1e29f ? __expf(sc[r + 1] - m) : 0.f;
+      const float p0 = sacc[r] > -1e29f ? __expf(sacc[r] - m) : 0.f;
+      const float p1 = sacc[r + 1] > -1e29f ? __expf(sacc[r + 1] - m) : 0.f;
       pk[r >> 1] = pack_bf2(p0, p1);
       pl2[r >> 1] = pack_bf2(p0 - bf_lo(pk[r >> 1]), p1 - bf_hi(pk[r >> 1]));
       l += p0 + p1;
     }
-    // out^T += rows^T . P^T, 16 positions (accumulator registers 8 kb2 .. 8 kb2 + 7) per MFMA; the transposed
-    // fragment of lane (column 32 c + qi, h) is two runs of four consecutive rows (see gqa_tile_walk)
-    typedef short s16x4_t __attribute__((ext_vector_type(4)));
-    const int k4 = (lane & 15) >> 2, q4 = lane & 3, g2 = (lane >> 4) & 1;
-    const int lsw = (2 * g2 + (q4 >> 1)) ^ latent_swz<CPR>(4 * h + k4);
-    const uint16_t* vb = kt + (4 * h + k4) * LD + 4 * (q4 & 1) + wc * KC * 32;
-#pragma unroll
-    for (int kb2 = 0; kb2 < 2; ++kb2) {
+    // out^T += rows^T . P^T, 16 positions (accumulator registers 8 kb2 .. 8 kb2 + 7) per MFMA
+    static_for<2 * KC>([&](auto fc) __attribute__((always_inline)) {
+      constexpr int f = decltype(fc)::value, kb2 = f / KC, c = f % KC;
       const u32x4_t pf = {pk[4 * kb2], pk[4 * kb2 + 1], pk[4 * kb2 + 2], pk[4 * kb2 + 3]};
       const u32x4_t pg = {pl2[4 * kb2], pl2[4 * kb2 + 1], pl2[4 * kb2 + 2], pl2[4 * kb2 + 3]};
-#pragma unroll
-      for (int c = 0; c < KC; ++c) {
-        s16x4_t run[2];
-#pragma unroll
-        for (int a2 = 0; a2 < 2; ++a2) {
-          const int row0 = 16 * kb2 + 8 * a2;
-          run[a2] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4_t*)(
-              vb + row0 * LD + ((lsw ^ (4 * c) ^ latent_swz<CPR>(row0)) << 3)));
-        }
-        uint32_t vw[4];
-        __builtin_memcpy(&vw[0], &run[0], 8);
-        __builtin_memcpy(&vw[2], &run[1], 8);
-        const u32x4_t vf = {vw[0], vw[1], vw[2], vw[3]};
-        o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, vf),
-                                                       __builtin_bit_cast(bf16x8_t, pf), o[c], 0, 0, 0);
-        o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, vf),
-                                                       __builtin_bit_cast(bf16x8_t, pg), o[c], 0, 0, 0);
-      }
-    }
+      constexpr int kLater = 2 * KC - 1 - f < R - 1 ? 2 * KC - 1 - f : R - 1;  // fragments requested behind this one
+      u32x2_t &v0 = vf[f % R][0], &v1 = vf[f % R][1];
+      asm volatile("s_waitcnt lgkmcnt(%2)" : "+v"(v0), "+v"(v1) : "i"(2 * kLater));
+      const u32x4_t v = {v0.x, v0.y, v1.x, v1.y};
+      o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, v), __builtin_bit_cast(bf16x8_t, pf),
+                                                     o[c], 0, 0, 0);
+      o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, v), __builtin_bit_cast(bf16x8_t, pg),
+                                                     o[c], 0, 0, 0);
+      if constexpr (f + R < 2 * KC) load_v(IC<f + R>{});
+      __builtin_amdgcn_sched_barrier(0);
+    });
   };
 
-  // position group wp takes the blocks b_beg + wp, b_beg + wp + WP, ...; all groups run the same number of rounds
-  const int rounds = b_end > b_beg ? (b_end - b_beg + WP - 1) / WP : 0;
-  auto blk_of = [&](int round) { return b_beg + round * WP + wp; };
-  auto fetch = [&](int round, int buf) __attribute__((always_inline)) {
-    if (round < rounds && blk_of(round) < b_end) dma(blk_of(round), tiles + buf * kTile);
-  };
-  uint8_t mb = mask_byte(blk_of(0));
-  if (SH::kBufs == 2) fetch(0, 0);
   for (int round = 0; round < rounds; ++round) {
     const int buf = SH::kBufs == 2 ? round & 1 : 0;
     if (SH::kBufs == 1) {
       __syncthreads();  // the last round's reads are complete
-      fetch(round, 0);
+      if (blk_of(round) < b_end) fetch(round, 0);
     }
     const uint32_t mbits = (uint32_t)__ballot(mb != 0);
     __builtin_amdgcn_s_waitcnt(0x0F70);  // this round's tile has landed
     __syncthreads();
     mb = mask_byte(blk_of(round + 1));
-    if (SH::kBufs == 2) fetch(round + 1, buf ^ 1);
+    if (SH::kBufs == 2 && blk_of(round + 1) < b_end) fetch(round + 1, buf ^ 1);
     if (blk_of(round) < b_end) block(tiles + buf * kTile, blk_of(round), mbits);
   }
   l += __shfl_xor(l, 32, 64);

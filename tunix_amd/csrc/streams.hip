@@ -29,6 +29,7 @@ __global__ __launch_bounds__(NTH) void stream_rows_kernel(StreamArgs a) {
   const int m = blockIdx.x;
   float* xs = a.xs + (size_t)m * S * a.Dp;
   const T* y = a.y ? reinterpret_cast<const T*>(a.y) + (size_t)m * a.Dp : nullptr;
+  const bool upd = y || a.y_part;
   const uint16_t *er = nullptr, *pr = nullptr;
   if (a.embed) {
     const int tpp = a.tpp > 0 ? a.tpp : 1;
@@ -44,9 +45,9 @@ __global__ __launch_bounds__(NTH) void stream_rows_kernel(StreamArgs a) {
 #pragma unroll
   for (int s = 0; s < S; ++s) {
     ci[s] = a.in[s];
-    co[s] = y ? a.out[s] : 0.f;
+    co[s] = upd ? a.out[s] : 0.f;
 #pragma unroll
-    for (int t = 0; t < S; ++t) cm[s][t] = y ? a.mix[s * S + t] : 0.f;
+    for (int t = 0; t < S; ++t) cm[s][t] = upd ? a.mix[s * S + t] : 0.f;
   }
   float ss = 0.f;
 #pragma unroll 2
@@ -64,8 +65,20 @@ __global__ __launch_bounds__(NTH) void stream_rows_kernel(StreamArgs a) {
 #pragma unroll
       for (int s = 0; s < S; ++s) x[s] = *reinterpret_cast<const float4*>(xs + (size_t)s * a.Dp + c);
     }
-    if (y) {
-      const float4 yv = act4(y + c);
+    if (upd) {
+      float4 yv;
+      if (a.y_part) {  // planes in ascending order, all requested before the first add
+        float4 pl[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          pl[i] = *reinterpret_cast<const float4*>(a.y_part + ((size_t)min(i, a.nsplit - 1) * gridDim.x + m) * a.Dp + c);
+        yv = pl[0];
+#pragma unroll
+        for (int i = 1; i < 4; ++i)
+          if (i < a.nsplit) { yv.x += pl[i].x; yv.y += pl[i].y; yv.z += pl[i].z; yv.w += pl[i].w; }
+      } else {
+        yv = act4(y + c);
+      }
       float4 old[S];
 #pragma unroll
       for (int s = 0; s < S; ++s) old[s] = x[s];
@@ -81,17 +94,17 @@ __global__ __launch_bounds__(NTH) void stream_rows_kernel(StreamArgs a) {
 #pragma unroll
     for (int s = 0; s < S; ++s) {
       fma4(u, ci[s], x[s]);
-      if (a.store && (er || y)) *reinterpret_cast<float4*>(xs + (size_t)s * a.Dp + c) = x[s];
+      if (a.store && (er || upd)) *reinterpret_cast<float4*>(xs + (size_t)s * a.Dp + c) = x[s];
     }
     *reinterpret_cast<float4*>(u_s + c) = u;
     ss += u.x * u.x + u.y * u.y + u.z * u.z + u.w * u.w;
   }
   ss = block_sum<NTH / 64>(ss, smem);
   const float inv = 1.f / sqrtf(ss / (float)a.D + a.eps);
-  T* xn = reinterpret_cast<T*>(a.xn) + (size_t)m * a.Dp;
+  T* xn = reinterpret_cast<T*>(a.xn);
   for (int c = threadIdx.x * 4; c < a.Dp; c += NTH * 4) {
     const float4 u = *reinterpret_cast<const float4*>(u_s + c), w = *reinterpret_cast<const float4*>(a.norm_w + c);
-    put_act4(xn + c, make_float4(u.x * inv * w.x, u.y * inv * w.y, u.z * inv * w.z, u.w * inv * w.w));
+    put_act4(xn + (a.xn_tiled ? act_tile_off(m, c, a.Dp) : (size_t)m * a.Dp + c), make_float4(u.x * inv * w.x, u.y * inv * w.y, u.z * inv * w.z, u.w * inv * w.w));
   }
 }
 
@@ -105,6 +118,7 @@ static void launch_streams(hipStream_t st, const StreamArgs& a, int M) {
 int stream_rows(hipStream_t st, int act, const StreamArgs& a, int M) {
   if (M <= 0 || a.Dp <= 0 || a.Dp % 64 || a.D > a.Dp || a.D <= 0 || a.Dp > 14336) return TMX_ERR_SHAPE;
   if (act != TMX_ACT_BF16 && act != TMX_ACT_F32) return TMX_ERR_ARG;
+  if (a.y_part && (a.nsplit < 1 || a.nsplit > 4)) return TMX_ERR_ARG;
 #define TMX_STREAMS(n)                                           \
   case n:                                                        \
     if (act == TMX_ACT_BF16) launch_streams<n, uint16_t>(st, a, M); \

@@ -34,6 +34,7 @@ struct LatentWorkspace {
   float* xs;            // residual streams [rows][S][Dp]
   void *xn, *z, *q, *lat, *val, *y, *act;
   float* attn_partial;
+  float* y_part;        // f32 planes of a projection whose K is split [nsplit][rows][Dp]
   float* logits;        // f32 models: products of the head [rows][Vp]
   void* head_partial;
   size_t total;

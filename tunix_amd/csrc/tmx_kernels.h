@@ -282,13 +282,30 @@ struct DenseArgs {
   void* y;
   int ldy, y_head;
   int M, K, N, heads, epi;
+  // Up to 128 bf16 rows may travel between launches in the order the matrix pipe reads them (act_tile_off) instead of
+  // row by row: x_tiled (heads == 1, ldx == K), y_tiled (ldy: columns of the tiled tensor).
+  bool x_tiled, y_tiled;
+  // nsplit > 1 (plain epilogue, heads == 1): slice s of K writes plane s of y_part [nsplit][M][N] f32, whose sum is the
+  // product; the bias is in plane 0.
+  int nsplit;
+  float* y_part;
 };
+
+// Element offset of (row, column) in a tiled activation tensor of `cols` columns (a multiple of 64): 32 rows x 64
+// columns are 2048 consecutive elements, in them the 8 columns 32 h + 8 t .. of row n at (t * 64 + 32 h + n) * 8.
+__host__ __device__ inline size_t act_tile_off(int row, int col, int cols) {
+  return ((size_t)(row >> 5) * (cols >> 6) + (col >> 6)) * 2048 + ((col >> 3) & 3) * 512 + ((col >> 5) & 1) * 256 +
+         (row & 31) * 8 + (col & 7);
+}
 
 // Mixing of the residual streams + the next sublayer's norm, see tmx_stream_rows; with `embed` set the streams are
 // first filled with embed[token] + pos_embed[position] of every row.
 struct StreamArgs {
   float* xs;           // [M][S][Dp]
   const void* y;       // act [M][Dp] or null
+  const float* y_part; // instead of y: f32 planes [nsplit][M][Dp], added in order
+  int nsplit;
+  bool xn_tiled;       // xn in the order of act_tile_off
   const float *mix, *out, *in, *norm_w;
   void* xn;
   int S, D, Dp, store;
@@ -331,6 +348,7 @@ struct LatentAttnArgs {  // see tmx_latent_attention
 };
 
 int dense_linear(hipStream_t st, int act, const DenseArgs& a);
+int dense_num_splits(int act, int M, int K, int N);  // slices of K worth their planes for a projection into the streams
 int stream_rows(hipStream_t st, int act, const StreamArgs& a, int M);
 int latent_rows(hipStream_t st, int act, const LatentRowsArgs& a, int M);
 int latent_attention(hipStream_t st, int act, LatentAttnArgs a);
