@@ -314,9 +314,10 @@ def main():
                   help='prefill and decode throughput of the latent-attention design at this size beside the closest '
                        'quantised model: a separate JSON line, not the headline metric')
   ap.add_argument('--latent-batches', type=int, nargs='+', default=[1, 16, 64])
+  ap.add_argument('--latent-prompt', type=int, default=512, help='--latent: prompt tokens in front of the decoding')
   args = ap.parse_args()
   if args.latent:
-    latent_bench(args.latent, args.latent_batches, 512, min(args.steps, 64))
+    latent_bench(args.latent, args.latent_batches, args.latent_prompt, min(args.steps, 64))
     return
   if args.pmc_summary:
     pmc_summary(args.pmc_summary[0], args.pmc_summary[1], args.match)

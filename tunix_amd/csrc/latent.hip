@@ -77,17 +77,23 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(LatentRowsArgs a) {
 //   SHARED (many query rows per sequence): WP = 1, all waves walk the same blocks;
 //   else (up to 32 query rows): WQ = 1, the position groups take different blocks and meet through LDS at the end.
 // WC = 2 at the full latent width, where the accumulators of 32 queries and the query fragments of one wave would not
-// fit its registers: both waves make the scores, each one half of the columns.
+// fit its registers: two waves share the query rows, each with half of the output columns.
+//   PAIR (SHARED with WC = 2): a round takes two blocks; each wave of a pair scores one of them and hands its
+//   probabilities to the other through LDS, so no score is computed twice.
+//   else with WC = 2: both waves make the scores.
 // KVT: latent width / 32, RT: width of the rotated part / 64.
 template <int KVT, int RT, bool SHARED>
 struct LatentShape {
   static constexpr int WC = KVT > 8 ? 2 : 1, WQ = SHARED ? 4 / WC : 1, WP = SHARED ? 1 : 4 / WC;
+  static constexpr bool PAIR = SHARED && WC == 2;
   static constexpr int kLd = KVT * 32 + RT * 64;
   static constexpr size_t kTile = (size_t)32 * kLd * 2;
-  static constexpr int kBufs = 2 * WP * kTile <= 160 * 1024 ? 2 : 1;  // tiles per position group
-  static constexpr size_t kTiles = kBufs * WP * kTile;
+  static constexpr int kGroup = PAIR ? 2 : 1;                     // tiles of a position group and round
+  static constexpr size_t kExchange = PAIR ? 4 * 4096 : 0;        // probabilities of a wave's block
+  static constexpr int kBufs = 2 * WP * kGroup * kTile + kExchange <= 160 * 1024 ? 2 : 1;
+  static constexpr size_t kTiles = kBufs * WP * kGroup * kTile;
   static constexpr size_t kMerge = SHARED ? 0 : (size_t)(WP / 2) * (KVT * 16 * 64 * 4 + WC * 2 * 32 * 4);
-  static constexpr size_t kBytes = kTiles > kMerge ? kTiles : kMerge;
+  static constexpr size_t kBytes = kTiles + kExchange > kMerge ? kTiles + kExchange : kMerge;
 };
 
 // 16-byte chunk c of row r lies at chunk c ^ swz(r).  Rows whose stride is a multiple of the 64 banks are told apart
@@ -105,6 +111,7 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
   extern __shared__ __align__(16) unsigned char la_smem[];
   constexpr int LD = SH::kLd, CPR = LD / 8, KS = LD / 16, CP = KVT * 32;
   constexpr int WC = SH::WC, WP = SH::WP, KC = KVT / WC;  // KC: column tiles of a wave
+  constexpr bool PAIR = SH::PAIR;
   constexpr int kTile = 32 * LD;                          // elements
   constexpr int WPW = 4 / WP;                             // waves per position group
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -119,18 +126,20 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
 
   const __amdgpu_buffer_rsrc_t rc = make_rsrc(reinterpret_cast<const uint16_t*>(a.cache) + (size_t)seq * a.C * LD,
                                               (uint32_t)a.C * LD * 2u);  // rows past the cache read zero
-  uint16_t* tiles = reinterpret_cast<uint16_t*>(la_smem) + wp * SH::kBufs * kTile;
-  // 32 rows of LD columns into a tile, 1 KiB per load, shared by n waves of which this is number i0
-  auto dma = [&](__amdgpu_buffer_rsrc_t src, int row0, uint16_t* tile, int i0, auto nc) __attribute__((always_inline)) {
-    constexpr int n = decltype(nc)::value;
-    int ln = lane;
-    asm volatile("" : "+v"(ln));  // the offsets are formed at the transfer, not kept in registers over the loop
+  uint16_t* tiles = reinterpret_cast<uint16_t*>(la_smem) + wp * SH::kBufs * SH::kGroup * kTile;
+  // 32 rows of LD columns into a tile, 1 KiB per load, shared by n waves of which this is number i0: load i0 + n i, whose
+  // byte offset in the 32 rows is this lane's row_off(i0 + n i)
+  auto row_off = [&](int ld) {
+    const int g = ld * 64 + lane, row = g / CPR, slot = g - row * CPR;
+    return (row * CPR + (slot ^ latent_swz<CPR>(row))) * 16;
+  };
+  constexpr int kDma = CPR / 2 / WPW;  // loads of a wave per tile
+  int doff[kDma];
 #pragma unroll
-    for (int i = 0; i < CPR / 2 / n; ++i) {
-      const int ld = i0 + n * i;
-      const int g = ld * 64 + ln, row = g / CPR, slot = g - row * CPR;
-      load_row_to_lds(src, tile + ld * 512, (row * CPR + (slot ^ latent_swz<CPR>(row))) * 16, row0 * (LD * 2));
-    }
+  for (int i = 0; i < kDma; ++i) doff[i] = row_off(wg + WPW * i);
+  auto dma = [&](int row0, uint16_t* tile) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < kDma; ++i) load_row_to_lds(rc, tile + (wg + WPW * i) * 512, doff[i], row0 * (LD * 2));
   };
   const uint8_t* mrow = a.input_mask + (size_t)seq * a.buf_len;
   auto mask_byte = [&](int blk) __attribute__((always_inline)) {
@@ -143,44 +152,61 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
   for (int c = 0; c < KC; ++c)
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[c][r] = 0.f;
-  float m = -1e30f, l = 0.f;
+  // running maximum and sum of the softmax; exponentials are powers of two throughout (scores times log2 e), a masked
+  // score is far below the maximum of a row that has seen none
+  constexpr float kLog2e = 1.44269504f, kUnseen = -1e30f, kHidden = -2e30f;
+  const float scale2 = a.scale * kLog2e;
+  float m = kUnseen, l = 0.f;
 
   // Blocks are dealt out in turn to the position groups of all splits: the first one does not depend on *step, so its
   // transfer starts at once.  All groups of a workgroup run the same number of rounds.
-  const int blk0 = split * WP + wp, stride = a.nsplit * WP;
-  auto blk_of = [&](int round) { return blk0 + round * stride; };
+  constexpr int BG = PAIR ? 2 : WP;  // blocks of a workgroup and round
+  const int blk0 = split * BG + (PAIR ? wc : wp), stride = a.nsplit * BG;
+  auto blk_of = [&](int round) { return blk0 + round * stride; };  // the block this wave scores
   auto fetch = [&](int round, int buf) __attribute__((always_inline)) {
-    dma(rc, blk_of(round) * 32, tiles + buf * kTile, wg, IC<WPW>{});
+    if constexpr (PAIR) {  // (both tiles also where the second block lies behind the last: zeros or older rows)
+#pragma unroll
+      for (int e = 0; e < 2; ++e) dma((split * BG + e + round * stride) * 32, tiles + (buf * 2 + e) * kTile);
+    } else {
+      dma(blk_of(round) * 32, tiles + buf * kTile);
+    }
   };
+  constexpr int kBuf0 = PAIR && SH::kBufs == 2 ? 1 : 0;  // tile buffer of round 0
   // The query fragments come through LDS as well (read from memory they would be 16-byte pieces of 32 rows per load):
   // the query groups of the workgroup, two at a time, through the tiles that are not in use yet.
   u32x4_t qf[KS];
   {
-    constexpr bool early = !SHARED && SH::kBufs == 2;  // the first tile of every position group is in buffer 0
+    // the first tiles start with the queries where there is room beside them: they go to the buffer that round 0 uses
+    constexpr bool early = (!SHARED || PAIR) && SH::kBufs == 2;
     const __amdgpu_buffer_rsrc_t rq = make_rsrc(reinterpret_cast<const uint16_t*>(a.q) + (size_t)seq * rows * LD, (uint32_t)rows * LD * 2u);
     uint16_t* const lds = reinterpret_cast<uint16_t*>(la_smem);
-    if (early) fetch(0, 0);
-    constexpr int kStage = SHARED ? 2 : 1;  // query groups per turn
+    if (early) fetch(0, kBuf0);
+    constexpr int kStage = SHARED ? 2 : 1;             // query groups per turn
+    constexpr int kQTile = early && !PAIR ? 1 : 0;    // tile (of the workgroup) they pass through
 #pragma unroll
     for (int g = 0; g < SH::WQ; g += kStage) {
 #pragma unroll
-      for (int e = 0; e < kStage; ++e) dma(rq, q0 + (g + e) * 32, lds + (early ? 1 : e) * kTile, wave, IC<4>{});
+      for (int e = 0; e < kStage; ++e)
+#pragma unroll
+        for (int i = 0; i < CPR / 8; ++i)
+          load_row_to_lds(rq, lds + (kQTile + e) * kTile + (wave + 4 * i) * 512, row_off(wave + 4 * i), (q0 + (g + e) * 32) * (LD * 2));
       __builtin_amdgcn_s_waitcnt(0x0F70);
       __syncthreads();
       if (wq >= g && wq < g + kStage) {
-        const uint16_t* qb = lds + (early ? 1 : wq - g) * kTile + qi * LD;
+        const uint16_t* qb = lds + (kQTile + wq - g) * kTile + qi * LD;
 #pragma unroll
         for (int t = 0; t < KS; ++t)
           qf[t] = *reinterpret_cast<const u32x4_t*>(qb + (((KS * h + t) ^ latent_swz<CPR>(qi)) << 3));
       }
       __syncthreads();
     }
-    if (!early && SH::kBufs == 2) fetch(0, 0);
+    if (!early && SH::kBufs == 2) fetch(0, kBuf0);
   }
   const int step0 = max(min(*a.step, min(a.C, a.buf_len) - a.tpp), 0);  // clamped: every slot read lies in the cache
   const int limit = step0 + qr_l / a.H;                               // newest slot this query sees
+  const int limit0 = step0 + min(q0 + wq * 32, rows - 1) / a.H;       // the smallest one in the wave
   const int b_end = (step0 + (min(q0 + 32 * SH::WQ, rows) - 1) / a.H + 32) >> 5;  // blocks up to the workgroup's newest slot
-  const int rounds = b_end > split * WP ? (b_end - split * WP + stride - 1) / stride : 0;
+  const int rounds = b_end > split * BG ? (b_end - split * BG + stride - 1) / stride : 0;
   uint8_t mb = mask_byte(blk_of(0));
   // transposed fragments of the output product: lane (column 32 c + qi, h) takes two runs of four consecutive rows
   // (see gqa_tile_walk)
@@ -188,28 +214,18 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
   const uint32_t lsw = ((2 * g2 + (q4 >> 1)) ^ latent_swz<CPR>(4 * h + k4)) * 16;
   const uint32_t vbase = ((4 * h + k4) * LD + 4 * (q4 & 1) + wc * KC * 32) * 2;
   const int kbase = qi * LD;
-  auto block = [&](const uint16_t* kt, int blk, uint32_t mbits) __attribute__((always_inline)) {
-    constexpr int R = 4;  // LDS fragments in flight
+  constexpr int R = 4;  // LDS fragments in flight
+  auto lds_addr = [](const uint16_t* p) __attribute__((always_inline)) {
+    return (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const uint16_t*)p;
+  };
+  // scaled scores of a block; the largest one of this lane's query in mn
+  auto scores = [&](const uint16_t* kt, int blk, uint32_t mbits, f32x16_t& sacc, float& mn) __attribute__((always_inline)) {
     const int sw = latent_swz<CPR>(qi);
     bf16x8_t kf[R];
     auto load_k = [&](auto tc) __attribute__((always_inline)) {
       constexpr int t = decltype(tc)::value;
       kf[t % R] = *reinterpret_cast<const bf16x8_t*>(kt + kbase + (((KS * h + t) ^ sw) << 3));
     };
-    // (the reads are spelled in assembly: for the builtin the compiler waits for every direct-to-LDS load in flight,
-    // i.e. for the next tile; the waits below count them instead)
-    const uint32_t vb = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const uint16_t*)kt + vbase;
-    u32x2_t vf[R][2];
-    auto load_v = [&](auto fc) __attribute__((always_inline)) {
-      constexpr int f = decltype(fc)::value, kb2 = f / KC, c = f % KC;
-      static_for<2>([&](auto ac) __attribute__((always_inline)) {
-        constexpr int a2 = decltype(ac)::value, row0 = 16 * kb2 + 8 * a2;
-        const uint32_t ad = vb + (lsw ^ (uint32_t)(((4 * c) ^ latent_swz<CPR>(row0)) * 16));
-        u32x2_t& dst = vf[f % R][a2];
-        asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(dst) : "v"(ad), "i"(row0 * LD * 2));
-      });
-    };
-    f32x16_t sacc;
 #pragma unroll
     for (int r = 0; r < 16; ++r) sacc[r] = 0.f;
     static_for<R>([&](auto tc) __attribute__((always_inline)) { load_k(tc); });
@@ -220,21 +236,31 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
       if constexpr (t + R < KS) load_k(IC<t + R>{});
       __builtin_amdgcn_sched_barrier(0);
     });
-    static_for<R>([&](auto fc) __attribute__((always_inline)) { load_v(fc); });  // they do not wait for the softmax
-    __builtin_amdgcn_sched_barrier(0);
-    float mn = m;
+    mn = kUnseen;
+    if (mbits == 0xFFFFFFFFu && blk * 32 + 31 <= limit0) {  // every query of the wave sees the whole block
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      const int pl = acc_row(r, lane);
-      const bool ok = blk * 32 + pl <= limit && ((mbits >> pl) & 1u);
-      sacc[r] = ok ? sacc[r] * a.scale : -1e30f;
-      mn = fmaxf(mn, sacc[r]);
+      for (int r = 0; r < 16; ++r) {
+        sacc[r] *= scale2;
+        mn = fmaxf(mn, sacc[r]);
+      }
+    } else {
+      const int lim = limit - blk * 32 - 4 * h;
+      const uint32_t mb2 = mbits >> (4 * h);
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const int pc = (r >> 2) * 8 + (r & 3);  // acc_row(r, lane) without the lane's half
+        sacc[r] = pc <= lim && ((mb2 >> pc) & 1u) ? sacc[r] * scale2 : kHidden;
+        mn = fmaxf(mn, sacc[r]);
+      }
     }
     mn = fmaxf(mn, __shfl_xor(mn, 32, 64));
-    // the reference point of the exponentials moves only when a score has left it by more than 8: until then the
-    // probabilities stay below e^8 and the accumulators need no rescaling
-    if (__any(mn > m + 8.f)) {
-      const float alpha = __expf(m - mn);
+  };
+  // The reference point of the exponentials moves only when a score has left it by more than 12: until then the
+  // probabilities stay below 2^12 and the accumulators need no rescaling.
+  auto move_reference = [&](float mn) __attribute__((always_inline)) {
+    if (__any(mn > m + 12.f)) {
+      mn = fmaxf(mn, m);
+      const float alpha = __builtin_amdgcn_exp2f(m - mn);
       m = mn;
       l *= alpha;
 #pragma unroll
@@ -242,45 +268,125 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
 #pragma unroll
         for (int r = 0; r < 16; ++r) o[c][r] *= alpha;
     }
-    uint32_t pk[8], pl2[8];
+  };
+  // probabilities as bf16 hi (p[0], p[1]) and lo (p[2], p[3]), 16 positions each
+  auto probabilities = [&](const f32x16_t& sacc, u32x4_t* p) __attribute__((always_inline)) {
 #pragma unroll
     for (int r = 0; r < 16; r += 2) {
-      const float p0 = sacc[r] > -1e29f ? __expf(sacc[r] - m) : 0.f;
-      const float p1 = sacc[r + 1] > -1e29f ? __expf(sacc[r + 1] - m) : 0.f;
-      pk[r >> 1] = pack_bf2(p0, p1);
-      pl2[r >> 1] = pack_bf2(p0 - bf_lo(pk[r >> 1]), p1 - bf_hi(pk[r >> 1]));
+      const float p0 = __builtin_amdgcn_exp2f(sacc[r] - m), p1 = __builtin_amdgcn_exp2f(sacc[r + 1] - m);
+      const uint32_t hi = pack_bf2(p0, p1);
+      p[r >> 3][(r >> 1) & 3] = hi;
+      p[2 + (r >> 3)][(r >> 1) & 3] = pack_bf2(p0 - bf_lo(hi), p1 - bf_hi(hi));
       l += p0 + p1;
     }
-    // out^T += rows^T . P^T, 16 positions (accumulator registers 8 kb2 .. 8 kb2 + 7) per MFMA
+  };
+  // Transposed fragments f = (half kb2 of the block, column tile c) of a tile.  (The reads are spelled in assembly: for
+  // the builtin the compiler waits for every direct-to-LDS load in flight, i.e. for the next tile; the waits in
+  // `product` count them instead.)
+  u32x2_t vf[R][2];
+  auto load_v = [&](uint32_t vb, auto fc) __attribute__((always_inline)) {
+    constexpr int f = decltype(fc)::value, kb2 = f / KC, c = f % KC;
+    static_for<2>([&](auto ac) __attribute__((always_inline)) {
+      constexpr int a2 = decltype(ac)::value, row0 = 16 * kb2 + 8 * a2;
+      const uint32_t ad = vb + (lsw ^ (uint32_t)(((4 * c) ^ latent_swz<CPR>(row0)) * 16));
+      u32x2_t& dst = vf[f % R][a2];
+      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(dst) : "v"(ad), "i"(row0 * LD * 2));
+    });
+  };
+  auto request_v = [&](const uint16_t* kt) __attribute__((always_inline)) {  // the first R fragments of a tile
+    const uint32_t vb = lds_addr(kt) + vbase;
+    static_for<R>([&](auto fc) __attribute__((always_inline)) { load_v(vb, fc); });
+    __builtin_amdgcn_sched_barrier(0);
+  };
+  // out^T += rows^T . P^T, 16 positions (accumulator registers 8 kb2 .. 8 kb2 + 7) per MFMA
+  auto product = [&](const uint16_t* kt, const u32x4_t* p) __attribute__((always_inline)) {
+    const uint32_t vb = lds_addr(kt) + vbase;
     static_for<2 * KC>([&](auto fc) __attribute__((always_inline)) {
       constexpr int f = decltype(fc)::value, kb2 = f / KC, c = f % KC;
-      const u32x4_t pf = {pk[4 * kb2], pk[4 * kb2 + 1], pk[4 * kb2 + 2], pk[4 * kb2 + 3]};
-      const u32x4_t pg = {pl2[4 * kb2], pl2[4 * kb2 + 1], pl2[4 * kb2 + 2], pl2[4 * kb2 + 3]};
       constexpr int kLater = 2 * KC - 1 - f < R - 1 ? 2 * KC - 1 - f : R - 1;  // fragments requested behind this one
       u32x2_t &v0 = vf[f % R][0], &v1 = vf[f % R][1];
       asm volatile("s_waitcnt lgkmcnt(%2)" : "+v"(v0), "+v"(v1) : "i"(2 * kLater));
       const u32x4_t v = {v0.x, v0.y, v1.x, v1.y};
-      o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, v), __builtin_bit_cast(bf16x8_t, pf),
+      o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, v), __builtin_bit_cast(bf16x8_t, p[kb2]),
                                                      o[c], 0, 0, 0);
-      o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, v), __builtin_bit_cast(bf16x8_t, pg),
-                                                     o[c], 0, 0, 0);
-      if constexpr (f + R < 2 * KC) load_v(IC<f + R>{});
+      o[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, v),
+                                                     __builtin_bit_cast(bf16x8_t, p[2 + kb2]), o[c], 0, 0, 0);
+      if constexpr (f + R < 2 * KC) load_v(vb, IC<f + R>{});
       __builtin_amdgcn_sched_barrier(0);
     });
   };
+  // LDS traffic between the waves of a pair, past the transfers in flight: a barrier that waits for LDS operations only
+  auto lds_barrier = [&]() __attribute__((always_inline)) {
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+  };
+  const uint32_t xch = lds_addr(reinterpret_cast<const uint16_t*>(la_smem)) + (uint32_t)SH::kTiles;
+  const uint32_t own_x = xch + wave * 4096 + lane * 16, mate_x = xch + (wave ^ 1) * 4096 + lane * 16;
 
   for (int round = 0; round < rounds; ++round) {
-    const int buf = SH::kBufs == 2 ? round & 1 : 0;
+    const int buf = SH::kBufs == 2 ? (round & 1) ^ kBuf0 : 0;
     if (SH::kBufs == 1) {
       __syncthreads();  // the last round's reads are complete
-      if (blk_of(round) < b_end) fetch(round, 0);
+      if (PAIR || blk_of(round) < b_end) fetch(round, 0);
     }
     const uint32_t mbits = (uint32_t)__ballot(mb != 0);
-    __builtin_amdgcn_s_waitcnt(0x0F70);  // this round's tile has landed
+    __builtin_amdgcn_s_waitcnt(0x0F70);  // this round's tiles have landed
     __syncthreads();
     mb = mask_byte(blk_of(round + 1));
-    if (SH::kBufs == 2 && blk_of(round + 1) < b_end) fetch(round + 1, buf ^ 1);
-    if (blk_of(round) < b_end) block(tiles + buf * kTile, blk_of(round), mbits);
+    if (SH::kBufs == 2 && (PAIR ? round + 1 < rounds : blk_of(round + 1) < b_end)) fetch(round + 1, buf ^ 1);
+    if constexpr (PAIR) {
+      const uint16_t *own = tiles + (buf * 2 + wc) * kTile, *mate = tiles + (buf * 2 + (wc ^ 1)) * kTile;
+      f32x16_t sacc;
+      float mn, mn2;
+      u32x4_t p[4], p2[4];
+      scores(own, blk_of(round), mbits, sacc, mn);
+      // the pair agrees on the reference point: a wave leaves its maximum in the mate's exchange area, which only the
+      // mate writes to afterwards
+      asm volatile("ds_write_b32 %0, %1" ::"v"(mate_x), "v"(mn) : "memory");
+      lds_barrier();
+      asm volatile("ds_read_b32 %0, %1\n\ts_waitcnt lgkmcnt(0)" : "=v"(mn2) : "v"(own_x) : "memory");
+      request_v(own);
+      move_reference(fmaxf(mn, mn2));
+      probabilities(sacc, p);
+      static_for<4>([&](auto ic) __attribute__((always_inline)) {
+        constexpr int i = decltype(ic)::value;
+        const u32x4_t& src = p[i];
+        const uint32_t at = own_x;
+        asm volatile("ds_write_b128 %0, %1 offset:%2" ::"v"(at), "v"(src), "i"(i * 1024) : "memory");
+      });
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      product(own, p);
+      lds_barrier();
+      static_for<4>([&](auto ic) __attribute__((always_inline)) {
+        constexpr int i = decltype(ic)::value;
+        u32x4_t& dst = p2[i];
+        const uint32_t at = mate_x;
+        asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(dst) : "v"(at), "i"(i * 1024) : "memory");
+      });
+      request_v(mate);
+      {
+        u32x4_t &q0_ = p2[0], &q1_ = p2[1], &q2_ = p2[2], &q3_ = p2[3];
+        asm volatile("s_waitcnt lgkmcnt(%4)" : "+v"(q0_), "+v"(q1_), "+v"(q2_), "+v"(q3_) : "i"(2 * R));
+      }
+      product(mate, p2);
+    } else if (blk_of(round) < b_end) {
+      const uint16_t* kt = tiles + buf * kTile;
+      f32x16_t sacc;
+      float mn;
+      u32x4_t p[4];
+      scores(kt, blk_of(round), mbits, sacc, mn);
+      request_v(kt);  // they do not wait for the softmax
+      move_reference(mn);
+      probabilities(sacc, p);
+      product(kt, p);
+    }
+  }
+  if constexpr (PAIR) {  // each wave has counted its own blocks
+    float l2;
+    lds_barrier();
+    asm volatile("ds_write_b32 %0, %1" ::"v"(mate_x), "v"(l) : "memory");
+    lds_barrier();
+    asm volatile("ds_read_b32 %0, %1\n\ts_waitcnt lgkmcnt(0)" : "=v"(l2) : "v"(own_x) : "memory");
+    l += l2;
   }
   l += __shfl_xor(l, 32, 64);
   if constexpr (WP > 1) {
@@ -300,7 +406,7 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
     };
     auto take = [&](int s) __attribute__((always_inline)) {
       const float m2 = ml[(s * WC + wc) * 64 + qi], l2 = ml[(s * WC + wc) * 64 + 32 + qi];
-      const float mm = fmaxf(m, m2), w1 = __expf(m - mm), w2 = __expf(m2 - mm);
+      const float mm = fmaxf(m, m2), w1 = __builtin_amdgcn_exp2f(m - mm), w2 = __builtin_amdgcn_exp2f(m2 - mm);
 #pragma unroll
       for (int c = 0; c < KC; ++c)
 #pragma unroll
@@ -318,16 +424,19 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
     }
     if (wp != 0) return;
   }
-  if (qr >= rows) return;
+  constexpr int kOut = KC * 32 + 8;  // PAIR: row stride of the results in LDS
+  if constexpr (PAIR) __syncthreads();  // the tiles are free
+  if ((PAIR && a.nsplit == 1 ? q0 + wq * 32 : qr) >= rows) return;
   if (a.nsplit == 1) {
     float w = 1.f;
     if (a.sink) {  // one more term of the denominator, without a value
-      const float s = a.sink[qr % a.H], mm = fmaxf(m, s);
-      w = __expf(m - mm);
-      l = l * w + __expf(s - mm);
+      const float s = a.sink[qr % a.H] * kLog2e, mm = fmaxf(m, s);
+      w = __builtin_amdgcn_exp2f(m - mm);
+      l = l * w + __builtin_amdgcn_exp2f(s - mm);
     }
     const float inv = l > 0.f ? w / l : 0.f;
     uint16_t* dst = reinterpret_cast<uint16_t*>(a.out) + qrow * CP + wc * KC * 32;
+    if constexpr (PAIR) dst = reinterpret_cast<uint16_t*>(la_smem) + wave * kOut * 32 + qi * kOut;
 #pragma unroll
     for (int c = 0; c < KC; ++c)
 #pragma unroll
@@ -337,19 +446,29 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
         v.y = pack_bf2(o[c][4 * i + 2] * inv, o[c][4 * i + 3] * inv);
         *reinterpret_cast<uint2*>(dst + 32 * c + 8 * i + 4 * h) = v;
       }
+    if constexpr (PAIR) {  // the wave's own rows, out again in whole lines
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      constexpr int CPO = KC * 4;  // 16-byte chunks of a row
+#pragma unroll
+      for (int i = 0; i < 32 * CPO / 64; ++i) {
+        const int g = i * 64 + lane, row = g / CPO, ch = g % CPO, q = q0 + wq * 32 + row;
+        const u32x4_t v = *reinterpret_cast<const u32x4_t*>(reinterpret_cast<const uint16_t*>(la_smem) + wave * kOut * 32 + row * kOut + ch * 8);
+        if (q < rows)
+          *reinterpret_cast<u32x4_t*>(reinterpret_cast<uint16_t*>(a.out) + ((size_t)seq * rows + q) * CP + wc * KC * 32 + ch * 8) = v;
+      }
+    }
     return;
   }
-  float* pr = a.partial + (qrow * a.nsplit + split) * (CP + 2);
+  float* pr = a.partial + (qrow * a.nsplit + split) * (CP + 4);
 #pragma unroll
   for (int c = 0; c < KC; ++c)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       float* d = pr + 32 * (wc * KC + c) + 8 * i + 4 * h;
-      *reinterpret_cast<f32x2_t*>(d) = f32x2_t{o[c][4 * i], o[c][4 * i + 1]};
-      *reinterpret_cast<f32x2_t*>(d + 2) = f32x2_t{o[c][4 * i + 2], o[c][4 * i + 3]};
+      *reinterpret_cast<f32x4_t*>(d) = f32x4_t{o[c][4 * i], o[c][4 * i + 1], o[c][4 * i + 2], o[c][4 * i + 3]};
     }
   if (h == 0 && wc == 0) {
-    pr[CP] = m;
+    pr[CP] = m * (1.f / kLog2e);  // (natural units, as the sink)
     pr[CP + 1] = l;
   }
 }
@@ -358,18 +477,18 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a) {
 __global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnArgs a) {
   const int CP = a.rank_p;
   const size_t row = blockIdx.x;
-  const float* pr = a.partial + row * a.nsplit * (CP + 2);
+  const float* pr = a.partial + row * a.nsplit * (CP + 4);  // [split][CP values | max | sum | -]
   float mm = a.sink ? a.sink[row % a.H] : -1e30f;
   const float sink = mm;
-  for (int s = 0; s < a.nsplit; ++s) mm = fmaxf(mm, pr[(size_t)s * (CP + 2) + CP]);
+  for (int s = 0; s < a.nsplit; ++s) mm = fmaxf(mm, pr[(size_t)s * (CP + 4) + CP]);
   float l = a.sink ? __expf(sink - mm) : 0.f;
-  for (int s = 0; s < a.nsplit; ++s) l += pr[(size_t)s * (CP + 2) + CP + 1] * __expf(pr[(size_t)s * (CP + 2) + CP] - mm);
+  for (int s = 0; s < a.nsplit; ++s) l += pr[(size_t)s * (CP + 4) + CP + 1] * __expf(pr[(size_t)s * (CP + 4) + CP] - mm);
   const float inv = l > 0.f ? 1.f / l : 0.f;
   for (int c = threadIdx.x * 2; c < CP; c += 512) {
     f32x2_t v = {0.f, 0.f};
 #pragma unroll 4
     for (int s = 0; s < a.nsplit; ++s) {
-      const float* p = pr + (size_t)s * (CP + 2);
+      const float* p = pr + (size_t)s * (CP + 4);
       const float w = __expf(p[CP] - mm);
       const f32x2_t x = *reinterpret_cast<const f32x2_t*>(p + c);
       v.x = fmaf(x.x, w, v.x);
@@ -475,7 +594,7 @@ size_t latent_attn_partial_bytes(int rows, int H, int rank_p) {
   // nsplit > 1 only while nsplit * workgroups <= kLatentWgs, and a workgroup holds at most 128 query rows
   size_t parts = (size_t)rows * H * kLatentMaxSplits;
   if (parts > (size_t)kLatentWgs * 128) parts = (size_t)kLatentWgs * 128;
-  return parts * (rank_p + 2) * 4;
+  return parts * (rank_p + 4) * 4;
 }
 
 template <int KVT, int RT, bool SHARED>
@@ -541,7 +660,7 @@ extern "C" int tmx_latent_rows(void* stream, int act, const void* z, int ldz, in
 extern "C" size_t tmx_latent_attention_workspace_bytes(int n_seq, int T, int H, int rank_p, int C) {
   if (n_seq <= 0 || T <= 0 || H <= 0 || C <= 0) return 0;
   const LatentPlan p = latent_plan(n_seq, T, H, rank_p, C);
-  return p.nsplit == 1 ? 0 : (size_t)n_seq * T * H * p.nsplit * (rank_p + 2) * 4;
+  return p.nsplit == 1 ? 0 : (size_t)n_seq * T * H * p.nsplit * (rank_p + 4) * 4;
 }
 
 extern "C" int tmx_latent_attention(void* stream, int act, const void* q, const void* cache, const float* sink,

@@ -342,7 +342,7 @@ struct LatentAttnArgs {  // see tmx_latent_attention
   const int32_t* step;
   int buf_len;
   void* out;
-  float* partial;  // [rows H][nsplit][rank_p + 2]
+  float* partial;  // [rows H][nsplit][rank_p + 4]: values, maximum, sum
   int n_seq, tpp, H, rank_p, rot_p, C, nsplit;
   float scale;
 };

@@ -364,7 +364,10 @@ class LatentModel:
   def from_state(cls, config, state, device='cuda'):
     """state: name -> tensor, exactly the names and shapes of tensor_shapes(config)."""
     want = tensor_shapes(config)
-    missing, extra = sorted(set(want) - set(state)), sorted(set(state) - set(want))
+    # a layer without a feed-forward has no use for the norm and the stream coefficients in front of one
+    idle = tuple(f'l{i}.{n}' for i, l in enumerate(config.layers) if l.ff is None for n in ('norm2', 'hc2.'))
+    missing = sorted(set(want) - set(state))
+    extra = sorted(k for k in set(state) - set(want) if not (idle and k.startswith(idle)))
     if missing or extra:
       raise KeyError(f'checkpoint does not fit the configuration: missing {missing[:4]}, unexpected {extra[:4]}')
     for k, shape in want.items():
