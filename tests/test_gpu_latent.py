@@ -378,6 +378,21 @@ def test_more_rows_than_the_streaming_kernels_take():
   assert np.abs(lp[0] - ref).max() < 0.1
 
 
+@pytest.mark.parametrize('dtype', FORMATS)
+def test_projections_whose_k_is_split(dtype):
+  """Long K in front of the streams: the slices' planes are added by the stream row kernel, in both kernel forms."""
+  cfg = LC.config([LC.layer('latent_attention', 32, 20, 8, 60, 50, 4050), LC.layer('latent_attention_2', 17, 20, 8, 130, 50, 2100, kv_from=None)],
+                  vocab=96, width=250, streams=3, max_positions=80)
+  st = LC.make_state(cfg, 4)
+  m = LC.product(cfg, st, dtype)
+  rows = [np.random.default_rng(i).integers(0, 96, 24) for i in range(12)]
+  want = [LC.plain(cfg, st, r, dtype) for r in rows[:2]]
+  for n, cuts in ((1, [20, 1, 1, 2]), (2, [24]), (12, [22, 1, 1]), (12, [24])):
+    got = all_logits(sampler(m, 32), rows[:n], 32, cuts)
+    for g, w in zip(got, want):
+      assert LC.error(g, w) < LC.LIMIT[dtype], (n, cuts)
+
+
 # -- generation through the framework's entry points ------------------------------------
 @pytest.mark.parametrize('dtype', FORMATS)
 @pytest.mark.parametrize('name', ['mixed', 'wide'])

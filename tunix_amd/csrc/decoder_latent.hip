@@ -1,6 +1,6 @@
 // Layers of one pass of a TMX_FAMILY_LATENT model: dense weights, latent attention, several residual streams.
-// Per layer: fused projection of the normed input (query | latent | gate), rotation / norm / cache row, query into the
-// latent space, attention over the cache rows, values (with the output gate in the epilogue), output projection,
+// Per layer: fused projection of the normed input (query | latent | gate), rotation / norm / cache row and query into
+// the latent space (one launch up to 128 rows), attention over the cache rows, values (with the output gate in the epilogue), output projection,
 // stream row kernel; gate | up with SwiGLU, down, stream row kernel.  A row kernel between two sublayers applies the
 // first one's result to the streams and makes the second one's normed input.
 #include "tmx_decoder.h"
@@ -158,9 +158,14 @@ int latent_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_stat
       a.positions = s->positions; a.step = s->step; a.buf_len = L; a.tpp = T;
       a.q = w.q; a.cache = cache[i];
       a.H = H; a.rot = l.rot_dim; a.rank = l.kv_rank; a.rank_p = l.rank_p; a.rot_p = l.rot_p; a.C = C;
-      TMX_TRY(TMX_K_ROPE, latent_rows(st, act, a, M));
+      const DenseArgs d = args(l.uk, w.z, l.in.N, l.dim_p, w.q, H * ld, ld, TMX_DENSE_PLAIN);
+      if (tiled) {
+        TMX_TRY(TMX_K_LATENT_Q, latent_q_rows(st, d, a));
+      } else {
+        TMX_TRY(TMX_K_ROPE, latent_rows(st, act, a, M));
+        TMX_TRY(TMX_K_LATENT_Q, dense_linear(st, act, d));
+      }
     }
-    TMX_TRY(TMX_K_LATENT_Q, dense_linear(st, act, args(l.uk, w.z, l.in.N, l.dim_p, w.q, H * ld, ld, TMX_DENSE_PLAIN)));
     {
       LatentAttnArgs a = {};
       a.q = w.q; a.cache = cache[i]; a.sink = l.sink;

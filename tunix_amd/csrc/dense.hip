@@ -8,7 +8,7 @@
 //   more rows       dense_wide_kernel: 256 rows x 32 MT columns per workgroup; the weight slab of a k-step goes
 //                   global -> LDS by direct loads, the activations are the B operand straight from memory
 // f32: dense_f32_kernel, a plain tiled product on the vector ALU (no matrix pipe, no reduced precision).
-#include "tmx_kernels.h"
+#include "tmx_latent_rows.h"
 
 namespace tmx {
 
@@ -18,22 +18,23 @@ __device__ __forceinline__ float sigmoid(float z) { return 1.f / (1.f + expf(-z)
 // MT: 32-row tiles of x; WK: waves that share K (8 / WK column tiles per workgroup); NT = 2: SwiGLU pairs (a gate
 // tile and the up tile N / 64 tiles further).
 // XT: x is tiled (act_tile_off): a wave's load is 1 KiB of consecutive bytes instead of 16-byte pieces of 32 rows.
+// One workgroup: column tiles bx * 8 / WK .., matrix `head`, slice `slice` of K; lds: kDenseSmallLds bytes.
+constexpr int kDenseSmallLds = 65536;
 template <int MT, int WK, int NT, bool XT>
-__global__ __launch_bounds__(512, 2) void dense_small_kernel(DenseArgs a) {
+__device__ __forceinline__ void dense_small_block(const DenseArgs& a, int bx, int head, int slice, void* lds) {
   constexpr int WN = 8 / WK;
-  __shared__ float red[WK > 1 ? 2 : 1][WK > 1 ? 8 * 1024 : 1];
+  float* red = reinterpret_cast<float*>(lds);  // [2][8 waves][1024]
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int h = lane >> 5, nl = lane & 31;
   const int wn = wave / WK, wk = wave % WK;
   const int KT = a.K >> 6;
-  const int kts = (KT + a.nsplit - 1) / a.nsplit, slice = blockIdx.z;
+  const int kts = (KT + a.nsplit - 1) / a.nsplit;
   const int k_beg = slice * kts, k_end = k_beg + kts < KT ? k_beg + kts : KT, klast = k_end - 1;
   const int pair = a.N >> 6;  // tiles from a gate tile to its up tile
   const int tiles = NT == 2 ? pair : a.N >> 5;
-  const int tile = blockIdx.x * WN + wn;
+  const int tile = bx * WN + wn;
   const int tl = tile < tiles ? tile : tiles - 1;  // waves past the end repeat the last tile (dropped)
-  const int head = blockIdx.y;
   const u32x4_t* wsrc[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n)
@@ -96,54 +97,67 @@ __global__ __launch_bounds__(512, 2) void dense_small_kernel(DenseArgs a) {
 
   const float b0 = a.bias && slice == 0 ? a.bias[tl * 32 + nl] : 0.f;
   const float b1 = (NT == 2 && a.bias) ? a.bias[(tl + pair) * 32 + nl] : 0.f;
+  // Finished bf16 values wait in LDS [rows of x][WN * 32 columns] and leave 8 columns at a time.
+  constexpr int OW = WN * 32;
+  uint16_t* out_s = reinterpret_cast<uint16_t*>(lds);
+  const bool planes = NT == 1 && a.nsplit > 1;
   auto finish = [&](int m, int r, const float* s) __attribute__((always_inline)) {
     const int row = m * 32 + acc_row(r, lane), col = tile * 32 + nl;
-    if (row >= a.M || tile >= tiles) return;
     float v = s[0] + b0;
-    if (NT == 1 && a.nsplit > 1) {
-      a.y_part[((size_t)slice * a.M + row) * a.N + col] = v;
+    if (planes) {
+      if (row < a.M && tile < tiles) a.y_part[((size_t)slice * a.M + row) * a.N + col] = v;
       return;
     }
     if (NT == 2) v = silu(v) * (s[NT - 1] + b1);
-    if (a.epi == TMX_DENSE_GATED)
+    if (a.epi == TMX_DENSE_GATED && row < a.M && tile < tiles)
       v *= sigmoid(bf2f(reinterpret_cast<const uint16_t*>(a.gate)[(size_t)row * a.ldg + head * a.y_head + col]));
-    const int yc = head * a.y_head + col;
-    reinterpret_cast<uint16_t*>(a.y)[a.y_tiled ? act_tile_off(row, yc, a.ldy) : (size_t)row * a.ldy + yc] = f2bf(v);
+    out_s[row * OW + wn * 32 + nl] = f2bf(v);
   };
+  constexpr int E = 16 / WK;  // the WK waves of a column tile add their accumulators: each finishes 16 / WK registers
+  float s[MT][E][NT];
   if constexpr (WK == 1) {
-    static_for<MT>([&](auto mc) __attribute__((always_inline)) {
-      static_for<16>([&](auto rc) __attribute__((always_inline)) {
-        constexpr int m = decltype(mc)::value, r = decltype(rc)::value;
-        float s[NT];
+    static_for<MT * 16>([&](auto ic) __attribute__((always_inline)) {
+      constexpr int m = decltype(ic)::value / 16, r = decltype(ic)::value % 16;
 #pragma unroll
-        for (int n = 0; n < NT; ++n) s[n] = acc[n][m][r];
-        finish(m, r, s);
-      });
+      for (int n = 0; n < NT; ++n) s[m][r][n] = acc[n][m][r];
     });
   } else {
-    // the WK waves of a column tile add their accumulators through LDS: each takes 16 / WK registers of all of them
-    constexpr int E = 16 / WK;
-    static_for<MT>([&](auto mc) __attribute__((always_inline)) {
-      constexpr int m = decltype(mc)::value;
-      float s[E][NT];
-      static_for<NT>([&](auto nc) __attribute__((always_inline)) {
-        constexpr int n = decltype(nc)::value;
-        float* buf = red[(m * NT + n) & 1];
+    static_for<MT * NT>([&](auto ic) __attribute__((always_inline)) {
+      constexpr int m = decltype(ic)::value / NT, n = decltype(ic)::value % NT;
+      float* buf = red + (decltype(ic)::value & 1) * 8192;
 #pragma unroll
-        for (int r = 0; r < 16; ++r) buf[wave * 1024 + r * 64 + lane] = acc[n][m][r];
-        __syncthreads();  // (the buffer's readers of two rounds ago have passed the last round's barrier)
+      for (int r = 0; r < 16; ++r) buf[wave * 1024 + r * 64 + lane] = acc[n][m][r];
+      __syncthreads();  // (the buffer's readers of two rounds ago have passed the last round's barrier)
 #pragma unroll
-        for (int e = 0; e < E; ++e) {
-          float t = 0.f;
+      for (int e = 0; e < E; ++e) {
+        float t = 0.f;
 #pragma unroll
-          for (int w = 0; w < WK; ++w) t += buf[(wn * WK + w) * 1024 + (wk + e * WK) * 64 + lane];
-          s[e][n] = t;
-        }
-      });
-#pragma unroll
-      for (int e = 0; e < E; ++e) finish(m, wk + e * WK, s[e]);
+        for (int w = 0; w < WK; ++w) t += buf[(wn * WK + w) * 1024 + (wk + e * WK) * 64 + lane];
+        s[m][e][n] = t;
+      }
     });
+    if (!planes) __syncthreads();  // every sum is taken: the area is free for the results
   }
+  static_for<MT * E>([&](auto ic) __attribute__((always_inline)) {
+    constexpr int m = decltype(ic)::value / E, e = decltype(ic)::value % E;
+    finish(m, wk + e * WK, s[m][e]);
+  });
+  if (planes) return;
+  __syncthreads();
+  const int rows = a.M < MT * 32 ? a.M : MT * 32;
+  for (int i = tid; i < rows * (OW / 8); i += 512) {
+    const int row = i / (OW / 8), c8 = (i % (OW / 8)) * 8, col = bx * OW + c8;
+    if (col >= tiles * 32) continue;
+    const int yc = head * a.y_head + col;
+    *reinterpret_cast<u32x4_t*>(reinterpret_cast<uint16_t*>(a.y) + (a.y_tiled ? act_tile_off(row, yc, a.ldy) : (size_t)row * a.ldy + yc)) =
+        *reinterpret_cast<const u32x4_t*>(out_s + row * OW + c8);
+  }
+}
+
+template <int MT, int WK, int NT, bool XT>
+__global__ __launch_bounds__(512, 2) void dense_small_kernel(DenseArgs a) {
+  __shared__ __align__(16) unsigned char lds[kDenseSmallLds];
+  dense_small_block<MT, WK, NT, XT>(a, blockIdx.x, blockIdx.y, blockIdx.z, lds);
 }
 
 // ---------------------------------------------------------------------------
@@ -357,6 +371,34 @@ static int launch_small(hipStream_t st, const DenseArgs& a) {
   hipLaunchKernelGGL((dense_small_kernel<MT, WK, NT, XT>), dim3((tiles + wn - 1) / wn, a.heads, a.nsplit), dim3(512), 0, st, a);
   return check_launch();
 }
+// Queries into the latent space (one matrix per head) and the row part of latent attention, in one launch: the first
+// gx * heads workgroups are the projection's, the others one row each.
+template <int MT, int WK>
+__global__ __launch_bounds__(512, 2) void latent_q_rows_kernel(DenseArgs a, LatentRowsArgs r, int gx) {
+  __shared__ __align__(16) unsigned char lds[kDenseSmallLds];
+  const int b = blockIdx.x, nq = gx * a.heads;
+  if (b < nq) dense_small_block<MT, WK, 1, false>(a, b % gx, b / gx, 0, lds);
+  else latent_rows_block<uint16_t, 512>(r, b - nq, reinterpret_cast<float*>(lds));
+}
+template <int MT>
+static int launch_q_rows(hipStream_t st, const DenseArgs& a, const LatentRowsArgs& r) {
+  const int wk = a.K >= 128 ? 2 : 1, wn = 8 / wk, gx = (a.N / 32 + wn - 1) / wn;
+  const dim3 grid(gx * a.heads + a.M);
+  if (wk == 2) hipLaunchKernelGGL((latent_q_rows_kernel<MT, 2>), grid, dim3(512), 0, st, a, r, gx);
+  else hipLaunchKernelGGL((latent_q_rows_kernel<MT, 1>), grid, dim3(512), 0, st, a, r, gx);
+  return check_launch();
+}
+int latent_q_rows(hipStream_t st, DenseArgs a, const LatentRowsArgs& r) {
+  if (a.M <= 0 || a.M > 128 || a.K % 64 || a.N % 32 || a.heads <= 0 || a.bias || a.epi != TMX_DENSE_PLAIN || a.x_tiled || a.y_tiled ||
+      a.ldx % 8 || a.x_head % 8 || a.ldy % 8 || a.y_head % 8 || r.rot <= 0 || r.rot % 2 || r.rot > r.rot_p || r.rank <= 0 ||
+      r.rank > r.rank_p || !latent_attn_ok(r.rank_p, r.rot_p))
+    return TMX_ERR_SHAPE;
+  a.nsplit = 1;
+  if (a.M <= 32) return launch_q_rows<1>(st, a, r);
+  if (a.M <= 64) return launch_q_rows<2>(st, a, r);
+  return launch_q_rows<4>(st, a, r);
+}
+
 template <int MT, int NT, bool XT>
 static int launch_small_k(hipStream_t st, const DenseArgs& a) {
   const int KT = (a.K >> 6) / a.nsplit;
@@ -415,7 +457,7 @@ int dense_linear(hipStream_t st, int act, const DenseArgs& args) {
     return check_launch();
   }
   if (act != TMX_ACT_BF16) return TMX_ERR_ARG;
-  if (a.ldx % 8 || a.x_head % 8 || a.ldy % 4 || a.y_head % 4 || a.ldg % 4) return TMX_ERR_SHAPE;
+  if (a.ldx % 8 || a.x_head % 8 || a.ldy % 8 || a.y_head % 8 || a.ldg % 4) return TMX_ERR_SHAPE;
   if (a.M <= 128) {
     if (swiglu) {
       if (a.M <= 32) return launch_small_x<1, 2>(st, a);

@@ -351,6 +351,8 @@ int dense_linear(hipStream_t st, int act, const DenseArgs& a);
 int dense_num_splits(int act, int M, int K, int N);  // slices of K worth their planes for a projection into the streams
 int stream_rows(hipStream_t st, int act, const StreamArgs& a, int M);
 int latent_rows(hipStream_t st, int act, const LatentRowsArgs& a, int M);
+// dense_linear (bf16, up to 128 rows, one matrix per head) and latent_rows in one launch
+int latent_q_rows(hipStream_t st, DenseArgs a, const LatentRowsArgs& r);
 int latent_attention(hipStream_t st, int act, LatentAttnArgs a);
 bool latent_attn_ok(int rank_p, int rot_p);
 size_t latent_attn_partial_bytes(int rows, int H, int rank_p);  // room for every split of `rows` query rows
