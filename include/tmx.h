@@ -48,7 +48,7 @@ extern "C" {
 
 #define TMX_FAMILY_LLAMA3 0
 #define TMX_FAMILY_QWEN3 1
-#define TMX_FAMILY_LATENT 2 /* dense weights, latent attention, several residual streams: tmx_latent_layer_desc */
+#define TMX_FAMILY_DENSE 2 /* dense weights; mixer, feed-forward and residual are parameters: tmx_dense_layer_desc */
 
 #define TMX_ACT_BF16 0 /* activations, caches and matrix products in bf16 with f32 accumulation */
 #define TMX_ACT_F32 1  /* everything in f32 (no matrix pipe) */
@@ -56,6 +56,7 @@ extern "C" {
 #define TMX_MAX_STREAMS 8      /* residual streams of a model */
 #define TMX_MAX_LATENT_RANK 512 /* padded latent width of latent attention: 64, 128, 256 or 512 */
 #define TMX_MAX_LATENT_ROT 128  /* padded width of its shared rotated key part: 64 or 128 */
+#define TMX_MAX_HEAD_DIM 256    /* padded width of a head of grouped attention: 64, 128 or 256 */
 
 #define TMX_MAX_RPAD 128   /* widest padded LoRA projection (sum of fused ranks, rounded up to 32) */
 #define TMX_MAX_SPLITS 16  /* most K-slices a projection is split into */
@@ -72,9 +73,10 @@ extern "C" {
                               :207-226 selective_log_softmax) */
 
 const char* tmx_status_string(int status);
-/* Bumped whenever a struct of this header grows or an entry point changes: 8 = TMX_FAMILY_LATENT and the fields of
- * tmx_model_desc behind head_tiles are present.  A caller that fills the structs checks it once after loading. */
-#define TMX_ABI_VERSION 8
+/* Bumped whenever a struct of this header grows or an entry point changes: 9 = the fields of tmx_dense_layer_desc behind
+ * `down` and of tmx_model_desc behind logit_scale are present.  A caller that fills the structs checks it once after
+ * loading. */
+#define TMX_ABI_VERSION 9
 int tmx_abi_version(void);
 
 /* w_out[K, N] bf16 = bf16(q) * scale evaluated in bf16, bit-exact.
@@ -322,8 +324,8 @@ int tmx_moe_experts(void* stream, const void* x, int ldx, const void* qweight, c
                     const int32_t* expert_of, int P, int top_k, int E, int K, int N, int G, int down,
                     void* out, int ldo);
 
-/* ---- dense projections, residual streams, latent attention ------------------------
- * No counterpart in the reference: the mechanisms of TMX_FAMILY_LATENT models, each usable alone.  `act` is
+/* ---- dense projections, residuals, latent attention, grouped attention -------------
+ * No counterpart in the reference: the mechanisms of TMX_FAMILY_DENSE models, each usable alone.  `act` is
  * TMX_ACT_*; an "act tensor" holds bf16 or f32 accordingly.  Every width below is padded: columns past the real
  * width hold zeros in the weights and come out as zeros. */
 
@@ -333,11 +335,13 @@ int tmx_moe_experts(void* stream, const void* x, int ldx, const void* qweight, c
  *           TMX_ACT_F32: f32 row-major [heads][N][K].  K % 64 == 0, N % 32 == 0
  *   bias  : f32 [N] or NULL (heads == 1)
  *   epilogue TMX_DENSE_PLAIN; TMX_DENSE_SWIGLU: W holds N / 2 gate rows, then N / 2 up rows ((N / 2) % 32 == 0),
- *           y[m, n] = silu(gate) * up, N / 2 columns; TMX_DENSE_GATED: y = product * sigmoid(gate[m ldg + h y_head + n])
+ *           y[m, n] = silu(gate) * up, N / 2 columns; TMX_DENSE_GATED: y = product * sigmoid(gate[m ldg + h y_head + n]);
+ *           TMX_DENSE_RELU2: y = max(product + bias, 0)^2
  * Up to 128 rows stream the weights once; more rows run in 256-row blocks. */
 #define TMX_DENSE_PLAIN 0
 #define TMX_DENSE_SWIGLU 1
 #define TMX_DENSE_GATED 2
+#define TMX_DENSE_RELU2 3
 int tmx_dense_linear(void* stream, int act, const void* x, int ldx, int x_head, const void* w, const float* bias,
                      const void* gate, int ldg, void* y, int ldy, int y_head, int M, int K, int N, int heads,
                      int epilogue);
@@ -349,6 +353,14 @@ int tmx_dense_linear(void* stream, int act, const void* x, int ldx, int x_head, 
  *   store: 0 leaves the streams in memory untouched (the last boundary of a model needs only xn) */
 int tmx_stream_rows(void* stream, int act, float* streams, const void* y, const float* mix, const float* out,
                     const float* in, const float* norm_w, void* xn, int M, int S, int D, int Dp, float eps, int store);
+
+/* One residual stream x (f32 [M][Dp]): x <- x + (post_w ? y / sqrt(mean(y^2) + eps) * post_w : y), then
+ * xn = norm_w ? x / sqrt(mean(x^2) + eps) * norm_w : x (means over the real width D).  A norm behind the sublayer, in
+ * front of the next one, both or none.
+ *   y    : act tensor [M][Dp]; NULL: x stays as it is;  post_w, norm_w: f32 [Dp] or NULL;  xn: act tensor [M][Dp]
+ *   store: 0 leaves x in memory untouched */
+int tmx_residual_rows(void* stream, int act, float* x, const void* y, const float* post_w, const float* norm_w, void* xn,
+                      int M, int D, int Dp, float eps, int store);
 
 /* Row kernel of latent attention: takes the fused projection row z[m] = [query, unrotated: H dim_p | query,
  * rotated: H rot | latent: rank | shared key part: rot | ...] and writes
@@ -373,6 +385,29 @@ int tmx_latent_attention(void* stream, int act, const void* q, const void* cache
                          const uint8_t* input_mask, const int32_t* step, int buf_len, void* out, void* workspace,
                          int n_seq, int T, int H, int rank_p, int rot_p, int C, float scale);
 
+/* Row kernel of grouped attention: takes the fused projection row z[m] = [H query heads of dk | Kh key heads of dk | Kh
+ * value heads of dv] (dk, dv: padded widths; dim: real width of a query / key head) and writes
+ *   q[m][H][dk], and the rows of slot *step + m % T: kcache [sequence][Kh][C][dk], vcache [sequence][Kh][C][dv].
+ * Queries and keys are first divided by their root mean square (over dim) and multiplied by q_norm_w / k_norm_w (f32
+ * [dk], NULL: no norm), then their first `rot` columns are rotated: table f32 [positions_max][rot / 2][2] cos, sin; the
+ * pair of dimension i is i + rot / 2 (rot == 0: no rotation).
+ *   first: int32 [M], the first slot of the row's chunk of `chunk` positions (0 with chunk == 0), for tmx_head_attention.
+ *          Positions along a sequence's slots do not decrease; slots with input_mask 0 hold no token. */
+int tmx_head_rows(void* stream, int act, const void* z, int ldz, const float* q_norm_w, const float* k_norm_w, float eps,
+                  const float* table, int positions_max, const int32_t* positions, const uint8_t* input_mask,
+                  const int32_t* step, int buf_len, void* q, void* kcache, void* vcache, int32_t* first, int M, int T,
+                  int H, int Kh, int dim, int dk, int dv, int rot, int C, int chunk);
+
+/* out[m][h][dv] = sum_j softmax_j(q[m, h] . K[j] * scale) V[j] over the slots first[m] <= j <= *step + m % T with
+ * input_mask[m / T, j], K and V of kv head floor(h / (H / Kh)); with sink (f32 [H]) the denominator also holds
+ * exp(sink[h]).  dk and dv in {64, 128, 256}, H % Kh == 0, any H / Kh.
+ * chunk: the most slots a row sees (0: no bound), from which the launch is planned.
+ * workspace: tmx_head_attention_workspace_bytes(M / T, T, H, Kh, dv, C, chunk) bytes (may be 0 -> NULL allowed). */
+size_t tmx_head_attention_workspace_bytes(int n_seq, int T, int H, int Kh, int dv, int C, int chunk);
+int tmx_head_attention(void* stream, int act, const void* q, const void* kcache, const void* vcache, const float* sink,
+                       const int32_t* first, const uint8_t* input_mask, const int32_t* step, int buf_len, void* out,
+                       void* workspace, int n_seq, int T, int H, int Kh, int dk, int dv, int C, int chunk, float scale);
+
 /* ---- whole decode steps ------------------------------------------------------ */
 
 typedef struct {
@@ -386,6 +421,9 @@ typedef struct { /* coefficients of a sublayer's stream mixing, f32 on the devic
   const float* out; /* [S] */
   const float* mix; /* [S][S], [from, to] */
 } tmx_streams_desc;
+
+#define TMX_MIXER_LATENT 0 /* tmx_latent_rows, tmx_latent_attention */
+#define TMX_MIXER_HEADS 1  /* tmx_head_rows, tmx_head_attention */
 
 typedef struct {
   const float *norm1_w, *norm2_w; /* f32 [Dp] */
@@ -405,9 +443,15 @@ typedef struct {
   const float* table;             /* rotation table, see tmx_latent_rows */
   const float* sink;              /* f32 [heads] or NULL */
   /* feed-forward (gate_up.w == NULL: none) */
-  tmx_dense_desc gate_up;         /* gate rows, then up rows: [2 Fp, Dp] */
+  tmx_dense_desc gate_up;         /* TMX_DENSE_SWIGLU: gate rows, then up rows [2 Fp, Dp]; else up rows [Fp, Dp] */
   tmx_dense_desc down;            /* [Dp, Fp] */
-} tmx_latent_layer_desc;
+  int ff;                         /* activation of the feed-forward: TMX_DENSE_SWIGLU or TMX_DENSE_RELU2 */
+  int mixer;                      /* TMX_MIXER_* */
+  /* TMX_MIXER_HEADS uses heads, rot_dim, dim_p, vdim_p, scale, in ([query | key | value] heads), o, table, sink and */
+  int kv_heads, dim;              /* real sizes */
+  int chunk;                      /* positions of a chunk (0: a token sees every earlier one) */
+  const float *q_norm_w, *k_norm_w; /* f32 [dim_p] or NULL */
+} tmx_dense_layer_desc;
 
 typedef struct {
   const void* qweight;  /* q4t tiles of the (column-fused) weight [K, N] */
@@ -444,16 +488,20 @@ typedef struct {
   const void* head_tiles;   /* NULL, or the head matrix once more in the layout tmx_head_tiles_pack writes (V % 32
                                == 0, D % 64 == 0): steps of up to 64 sequences then stream that copy, every byte
                                in whole cache lines (the 1.05 GB head of the 8B shape: 190 us against 252 us) */
-  /* TMX_FAMILY_LATENT: num_layers, vocab_size, embed_dim and norm_eps hold the real sizes; embed [V, Dp] and
+  /* TMX_FAMILY_DENSE: num_layers, vocab_size, embed_dim and norm_eps hold the real sizes; embed [V, Dp] and
    * pos_embed are bf16; head is [Vp, Dp] bf16 (+ head_tiles) or f32; final_norm_w is f32 [Dp], with Dp = embed_dim
    * rounded up to 64 and Vp = vocab_size rounded up to 32; layers is NULL */
-  const tmx_latent_layer_desc* latent_layers; /* HOST array of num_layers entries */
+  const tmx_dense_layer_desc* dense_layers; /* HOST array of num_layers entries */
   int act;                  /* TMX_ACT_* */
   int streams;              /* 1 .. TMX_MAX_STREAMS */
-  int max_positions;        /* rows of pos_embed and of every rotation table (positions are clamped to it) */
+  int max_positions;        /* rows of pos_embed and of every rotation table (positions are clamped to them) */
   const void* pos_embed;    /* bf16 [max_positions, Dp], added to the embedding; NULL: none */
   const float* final_in;    /* f32 [streams]: weights of the streams in the final sum */
   float logit_scale;
+  float embed_scale;        /* the residual starts as embed_scale * embed[token] (+ pos_embed) */
+  int norm_after;           /* 0: norm1_w, norm2_w and the streams as tmx_stream_rows; 1: one residual stream, the sublayers
+                               read it as it is and norm1_w, norm2_w lie behind them (tmx_residual_rows); hc1, hc2 and
+                               final_in are not used */
 } tmx_model_desc;
 
 /* Mirrors _SamplingState (tunix/generate/sampler.py:53-109); all arrays on the device. */
@@ -465,8 +513,9 @@ typedef struct {
   float* logprobs;       /* [B, buf_len] or NULL */
   uint8_t* done;         /* [B] */
   int32_t* step;         /* device scalar: decoding_step */
-  void* kv_cache;        /* bf16 [layers][2 (k, v)][B][C][Kh][H]; TMX_FAMILY_LATENT: for every layer with a latent of
-                            its own, in layer order, an act tensor [B][C][rank_p + rot_p] (zero-filled before use) */
+  void* kv_cache;        /* bf16 [layers][2 (k, v)][B][C][Kh][H]; TMX_FAMILY_DENSE, in layer order (zero-filled before
+                            use): an act tensor [B][C][rank_p + rot_p] of every layer with a latent of its own, act
+                            tensors [B][Kh][C][dim_p], [B][Kh][C][vdim_p] of a layer with TMX_MIXER_HEADS */
   int sampling_mode;     /* TMX_SAMPLE_* */
   float temperature, top_p;
   int top_k;
@@ -475,7 +524,7 @@ typedef struct {
   int n_eos;
   const int32_t* forbidden;
   int n_forbidden;
-  float* logits_out;     /* optional f32 [B * tokens_per_pass, V] (TMX_FAMILY_LATENT: V rounded up to 32): logits of
+  float* logits_out;     /* optional f32 [B * tokens_per_pass, V] (TMX_FAMILY_DENSE: V rounded up to 32): logits of
                             the last executed pass */
   void* workspace;
   size_t workspace_bytes;
@@ -487,7 +536,7 @@ typedef struct {
                               attending to the slots up to its own column; *step advances by T.
                               Rows of a pass (batch * T, also for T <= 1): up to TMX_MAX_FILL_ROWS when
                               every projection has K % 128 == 0 (MoE models: rows * experts_per_tok <=
-                              TMX_MAX_MOE_PAIRS; TMX_FAMILY_LATENT: always), else 128.
+                              TMX_MAX_MOE_PAIRS; TMX_FAMILY_DENSE: always), else 128.
                               The workspace must be sized for batch * T rows. */
   int share_group;         /* 0 or 1: nothing is shared.  g > 1: the batch is made of consecutive groups of g
                               sequences whose cache slots [0, share_len) and input_mask entries are identical

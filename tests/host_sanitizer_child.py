@@ -14,7 +14,7 @@ import sys
 sys.path.insert(0, os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 
 from tunix_amd import _lib
-from tunix_amd.model import (DecodeState, DenseDesc, FAMILY_LATENT, LatentLayerDesc, LayerDesc, ModelDesc, QLinearDesc,
+from tunix_amd.model import (DecodeState, DenseDesc, FAMILY_DENSE, DenseLayerDesc, LayerDesc, ModelDesc, QLinearDesc,
                              StreamsDesc)
 
 FAKE = 0x1000  # a non-null "device pointer": never dereferenced on the host
@@ -61,8 +61,8 @@ def model_desc(family, layers, vocab, dm, f, n, kh, h, experts, per_tok, group, 
 
 
 def latent_desc(act, layers, vocab, d, ff, heads, dim_p, rot, rank, rank_p, vdim_p, streams):
-  """A TMX_FAMILY_LATENT model: every other layer reads the latents of the one before it."""
-  arr = (LatentLayerDesc * layers)()
+  """A TMX_FAMILY_DENSE model: every other layer reads the latents of the one before it."""
+  arr = (DenseLayerDesc * layers)()
   dp, rot_p = (d + 63) // 64 * 64, 64
   up32 = lambda v: (v + 31) // 32 * 32
   hc = StreamsDesc(FAKE, FAKE, FAKE)
@@ -71,7 +71,7 @@ def latent_desc(act, layers, vocab, d, ff, heads, dim_p, rot, rank, rank_p, vdim
     a.norm1_w = a.norm2_w = a.table = FAKE
     a.hc1 = a.hc2 = hc
     a.heads, a.rot_dim, a.kv_rank, a.dim_p, a.rot_p, a.rank_p, a.vdim_p = heads, rot, rank, dim_p, rot_p, rank_p, vdim_p
-    a.scale = 0.1
+    a.scale, a.ff = 0.1, 1
     a.off_qr = heads * dim_p
     n = a.off_qr + up32(heads * rot)
     a.off_kv = a.off_gate = -1
@@ -88,11 +88,53 @@ def latent_desc(act, layers, vocab, d, ff, heads, dim_p, rot, rank, rank_p, vdim
     if i != 1:
       a.gate_up, a.down = DenseDesc(FAKE, FAKE, dp, 2 * ff, 1), DenseDesc(FAKE, FAKE, ff, dp, 1)
   m = ModelDesc()
-  m.family, m.num_layers, m.vocab_size, m.embed_dim, m.norm_eps = FAMILY_LATENT, layers, vocab, d, 1e-5
+  m.family, m.num_layers, m.vocab_size, m.embed_dim, m.norm_eps = FAMILY_DENSE, layers, vocab, d, 1e-5
   m.embed = m.pos_embed = m.final_norm_w = m.head = m.final_in = FAKE
-  m.latent_layers = ctypes.cast(arr, ctypes.POINTER(LatentLayerDesc))
+  m.dense_layers = ctypes.cast(arr, ctypes.POINTER(DenseLayerDesc))
   m.act, m.streams, m.max_positions, m.logit_scale = act, streams, 64, 1.0
   return m, arr
+
+
+def heads_desc(act, layers, vocab, d, ff, heads, kv_heads, dim, dim_p, vdim_p, rot, chunk):
+  """A TMX_FAMILY_DENSE model of grouped attention with norms behind the sublayers; its second layer has no feed-forward."""
+  arr = (DenseLayerDesc * layers)()
+  dp = (d + 63) // 64 * 64
+  for i in range(layers):
+    a = arr[i]
+    a.norm1_w = a.norm2_w = a.table = a.sink = a.q_norm_w = a.k_norm_w = FAKE
+    a.mixer, a.ff, a.scale = 1, 3, 0.1
+    a.heads, a.kv_heads, a.dim, a.dim_p, a.vdim_p, a.rot_dim, a.chunk = heads, kv_heads, dim, dim_p, vdim_p, rot, chunk
+    a.in_ = DenseDesc(FAKE, FAKE, dp, heads * dim_p + kv_heads * (dim_p + vdim_p), 1)
+    a.o = DenseDesc(FAKE, None, heads * vdim_p, dp, 1)
+    if i != 1:
+      a.gate_up, a.down = DenseDesc(FAKE, None, dp, ff, 1), DenseDesc(FAKE, None, ff, dp, 1)
+  m = ModelDesc()
+  m.family, m.num_layers, m.vocab_size, m.embed_dim, m.norm_eps = FAMILY_DENSE, layers, vocab, d, 1e-5
+  m.embed = m.final_norm_w = m.head = FAKE
+  m.dense_layers = ctypes.cast(arr, ctypes.POINTER(DenseLayerDesc))
+  m.act, m.streams, m.max_positions, m.logit_scale, m.embed_scale, m.norm_after = act, 1, 64, 1.0, 2.0, 1
+  return m, arr
+
+
+def heads_plans(lib):
+  for shape in ((4, 1000, 200, 320, 6, 2, 50, 64, 128, 18, 7), (3, 128256, 4096, 14336, 32, 8, 128, 128, 128, 128, 8192)):
+    for act in (0, 1):
+      m, arr = heads_desc(act, *shape)
+      for batch in (1, 32, 129, 4096):
+        nb = lib.tmx_decode_workspace_bytes(ctypes.byref(m), batch, 640)
+        assert nb > 256, (shape, act, batch)
+        st = DecodeState()
+        st.batch, st.buf_len, st.cache_size = batch, 640, 640
+        st.token_buffer = st.positions = st.input_mask = st.done = st.step = st.kv_cache = st.workspace = FAKE
+        st.workspace_bytes = nb - 1
+        assert lib.tmx_decode_steps(ctypes.byref(m), ctypes.byref(st), None, 1, 1) == -2
+      arr[1].kv_heads = 5  # does not divide the query heads
+      assert lib.tmx_decode_workspace_bytes(ctypes.byref(m), 1, 640) == 0
+      assert lib.tmx_decode_steps(ctypes.byref(m), ctypes.byref(st), None, 1, 1) == -2
+  for n_seq in (1, 64, 4096):
+    for t in (1, 7, 128):
+      for h, kh in ((1, 1), (32, 8), (96, 1)):
+        lib.tmx_head_attention_workspace_bytes(n_seq, t, h, kh, 256, 4096, 1000)
 
 
 def latent_plans(lib):
@@ -155,6 +197,7 @@ def main():
       lib.tmx_head_sample_workspace_bytes(b, c[2])
       lib.tmx_nucleus_workspace_bytes(b, c[2])
   latent_plans(lib)
+  heads_plans(lib)
   assert lib.tmx_int4_dequant(None, None, None, None, 64, 32, 64) == -1
   assert lib.tmx_int4_dequant(None, FAKE, FAKE, FAKE, 65, 32, 64) == -2
   assert lib.tmx_qlora_linear_planes(None, FAKE, FAKE, FAKE, None, FAKE, None, 4, 100, 32, 64, 0, 1) == -2

@@ -9,7 +9,7 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.environ.get('TMX_LIB', os.path.join(_HERE, 'libtmx.so'))
 
 _lib = None
-ABI_VERSION = 8  # TMX_ABI_VERSION of include/tmx.h
+ABI_VERSION = 9  # TMX_ABI_VERSION of include/tmx.h
 
 vp, ci, cf, cu32 = ctypes.c_void_p, ctypes.c_int, ctypes.c_float, ctypes.c_uint32
 
@@ -46,6 +46,9 @@ SIGNATURES = {
     'tmx_moe_experts': [vp, vp, ci, vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, vp, ci],
     'tmx_dense_linear': [vp, ci, vp, ci, ci, vp, vp, vp, ci, vp, ci, ci, ci, ci, ci, ci, ci],
     'tmx_stream_rows': [vp, ci, vp, vp, vp, vp, vp, vp, vp, ci, ci, ci, ci, cf, ci],
+    'tmx_residual_rows': [vp, ci, vp, vp, vp, vp, vp, ci, ci, ci, cf, ci],
+    'tmx_head_rows': [vp, ci, vp, ci, vp, vp, cf, vp, ci, vp, vp, vp, ci, vp, vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, ci],
+    'tmx_head_attention': [vp, ci, vp, vp, vp, vp, vp, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, cf],
     'tmx_latent_rows': [vp, ci, vp, ci, ci, ci, vp, cf, vp, ci, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci],
     'tmx_latent_attention': [vp, ci, vp, vp, vp, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, cf],
     'tmx_decode_steps': [vp, vp, vp, ci, ci],
@@ -64,6 +67,7 @@ SIZE_FUNCS = {
     'tmx_qlora_linear_delta_workspace_bytes': [ci, ci, ci, ci, ci, ci],
     'tmx_decode_workspace_bytes': [vp, ci, ci],
     'tmx_latent_attention_workspace_bytes': [ci, ci, ci, ci, ci],
+    'tmx_head_attention_workspace_bytes': [ci, ci, ci, ci, ci, ci, ci],
     'tmx_qlora_gate_up_swiglu_handover_bytes': [ci, ci, ci, ci],
 }
 

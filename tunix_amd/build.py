@@ -16,9 +16,9 @@ HIPCC_FLAGS = [
     '-Xclang', '-target-feature', '-Xclang', '-packed-fp32-ops',
 ]
 
-# per source: the walk over latent cache rows keeps its accumulators in ordinary registers (in accumulation registers
+# per source: the walks of latent and grouped attention keep their accumulators in ordinary registers (in accumulation registers
 # they would be copied out and back around every rescaling)
-EXTRA_FLAGS = {'latent.hip': ['-mllvm', '-amdgpu-mfma-vgpr-form=1']}
+EXTRA_FLAGS = {f: ['-mllvm', '-amdgpu-mfma-vgpr-form=1'] for f in ('latent.hip', 'heads.hip')}
 
 
 def sources():

@@ -142,7 +142,7 @@ using namespace tmx;
 
 extern "C" size_t tmx_decode_workspace_bytes(const tmx_model_desc* m, int batch, int cache_size) {
   if (!m || batch <= 0) return 0;
-  if (m->family == TMX_FAMILY_LATENT) return latent_check(m) == TMX_OK ? latent_carve(m, batch, nullptr).total : 0;
+  if (m->family == TMX_FAMILY_DENSE) return dense_check(m) == TMX_OK ? dense_carve(m, batch, nullptr).total : 0;
   return carve(m, batch, cache_size, nullptr).total;
 }
 
@@ -152,9 +152,9 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
   if (!s->token_buffer || !s->positions || !s->input_mask || !s->done || !s->step || !s->kv_cache ||
       !s->workspace)
     return TMX_ERR_ARG;
-  const bool latent = m->family == TMX_FAMILY_LATENT;
-  if (!latent && !m->layers) return TMX_ERR_ARG;
-  int rc = latent ? latent_check(m) : TMX_OK;
+  const bool dense = m->family == TMX_FAMILY_DENSE;
+  if (!dense && !m->layers) return TMX_ERR_ARG;
+  int rc = dense ? dense_check(m) : TMX_OK;
   if (rc != TMX_OK) return rc;
   const bool moe = m->num_experts > 0;
   // rows of a pass: one per sequence, or tokens_per_pass consecutive tokens of every sequence
@@ -174,8 +174,8 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
   if (nucleus && !s->nucleus_workspace) return TMX_ERR_ARG;
   const int D = m->embed_dim, N = m->num_heads, Kh = m->num_kv_heads, H = m->head_dim;
   const int F = m->hidden_dim, NH = N * H, QKV = (N + 2 * Kh) * H;
-  if ((latent ? latent_carve(m, B, nullptr).total : carve(m, B, C, nullptr).total) > s->workspace_bytes) return TMX_ERR_SHAPE;
-  for (int i = 0; !latent && i < m->num_layers; ++i) {
+  if ((dense ? dense_carve(m, B, nullptr).total : carve(m, B, C, nullptr).total) > s->workspace_bytes) return TMX_ERR_SHAPE;
+  for (int i = 0; !dense && i < m->num_layers; ++i) {
     const tmx_layer_desc& l = m->layers[i];
     if (!l.norm1_w || !l.norm2_w) return TMX_ERR_ARG;
     if ((rc = check_linear(l.qkv, D, QKV)) || (rc = check_linear(l.o, NH, D))) return rc;
@@ -186,13 +186,13 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
     if ((rc = check_linear(l.gate_up, D, 2 * F)) || (rc = check_linear(l.down, F, D))) return rc;
   }
   hipStream_t st = (hipStream_t)stream;
-  const LatentWorkspace lw = latent ? latent_carve(m, B, (char*)s->workspace) : LatentWorkspace();
-  const Workspace w = latent ? Workspace() : carve(m, B, C, (char*)s->workspace);
+  const DenseWorkspace lw = dense ? dense_carve(m, B, (char*)s->workspace) : DenseWorkspace();
+  const Workspace w = dense ? Workspace() : carve(m, B, C, (char*)s->workspace);
   const size_t kv_elems = (size_t)NSEQ * C * Kh * H;
   const float theta = m->family == TMX_FAMILY_LLAMA3 ? 1000000.0f : m->rope_theta;
 
-  const Splits sp = latent ? Splits() : plan_splits(m, B);
-  const bool small = !latent && small_batch_ok(m, B, T);
+  const Splits sp = dense ? Splits() : plan_splits(m, B);
+  const bool small = !dense && small_batch_ok(m, B, T);
   auto lora_of = [&](const tmx_qlinear_desc& l, int) {
     LoraIn li = {};
     if (l.lora_a_t) {
@@ -231,15 +231,15 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
                              w.y16, w.t_part, w.t16, B, l.K, l.N, l.G, l.r_pad);
   };
   // the hand-over words of the fused gate | up launch start at zero (the kernel leaves them so)
-  if (!latent && !moe && B <= kFusedGateUpMaxRows && w.gu_sync && n_steps > 0) {
+  if (!dense && !moe && B <= kFusedGateUpMaxRows && w.gu_sync && n_steps > 0) {
     rc = zero_words(st, (uint32_t*)w.gu_sync, 64);
     if (rc != TMX_OK) return rc;
   }
   // samples of one prompt in consecutive rows: decode attention reads the prompt slots once per group
   const bool share_walk = T == 1 && !small && w.attn_partial && attn_share_ok(B, N, Kh, H, C, s->share_group, s->share_len);
   for (int it = 0; it < n_steps; ++it) {
-    if (latent) {
-      rc = latent_layers(st, m, s, lw, NSEQ, T, sample != 0, prof);
+    if (dense) {
+      rc = dense_layers(st, m, s, lw, NSEQ, T, sample != 0, prof);
       if (rc != TMX_OK) return rc;
     } else {  // embedding gather + first input norm + this step's RoPE table
       RowNormArgs a = {};
@@ -329,7 +329,7 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
         if (sample) TMX_TRY(TMX_K_ROWNORM, row_norm(st, a, B));
       }
     }
-    for (int i = 0; !small && !latent && i < m->num_layers; ++i) {
+    for (int i = 0; !small && !dense && i < m->num_layers; ++i) {
       const tmx_layer_desc& l = m->layers[i];
       // gate | up with LoRA + SwiGLU in its epilogue: K % 256 == 0 below 8192, unsplit, 2 r <= 32
       const bool fused_gu = !moe && B <= kFusedGateUpMaxRows && sp.gate_up == 1 && D % 256 == 0 && D < 8192 && F % 64 == 0 &&
@@ -495,16 +495,16 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
     }
     if (sample) {
       HeadArgs a = {};
-      a.x = (const uint16_t*)(latent ? lw.xn : w.xn);
+      a.x = (const uint16_t*)(dense ? lw.xn : w.xn);
       a.w = (const uint16_t*)m->head;
       a.M = B;
-      a.D = latent ? pad_to(D, 64) : D;
-      a.V = latent ? pad_to(m->vocab_size, 32) : m->vocab_size;
+      a.D = dense ? pad_to(D, 64) : D;
+      a.V = dense ? pad_to(m->vocab_size, 32) : m->vocab_size;
       a.mode = s->sampling_mode;
       a.temperature = s->temperature;
       a.k0 = s->seed_hi; a.k1 = s->seed_lo;
       a.step = s->step;
-      void* partial = latent ? lw.head_partial : w.head_partial;
+      void* partial = dense ? lw.head_partial : w.head_partial;
       a.part_f = (float*)partial;
       a.token_buffer = s->token_buffer;
       a.logprobs = s->logprobs;
@@ -512,11 +512,11 @@ static int decode_steps_impl(const tmx_model_desc* m, const tmx_decode_state* s,
       a.eos = s->eos_ids; a.n_eos = s->n_eos;
       a.buf_len = L;
       a.tpp = T;
-      if (latent) {
+      if (dense) {
         a.v_live = m->vocab_size;
         a.logit_scale = m->logit_scale;
       }
-      if (latent && m->act == TMX_ACT_F32) {
+      if (dense && m->act == TMX_ACT_F32) {
         // the products in f32 first; selection then reads them from memory
         DenseArgs d = {};
         d.x = lw.xn; d.ldx = a.D; d.w = m->head;

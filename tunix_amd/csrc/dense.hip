@@ -4,7 +4,7 @@
 // lanes of a wave feed them to v_mfma_f32_32x32x16_bf16), so every weight load is 1 KiB of consecutive bytes.
 //   up to 128 rows  dense_small_kernel: a weight stream; the waves of a workgroup share 32 (or 2 x 32) output columns
 //                   and split K between them, meeting once in LDS, so there are no partial planes in memory and the
-//                   epilogue (bias, SwiGLU, sigmoid gate) runs on the finished sums
+//                   epilogue (bias, SwiGLU, sigmoid gate, squared relu) runs on the finished sums
 //   more rows       dense_wide_kernel: 256 rows x 32 MT columns per workgroup; the weight slab of a k-step goes
 //                   global -> LDS by direct loads, the activations are the B operand straight from memory
 // f32: dense_f32_kernel, a plain tiled product on the vector ALU (no matrix pipe, no reduced precision).
@@ -14,6 +14,7 @@ namespace tmx {
 
 __device__ __forceinline__ float silu(float z) { return z / (1.f + expf(-z)); }
 __device__ __forceinline__ float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
+__device__ __forceinline__ float relu2(float z) { z = fmaxf(z, 0.f); return z * z; }
 
 // MT: 32-row tiles of x; WK: waves that share K (8 / WK column tiles per workgroup); NT = 2: SwiGLU pairs (a gate
 // tile and the up tile N / 64 tiles further).
@@ -109,6 +110,7 @@ __device__ __forceinline__ void dense_small_block(const DenseArgs& a, int bx, in
       return;
     }
     if (NT == 2) v = silu(v) * (s[NT - 1] + b1);
+    if (NT == 1 && a.epi == TMX_DENSE_RELU2) v = relu2(v);
     if (a.epi == TMX_DENSE_GATED && row < a.M && tile < tiles)
       v *= sigmoid(bf2f(reinterpret_cast<const uint16_t*>(a.gate)[(size_t)row * a.ldg + head * a.y_head + col]));
     out_s[row * OW + wn * 32 + nl] = f2bf(v);
@@ -299,6 +301,10 @@ __global__ __launch_bounds__(512, 1) void dense_wide_kernel(DenseArgs a, int row
       *reinterpret_cast<f32x4_t*>(a.y_part + ((size_t)slice * a.M + row) * a.N + col) = f32x4_t{v[0], v[1], v[2], v[3]};
       return;
     }
+    if (a.epi == TMX_DENSE_RELU2) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = relu2(v[e]);
+    }
     if (grow) {
       const uint2 g = *reinterpret_cast<const uint2*>(grow + col);
       v[0] *= sigmoid(bf_lo(g.x)); v[1] *= sigmoid(bf_hi(g.x));
@@ -358,6 +364,7 @@ __global__ __launch_bounds__(256) void dense_f32_kernel(DenseArgs a) {
       if (row >= a.M || col >= cols) continue;
       float v = acc[0][i][j] + (a.bias ? a.bias[col] : 0.f);
       if (SWIGLU) v = silu(v) * (acc[NT - 1][i][j] + (a.bias ? a.bias[cols + col] : 0.f));
+      if (a.epi == TMX_DENSE_RELU2) v = relu2(v);
       if (a.epi == TMX_DENSE_GATED)
         v *= sigmoid(reinterpret_cast<const float*>(a.gate)[(size_t)row * a.ldg + head * a.y_head + col]);
       reinterpret_cast<float*>(a.y)[(size_t)row * a.ldy + head * a.y_head + col] = v;
@@ -486,7 +493,7 @@ extern "C" int tmx_dense_linear(void* stream, int act, const void* x, int ldx, i
                                 const float* bias, const void* gate, int ldg, void* y, int ldy, int y_head, int M,
                                 int K, int N, int heads, int epilogue) {
   if (!x || !w || !y || (epilogue == TMX_DENSE_GATED && !gate)) return TMX_ERR_ARG;
-  if (epilogue != TMX_DENSE_PLAIN && epilogue != TMX_DENSE_SWIGLU && epilogue != TMX_DENSE_GATED) return TMX_ERR_UNSUPPORTED;
+  if (epilogue < TMX_DENSE_PLAIN || epilogue > TMX_DENSE_RELU2) return TMX_ERR_UNSUPPORTED;
   DenseArgs a = {};
   a.x = x; a.ldx = ldx; a.x_head = x_head;
   a.w = w; a.bias = bias; a.gate = gate; a.ldg = ldg;

@@ -29,20 +29,21 @@ struct Prof {
     if (rc != TMX_OK) return rc;       \
   }
 
-// TMX_FAMILY_LATENT: workspace of a pass of `rows` rows (the first 256 bytes are the status block of every family).
-struct LatentWorkspace {
+// TMX_FAMILY_DENSE: workspace of a pass of `rows` rows (the first 256 bytes are the status block of every family).
+struct DenseWorkspace {
   float* xs;            // residual streams [rows][S][Dp]
   void *xn, *z, *q, *lat, *val, *y, *act;
+  int32_t* first;       // first slot every row sees (TMX_MIXER_HEADS)
   float* attn_partial;
   float* y_part;        // f32 planes of a projection whose K is split [nsplit][rows][Dp]
   float* logits;        // f32 models: products of the head [rows][Vp]
   void* head_partial;
   size_t total;
 };
-LatentWorkspace latent_carve(const tmx_model_desc* m, int rows, char* base);
-int latent_check(const tmx_model_desc* m);
+DenseWorkspace dense_carve(const tmx_model_desc* m, int rows, char* base);
+int dense_check(const tmx_model_desc* m);
 // Embedding and every layer of one pass; with final_norm w.xn is the head's input afterwards.
-int latent_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_state* s, const LatentWorkspace& w,
+int dense_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_state* s, const DenseWorkspace& w,
                   int n_seq, int T, bool final_norm, Prof* prof);
 inline int pad_to(int v, int k) { return (v + k - 1) / k * k; }
 

@@ -299,7 +299,7 @@ __host__ __device__ inline size_t act_tile_off(int row, int col, int cols) {
 }
 
 // Mixing of the residual streams + the next sublayer's norm, see tmx_stream_rows; with `embed` set the streams are
-// first filled with embed[token] + pos_embed[position] of every row.
+// first filled with embed_scale * embed[token] + pos_embed[position] of every row.
 struct StreamArgs {
   float* xs;           // [M][S][Dp]
   const void* y;       // act [M][Dp] or null
@@ -311,6 +311,7 @@ struct StreamArgs {
   int S, D, Dp, store;
   float eps;
   const uint16_t* embed;      // bf16 [vocab, Dp]
+  float embed_scale;
   const uint16_t* pos_embed;  // bf16 [max_positions, Dp] or null
   int vocab, max_positions;
   const int32_t* token_buffer;
@@ -346,6 +347,62 @@ struct LatentAttnArgs {  // see tmx_latent_attention
   int n_seq, tpp, H, rank_p, rot_p, C, nsplit;
   float scale;
 };
+
+// One residual stream with a norm behind and / or in front of the sublayers, see tmx_residual_rows; with `embed` set x is
+// first filled with embed_scale * embed[token] of every row.
+struct ResidualArgs {
+  float* x;            // [M][Dp]
+  const void* y;       // act [M][Dp] or null
+  const float* y_part; // instead of y: f32 planes [nsplit][M][Dp], added in order
+  int nsplit;
+  const float *post_w, *norm_w;
+  void* xn;
+  bool xn_tiled;       // xn in the order of act_tile_off
+  int D, Dp, store;
+  float eps;
+  const uint16_t* embed;  // bf16 [vocab, Dp]
+  float embed_scale;
+  int vocab;
+  const int32_t* token_buffer;
+  const int32_t* step;
+  int buf_len, tpp;
+};
+
+struct HeadRowsArgs {  // see tmx_head_rows
+  const void* z;
+  int ldz;
+  const float *q_norm_w, *k_norm_w;
+  float eps;
+  const float* table;
+  int max_positions;
+  const int32_t* positions;
+  const uint8_t* input_mask;
+  const int32_t* step;
+  int buf_len, tpp;
+  void *q, *kcache, *vcache;
+  int32_t* first;
+  int H, Kh, dim, dk, dv, rot, C, chunk;
+};
+
+struct HeadAttnArgs {  // see tmx_head_attention
+  const void *q, *kcache, *vcache;
+  const float* sink;
+  const int32_t* first;
+  const uint8_t* input_mask;
+  const int32_t* step;
+  int buf_len;
+  void* out;
+  bool out_tiled;  // out in the order of act_tile_off (H dv columns)
+  float* partial;  // [rows H][nsplit][dv + 4]: values, maximum, sum
+  int n_seq, tpp, H, Kh, dk, dv, C, chunk, nsplit;
+  float scale;
+};
+
+int residual_rows(hipStream_t st, int act, const ResidualArgs& a, int M);
+int head_rows(hipStream_t st, int act, const HeadRowsArgs& a, int M);
+int head_attention(hipStream_t st, int act, HeadAttnArgs a);
+bool head_attn_ok(int dk, int dv);
+size_t head_attn_partial_bytes(int rows, int H, int dv);  // room for every split of `rows` query rows
 
 int dense_linear(hipStream_t st, int act, const DenseArgs& a);
 int dense_num_splits(int act, int M, int K, int N);  // slices of K worth their planes for a projection into the streams

@@ -14,7 +14,7 @@ import torch
 from tunix_amd import quant
 from tunix_amd import _lib
 
-FAMILY_LLAMA3, FAMILY_QWEN3, FAMILY_LATENT = 0, 1, 2
+FAMILY_LLAMA3, FAMILY_QWEN3, FAMILY_DENSE = 0, 1, 2
 SAMPLE_GREEDY, SAMPLE_TOP_P, SAMPLE_SCORE = 0, 1, 2
 MAX_RPAD = 128
 
@@ -123,14 +123,16 @@ class StreamsDesc(ctypes.Structure):
   _fields_ = [('in_', ctypes.c_void_p), ('out', ctypes.c_void_p), ('mix', ctypes.c_void_p)]
 
 
-class LatentLayerDesc(ctypes.Structure):
+class DenseLayerDesc(ctypes.Structure):
   _fields_ = [('norm1_w', ctypes.c_void_p), ('norm2_w', ctypes.c_void_p), ('hc1', StreamsDesc), ('hc2', StreamsDesc),
               ('heads', ctypes.c_int), ('rot_dim', ctypes.c_int), ('kv_rank', ctypes.c_int), ('dim_p', ctypes.c_int),
               ('rot_p', ctypes.c_int), ('rank_p', ctypes.c_int), ('vdim_p', ctypes.c_int), ('off_qr', ctypes.c_int),
               ('off_kv', ctypes.c_int), ('off_gate', ctypes.c_int), ('kv_layer', ctypes.c_int),
               ('scale', ctypes.c_float), ('in_', DenseDesc), ('uk', DenseDesc), ('uv', DenseDesc), ('o', DenseDesc),
               ('kv_norm_w', ctypes.c_void_p), ('table', ctypes.c_void_p), ('sink', ctypes.c_void_p),
-              ('gate_up', DenseDesc), ('down', DenseDesc)]
+              ('gate_up', DenseDesc), ('down', DenseDesc), ('ff', ctypes.c_int), ('mixer', ctypes.c_int),
+              ('kv_heads', ctypes.c_int), ('dim', ctypes.c_int), ('chunk', ctypes.c_int), ('q_norm_w', ctypes.c_void_p),
+              ('k_norm_w', ctypes.c_void_p)]
 
 
 class ModelDesc(ctypes.Structure):
@@ -140,9 +142,9 @@ class ModelDesc(ctypes.Structure):
               ('experts_per_tok', ctypes.c_int), ('rope_theta', ctypes.c_float),
               ('norm_eps', ctypes.c_float), ('embed', ctypes.c_void_p), ('final_norm_w', ctypes.c_void_p),
               ('head', ctypes.c_void_p), ('layers', ctypes.POINTER(LayerDesc)), ('head_tiles', ctypes.c_void_p),
-              ('latent_layers', ctypes.POINTER(LatentLayerDesc)), ('act', ctypes.c_int), ('streams', ctypes.c_int),
+              ('dense_layers', ctypes.POINTER(DenseLayerDesc)), ('act', ctypes.c_int), ('streams', ctypes.c_int),
               ('max_positions', ctypes.c_int), ('pos_embed', ctypes.c_void_p), ('final_in', ctypes.c_void_p),
-              ('logit_scale', ctypes.c_float)]
+              ('logit_scale', ctypes.c_float), ('embed_scale', ctypes.c_float), ('norm_after', ctypes.c_int)]
 
 
 class DecodeState(ctypes.Structure):
@@ -424,6 +426,9 @@ class QLoRAModel:
     d.layers = ctypes.cast(arr, ctypes.POINTER(LayerDesc))
     self._desc, self._keep = d, arr
     return d
+
+  def reserve_positions(self, n):
+    del n  # rotations are computed from the position: no table to extend
 
   def expert_fraction(self, batch):
     """Expected fraction of a layer's experts that a step of `batch` tokens touches under

@@ -11,6 +11,7 @@ from typing import Callable, NamedTuple
 import torch
 
 from tunix_amd import checkpoint
+from tunix_amd.grouped import GroupedConfig, GroupedModel
 from tunix_amd.latent import LatentConfig, LatentModel
 from tunix_amd.model import ModelConfig
 
@@ -40,8 +41,8 @@ def read_tensors(folder):
   return out
 
 
-def _load_latent(folder, config, device):
-  return LatentModel.from_state(config, read_tensors(folder), device=device)
+def _load_dense(model):
+  return lambda folder, config, device: model.from_state(config, read_tensors(folder), device=device)
 
 
 def _hf_config(family):
@@ -63,7 +64,8 @@ def _load_quantised(folder, config, device, **options):
 
 
 ARCHITECTURES = {
-    'Kagapel': Entry(('bfloat16', 'float32'), LatentConfig.from_dict, _load_latent),
+    'Feduzen': Entry(('bfloat16', 'float32'), GroupedConfig.from_dict, _load_dense(GroupedModel)),
+    'Kagapel': Entry(('bfloat16', 'float32'), LatentConfig.from_dict, _load_dense(LatentModel)),
     'LlamaForCausalLM': Entry(('bfloat16',), _hf_config('llama3'), _load_quantised),
     'Qwen3ForCausalLM': Entry(('bfloat16',), _hf_config('qwen3'), _load_quantised),
     'Qwen3MoeForCausalLM': Entry(('bfloat16',), _hf_config('qwen3'), _load_quantised),

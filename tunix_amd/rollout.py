@@ -52,9 +52,9 @@ class TmxRollout(BaseRollout):
 
   @staticmethod
   def _as_policy(actor, group, lora_alpha, quant_bound):
-    from tunix_amd.latent import LatentConfig
+    from tunix_amd.dense import DenseConfig
     from tunix_amd.model import ModelConfig, QLoRAModel
-    if isinstance(actor, QLoRAModel) or isinstance(getattr(actor, 'config', None), (ModelConfig, LatentConfig)):
+    if isinstance(actor, QLoRAModel) or isinstance(getattr(actor, 'config', None), (ModelConfig, DenseConfig)):
       return actor  # already a policy of this package (its config is this package's ModelConfig)
     if isinstance(actor, tuple) and len(actor) == 2:
       cfg, tree = actor

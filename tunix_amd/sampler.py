@@ -214,6 +214,7 @@ class Sampler:
     positions = utils.build_positions_from_mask(input_mask)
     share = shared_prompt_groups(ids, input_mask[:, :p]) if self.share_prompt_kv else (1, 0, 0)
     c = self._transformer.config
+    self._transformer.reserve_positions(total_sampling_steps)
     need = c.cache_shape(b, self.cache_config.cache_size)
     if self._cache is None or tuple(self._cache.shape) != need:
       self._cache = None
