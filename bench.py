@@ -47,6 +47,13 @@ LATENT_SIZES = {
     '4k': (4096, 14336, 32, 128, 64, 128, 512, 4, 8, 128256),
     '4k-r256': (4096, 14336, 32, 64, 32, 64, 256, 2, 8, 128256),
 }
+# --grouped: the same for the dense design of chunked grouped-query attention:
+# (width, ff, heads, kv_heads, dim, vdim, chunk, layers, vocab)
+GROUPED_SIZES = {
+    '2k': (2048, 8192, 32, 8, 64, 64, 8192, 8, 128256),
+    '4k': (4096, 14336, 32, 8, 128, 128, 8192, 8, 128256),
+    '4k-c256': (4096, 14336, 32, 8, 128, 128, 256, 8, 128256),
+}
 
 
 def linear_bytes(pl, batch, frac=1.0):
@@ -130,12 +137,25 @@ def class_work(model, rows, keys, decode):
   c = model.config
   out = {}
   layer = model.layers[0]
+  def dense(k, n_out, heads=1):
+    return 2.0 * heads * k * n_out + 2.0 * rows * heads * (k + n_out), 2.0 * rows * heads * k * n_out
+  if hasattr(c, 'embed_scale'):
+    l = c.layers[0]
+    qk, v = (l.heads + l.kv_heads) * l.dim, l.kv_heads * l.vdim
+    out['row_norm'] = (rows * c.embed_dim * (2 * 4 + 4), rows * c.embed_dim * 6)
+    out['qkv_linear'] = dense(c.embed_dim, qk + v)
+    out['rope_kvwrite'] = (rows * 4.0 * (qk + v), 0)
+    kv = 2.0 * l.kv_heads * (l.dim + l.vdim)
+    out['attention'] = ((rows * keys if decode else keys) * kv + rows * 2.0 * l.heads * (l.dim + l.vdim),
+                        2.0 * rows * keys * l.heads * (l.dim + l.vdim))
+    out['o_linear'] = dense(l.heads * l.vdim, c.embed_dim)
+    out['gate_up_linear'], out['down_linear'] = dense(c.embed_dim, l.ff), dense(l.ff, c.embed_dim)
+    out['head_sample'] = (2.0 * c.vocab_size * c.embed_dim, 2.0 * rows * c.vocab_size * c.embed_dim)
+    return out
   if hasattr(c, 'layers'):
     l = c.layers[0]
     n = c.streams
     out['row_norm'] = (rows * c.embed_dim * (2 * n * 4 + 4), rows * c.embed_dim * 2 * n * (n + 2))
-    def dense(k, n_out, heads=1):
-      return 2.0 * heads * k * n_out + 2.0 * rows * heads * (k + n_out), 2.0 * rows * heads * k * n_out
     own = l.heads * (l.dim + l.rot_dim) + l.kv_rank + l.rot_dim + (l.heads * l.vdim if l.gate else 0)
     width = l.kv_rank + l.rot_dim
     out['qkv_linear'] = dense(c.embed_dim, own)
@@ -163,17 +183,25 @@ def class_work(model, rows, keys, decode):
   return out
 
 
-def latent_bench(size, batches, prompt, steps):
-  """Prefill and decode throughput of the latent-attention design beside the closest quantised model, with the
+def dense_bench(design, size, batches, prompt, steps):
+  """Prefill and decode throughput of a dense design ('kagapel', 'feduzen') beside the closest quantised model, with the
   distance of every launch class from its roofline (measured event time over the larger of bytes / 8 TB/s and
   flops / 2.5 PFLOP/s).  Prints one JSON line."""
   import torch
   from tunix_amd import _lib
   from tunix_amd.configs import CacheConfig
+  from tunix_amd.grouped import GroupedConfig, GroupedModel
   from tunix_amd.latent import LatentConfig, LatentModel
   from tunix_amd.model import ModelConfig, QLoRAModel
   from tunix_amd.sampler import Sampler
-  d, ff, heads, dim, rot, vdim, rank, streams, layers, vocab = LATENT_SIZES[size]
+  if design == 'kagapel':
+    d, ff, heads, dim, rot, vdim, rank, streams, layers, vocab = LATENT_SIZES[size]
+    like, chunk = (d // 128, 128, 8), None
+    sizes = {'rot_dim': rot, 'kv_rank': rank, 'streams': streams}
+  else:
+    d, ff, heads, kv_heads, dim, vdim, chunk, layers, vocab = GROUPED_SIZES[size]
+    like = (heads, dim, kv_heads)
+    sizes = {'kv_heads': kv_heads, 'chunk': chunk}
   torch.cuda.set_device(0)
   lib = _lib.lib()
   rng = np.random.default_rng(0)
@@ -181,7 +209,9 @@ def latent_bench(size, batches, prompt, steps):
   def build(kind):
     if kind == 'kagapel':
       return LatentModel.random_init(LatentConfig.uniform(layers, vocab, d, ff, heads, dim, rot, vdim, rank, streams))
-    cfg = ModelConfig('llama3', layers, vocab, d, ff, d // 128, 128, 8, 500_000, 1e-5, False)
+    if kind == 'feduzen':
+      return GroupedModel.random_init(GroupedConfig.uniform(layers, vocab, d, ff, heads, kv_heads, dim, vdim, chunk))
+    cfg = ModelConfig('llama3', layers, vocab, d, ff, *like, 500_000, 1e-5, False)
     return QLoRAModel.random_init(cfg, seed=0, group=64, lora_rank=16, lora_alpha=32.0)
 
   def profiled(s, st, t, n, sample):
@@ -207,11 +237,18 @@ def latent_bench(size, batches, prompt, steps):
                 'frac': round(bound / sec, 4)}
     return out
 
-  result = {'metric': f'prefill and decode tokens/s, latent-attention design, {size} layers', 'unit': 'tokens/s',
+  label = 'latent-attention' if design == 'kagapel' else 'chunked grouped-attention'
+  result = {'metric': f'prefill and decode tokens/s, {label} design, {size} layers', 'unit': 'tokens/s',
             'n_gpus': 1, 'higher_is_better': True, 'data': 'synthetic (random-init weights, uniform-random token ids)',
-            'config': {'width': d, 'ff': ff, 'heads': heads, 'dim': dim, 'rot_dim': rot, 'vdim': vdim, 'kv_rank': rank,
-                       'streams': streams, 'layers': layers, 'vocab': vocab, 'prompt': prompt, 'decode_steps': steps}}
-  for kind in ('kagapel', 'llama3-int4'):
+            'config': {'width': d, 'ff': ff, 'heads': heads, 'dim': dim, 'vdim': vdim, **sizes, 'layers': layers,
+                       'vocab': vocab, 'prompt': prompt, 'decode_steps': steps}}
+
+  def seen(kind, first, n):
+    """Slots the n tokens from position `first` on see on average."""
+    size = chunk if kind == 'feduzen' and chunk else first + n
+    return float(np.mean(np.arange(first, first + n) % size + 1))
+
+  for kind in (design, 'llama3-int4'):
     model = build(kind)
     c = model.config
     total = prompt + steps + 40
@@ -240,14 +277,14 @@ def latent_bench(size, batches, prompt, steps):
       r = {'prefill_tokens_per_s': round(b * (prompt - 1) / fill), 'prefill_ms': round(fill * 1e3, 3),
            'decode_tokens_per_s': round(b * steps / dec), 'decode_ms_per_step': round(dec / steps * 1e3, 4)}
       ctx = int(st['step'].item()) + 4
-      r['decode_kernels'] = distances(profiled(s, st, 1, 8, 1), class_work(model, b, ctx, True))
+      r['decode_kernels'] = distances(profiled(s, st, 1, 8, 1), class_work(model, b, seen(kind, ctx - 4, 8), True))
       # one pass of the prompt walk, its tokens in the middle of the prompt
       per = min(128, max(1, s._fill_rows() // b), prompt // 2)
       st = fresh()
       s.walk(st, prompt // 2)
-      work = class_work(model, b * per, prompt // 2 + per / 2.0, False)
+      work = class_work(model, b * per, seen(kind, prompt // 2, per), False)
       by, fl = work['attention']
-      kb = (prompt // 2 + per) * (c.cache_bytes_per_token() / c.num_layers if hasattr(c, 'layers') else c.num_kv_heads * c.head_dim * 4.0)
+      kb = (min(prompt // 2, (chunk or prompt) if kind == 'feduzen' else prompt) + per) * (c.cache_bytes_per_token() / c.num_layers if hasattr(c, 'layers') else c.num_kv_heads * c.head_dim * 4.0)
       work['attention'] = (b * kb, fl)
       r['prefill_kernels'] = distances(profiled(s, st, per, 1, 0), work)
       r['prefill_rows_per_pass'] = b * per
@@ -255,12 +292,12 @@ def latent_bench(size, batches, prompt, steps):
     result[kind] = rec
     del model, s, st
     torch.cuda.empty_cache()
-  result['value'] = result['kagapel'][f'batch_{batches[-1]}']['decode_tokens_per_s']
+  result['value'] = result[design][f'batch_{batches[-1]}']['decode_tokens_per_s']
   # how much farther from its roofline a launch class of the design is than the like class of the closest model
   rel = {}
   for b in batches:
     for phase in ('decode_kernels', 'prefill_kernels'):
-      new, old = (result[k][f'batch_{b}'][phase] for k in ('kagapel', 'llama3-int4'))
+      new, old = (result[k][f'batch_{b}'][phase] for k in (design, 'llama3-int4'))
       for k, v in new.items():
         like = {'latent_q': 'o_linear', 'latent_v': 'o_linear'}.get(k, k)
         if like in old:
@@ -313,11 +350,15 @@ def main():
   ap.add_argument('--latent', choices=sorted(LATENT_SIZES), default=None,
                   help='prefill and decode throughput of the latent-attention design at this size beside the closest '
                        'quantised model: a separate JSON line, not the headline metric')
-  ap.add_argument('--latent-batches', type=int, nargs='+', default=[1, 16, 64])
-  ap.add_argument('--latent-prompt', type=int, default=512, help='--latent: prompt tokens in front of the decoding')
+  ap.add_argument('--grouped', choices=sorted(GROUPED_SIZES), default=None,
+                  help='the same for the chunked grouped-attention design')
+  ap.add_argument('--dense-batches', '--latent-batches', type=int, nargs='+', default=[1, 16, 64])
+  ap.add_argument('--dense-prompt', '--latent-prompt', type=int, default=512,
+                  help='--latent, --grouped: prompt tokens in front of the decoding')
   args = ap.parse_args()
-  if args.latent:
-    latent_bench(args.latent, args.latent_batches, args.latent_prompt, min(args.steps, 64))
+  if args.latent or args.grouped:
+    dense_bench('kagapel' if args.latent else 'feduzen', args.latent or args.grouped, args.dense_batches, args.dense_prompt,
+                min(args.steps, 64))
     return
   if args.pmc_summary:
     pmc_summary(args.pmc_summary[0], args.pmc_summary[1], args.match)

@@ -385,28 +385,39 @@ int tmx_latent_attention(void* stream, int act, const void* q, const void* cache
                          const uint8_t* input_mask, const int32_t* step, int buf_len, void* out, void* workspace,
                          int n_seq, int T, int H, int rank_p, int rot_p, int C, float scale);
 
+/* place[m] (int32 [M][2]) of the token at slot *step + m % T of sequence m / T: the first slot of its chunk of `chunk`
+ * positions (0 with chunk == 0), and its position.  Positions along a sequence's slots do not decrease; slots with
+ * input_mask 0 hold no token. */
+int tmx_row_places(void* stream, const int32_t* positions, const uint8_t* input_mask, const int32_t* step, int buf_len,
+                   int32_t* place, int M, int T, int C, int chunk);
+
 /* Row kernel of grouped attention: takes the fused projection row z[m] = [H query heads of dk | Kh key heads of dk | Kh
  * value heads of dv] (dk, dv: padded widths; dim: real width of a query / key head) and writes
  *   q[m][H][dk], and the rows of slot *step + m % T: kcache [sequence][Kh][C][dk], vcache [sequence][Kh][C][dv].
  * Queries and keys are first divided by their root mean square (over dim) and multiplied by q_norm_w / k_norm_w (f32
  * [dk], NULL: no norm), then their first `rot` columns are rotated: table f32 [positions_max][rot / 2][2] cos, sin; the
- * pair of dimension i is i + rot / 2 (rot == 0: no rotation).
- *   first: int32 [M], the first slot of the row's chunk of `chunk` positions (0 with chunk == 0), for tmx_head_attention.
- *          Positions along a sequence's slots do not decrease; slots with input_mask 0 hold no token. */
+ * pair of dimension i is i + rot / 2 (rot == 0: no rotation).  place: see tmx_row_places. */
 int tmx_head_rows(void* stream, int act, const void* z, int ldz, const float* q_norm_w, const float* k_norm_w, float eps,
-                  const float* table, int positions_max, const int32_t* positions, const uint8_t* input_mask,
-                  const int32_t* step, int buf_len, void* q, void* kcache, void* vcache, int32_t* first, int M, int T,
-                  int H, int Kh, int dim, int dk, int dv, int rot, int C, int chunk);
+                  const float* table, int positions_max, const int32_t* place, const int32_t* step, int buf_len, void* q,
+                  void* kcache, void* vcache, int M, int T, int H, int Kh, int dim, int dk, int dv, int rot, int C);
 
-/* out[m][h][dv] = sum_j softmax_j(q[m, h] . K[j] * scale) V[j] over the slots first[m] <= j <= *step + m % T with
+/* out[m][h][dv] = sum_j softmax_j(q[m, h] . K[j] * scale) V[j] over the slots place[m][0] <= j <= *step + m % T with
  * input_mask[m / T, j], K and V of kv head floor(h / (H / Kh)); with sink (f32 [H]) the denominator also holds
  * exp(sink[h]).  dk and dv in {64, 128, 256}, H % Kh == 0, any H / Kh.
  * chunk: the most slots a row sees (0: no bound), from which the launch is planned.
  * workspace: tmx_head_attention_workspace_bytes(M / T, T, H, Kh, dv, C, chunk) bytes (may be 0 -> NULL allowed). */
 size_t tmx_head_attention_workspace_bytes(int n_seq, int T, int H, int Kh, int dv, int C, int chunk);
 int tmx_head_attention(void* stream, int act, const void* q, const void* kcache, const void* vcache, const float* sink,
-                       const int32_t* first, const uint8_t* input_mask, const int32_t* step, int buf_len, void* out,
+                       const int32_t* place, const uint8_t* input_mask, const int32_t* step, int buf_len, void* out,
                        void* workspace, int n_seq, int T, int H, int Kh, int dk, int dv, int C, int chunk, float scale);
+
+/* tmx_head_rows and tmx_head_attention of one bf16 token per sequence in one launch (the queries stay on the chip);
+ * H / Kh <= 32.  workspace: tmx_head_attention_workspace_bytes(n_seq, 1, ...). */
+int tmx_head_decode(void* stream, const void* z, int ldz, const float* q_norm_w, const float* k_norm_w, float eps,
+                    const float* table, int positions_max, const int32_t* place, void* kcache, void* vcache,
+                    const float* sink, const uint8_t* input_mask, const int32_t* step, int buf_len, void* out,
+                    void* workspace, int n_seq, int H, int Kh, int dim, int dk, int dv, int rot, int C, int chunk,
+                    float scale);
 
 /* ---- whole decode steps ------------------------------------------------------ */
 

@@ -4,6 +4,8 @@ import ctypes
 import numpy as np
 import torch
 
+import common as C
+from oracle.bf16 import bf16_round
 from tunix_amd import _lib
 
 DEV = 'cuda'
@@ -85,3 +87,55 @@ class Keep:
 
   def u8(self, x):
     return self._k(u8(x))
+
+
+# -- dense decoders: number formats, and whole models through the Sampler ------------------
+def dev(x, dtype):
+  return f32(x) if dtype == 'float32' else bf(x)
+
+
+def act(dtype):
+  return 1 if dtype == 'float32' else 0
+
+
+def rounded(x, dtype):
+  return x if dtype == 'float32' else bf16_round(x)
+
+
+def up(v, k):
+  return -(-v // k) * k
+
+
+def sampler(m, size):
+  from tunix_amd.configs import CacheConfig
+  from tunix_amd.sampler import Sampler
+  c = m.config
+  s = Sampler(m, C.ToyTokenizer(), CacheConfig(size, c.num_layers, c.num_kv_heads, c.head_dim))
+  s.eos_ids = np.array([-1])
+  return s
+
+
+def batch_state(s, rows, total):
+  width = max(len(r) for r in rows)
+  ids = np.zeros((len(rows), width), np.int32)
+  for i, r in enumerate(rows):
+    ids[i, width - len(r):] = r
+  st = s.init_sample_state(ids, total, False, None, 1.0, None, None, 0, prompt_lengths=np.array([len(r) for r in rows]))
+  st['fresh'] = False
+  return st, width
+
+
+def all_logits(s, rows, total, cuts=None):
+  """Logits of every token of every row; the columns in portions of `cuts` (None: as the walk likes)."""
+  st, width = batch_state(s, rows, total)
+  got = [np.zeros((len(r), s.transformer.config.vocab_size)) for r in rows]
+  beg = 0
+  for n in (cuts or [width]):
+    wanted = [(i, c - beg) for i, r in enumerate(rows) for c in range(beg, beg + n) if c >= width - len(r)]
+    lg = s.walk_logits(st, n, wanted).cpu().numpy()
+    for (i, off), v in zip(wanted, lg):
+      got[i][beg + off - (width - len(rows[i]))] = v
+    beg += n
+  assert beg == width
+  s.check_device_status(st)
+  return got

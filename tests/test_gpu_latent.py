@@ -13,37 +13,21 @@ import torch
 import common as C
 import gpu_util as G
 import latent_common as LC
+from gpu_util import act, all_logits, dev, rounded, sampler, up
 from oracle import latent as OL
 from oracle.bf16 import bf16_round
 from tunix_amd import _lib
-from tunix_amd.configs import CacheConfig, RolloutConfig
+from tunix_amd.configs import RolloutConfig
 from tunix_amd.latent import pack_tiles
-from tunix_amd.sampler import Sampler
 
 pytestmark = pytest.mark.gpu
 S = _lib.stream
 FORMATS = ['float32', 'bfloat16']
 
 
-def dev(x, dtype):
-  return G.f32(x) if dtype == 'float32' else G.bf(x)
-
-
-def act(dtype):
-  return 1 if dtype == 'float32' else 0
-
-
-def rounded(x, dtype):
-  return x if dtype == 'float32' else bf16_round(x)
-
-
-def up(v, k):
-  return -(-v // k) * k
-
-
 # -- mechanisms alone -------------------------------------------------------------
 @pytest.mark.parametrize('dtype', FORMATS)
-@pytest.mark.parametrize('epi', [0, 1, 2])
+@pytest.mark.parametrize('epi', [0, 1, 2, 3])
 def test_dense_projection(dtype, epi):
   """Row counts on both sides of every kernel form's limits, K from one tile up, several matrices side by side."""
   rng = np.random.default_rng(epi)
@@ -65,6 +49,8 @@ def test_dense_projection(dtype, epi):
       y = g * OL.sigmoid(g) * u
     elif epi == 2:
       y = y * OL.sigmoid(gate.astype(np.float64))
+    elif epi == 3:
+      y = np.maximum(y, 0.0) ** 2
     wt = torch.from_numpy(w.reshape(heads * n, k))
     wt = wt.to(G.DEV) if dtype == 'float32' else pack_tiles(wt.to(torch.bfloat16)).to(G.DEV)
     keep = [dev(x, dtype), wt, None if bias is None else G.f32(bias), dev(gate, dtype)]
@@ -241,39 +227,6 @@ def plain(name, st, t, dtype):
   if key not in _plain:
     _plain[key] = LC.plain(LC.CONFIGS[name], st, t, dtype)
   return _plain[key]
-
-
-def sampler(m, size):
-  c = m.config
-  s = Sampler(m, C.ToyTokenizer(), CacheConfig(size, c.num_layers, c.num_kv_heads, c.head_dim))
-  s.eos_ids = np.array([-1])
-  return s
-
-
-def batch_state(s, rows, total):
-  width = max(len(r) for r in rows)
-  ids = np.zeros((len(rows), width), np.int32)
-  for i, r in enumerate(rows):
-    ids[i, width - len(r):] = r
-  st = s.init_sample_state(ids, total, False, None, 1.0, None, None, 0, prompt_lengths=np.array([len(r) for r in rows]))
-  st['fresh'] = False
-  return st, width
-
-
-def all_logits(s, rows, total, cuts=None):
-  """Logits of every token of every row; the columns in portions of `cuts` (None: as the walk likes)."""
-  st, width = batch_state(s, rows, total)
-  got = [np.zeros((len(r), s.transformer.config.vocab_size)) for r in rows]
-  beg = 0
-  for n in (cuts or [width]):
-    wanted = [(i, c - beg) for i, r in enumerate(rows) for c in range(beg, beg + n) if c >= width - len(r)]
-    lg = s.walk_logits(st, n, wanted).cpu().numpy()
-    for (i, off), v in zip(wanted, lg):
-      got[i][beg + off - (width - len(rows[i]))] = v
-    beg += n
-  assert beg == width
-  s.check_device_status(st)
-  return got
 
 
 def toks(name, n, seed):

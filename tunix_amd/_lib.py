@@ -47,7 +47,9 @@ SIGNATURES = {
     'tmx_dense_linear': [vp, ci, vp, ci, ci, vp, vp, vp, ci, vp, ci, ci, ci, ci, ci, ci, ci],
     'tmx_stream_rows': [vp, ci, vp, vp, vp, vp, vp, vp, vp, ci, ci, ci, ci, cf, ci],
     'tmx_residual_rows': [vp, ci, vp, vp, vp, vp, vp, ci, ci, ci, cf, ci],
-    'tmx_head_rows': [vp, ci, vp, ci, vp, vp, cf, vp, ci, vp, vp, vp, ci, vp, vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, ci],
+    'tmx_row_places': [vp, vp, vp, vp, ci, vp, ci, ci, ci, ci],
+    'tmx_head_rows': [vp, ci, vp, ci, vp, vp, cf, vp, ci, vp, vp, ci, vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci],
+    'tmx_head_decode': [vp, vp, ci, vp, vp, cf, vp, ci, vp, vp, vp, vp, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, cf],
     'tmx_head_attention': [vp, ci, vp, vp, vp, vp, vp, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, cf],
     'tmx_latent_rows': [vp, ci, vp, ci, ci, ci, vp, cf, vp, ci, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci],
     'tmx_latent_attention': [vp, ci, vp, vp, vp, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, cf],

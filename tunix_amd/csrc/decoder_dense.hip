@@ -3,23 +3,35 @@
 //   latent attention   fused projection (query | latent | gate), rotation / norm / cache row and query into the latent
 //                      space (one launch up to 128 rows), attention over the cache rows, values (with the output gate
 //                      in the epilogue), output projection
-//   grouped attention  fused projection (query | key | value heads), norm / rotation / cache rows, attention, output
-//                      projection
+//   grouped attention  fused projection (query | key | value heads), norm / rotation / cache rows and attention (one
+//                      launch for one token per sequence), output projection
 //   feed-forward       gate | up with SwiGLU or up with a squared relu, down
 //   residual           streams mixed at every boundary with a norm in front of the sublayers (stream_rows), or one stream
 //                      with the norm behind them (residual_rows)
+#include <algorithm>
+
 #include "tmx_decoder.h"
 
 namespace tmx {
 
 static size_t act_bytes(const tmx_model_desc* m) { return m->act == TMX_ACT_F32 ? 4 : 2; }
 
+// The different chunk sizes of the layers with grouped attention.
+static std::vector<int> chunk_sizes(const tmx_model_desc* m) {
+  std::vector<int> out;
+  for (int i = 0; i < m->num_layers; ++i) {
+    const tmx_dense_layer_desc& l = m->dense_layers[i];
+    if (l.mixer == TMX_MIXER_HEADS && std::find(out.begin(), out.end(), l.chunk) == out.end()) out.push_back(l.chunk);
+  }
+  return out;
+}
+
 DenseWorkspace dense_carve(const tmx_model_desc* m, int rows, char* base) {
   DenseWorkspace w = {};
   size_t off = 0;
   auto take = [&](size_t bytes) { char* p = (base && bytes) ? base + off : nullptr; off += align256(bytes); return p; };
   const size_t B = rows, Bt = pad_to(rows, 32), Dp = pad_to(m->embed_dim, 64), e = act_bytes(m);
-  size_t z = 0, q = 0, lat = 0, val = 0, act = 0, part = 0, splits = 1, heads = 0;
+  size_t z = 0, q = 0, lat = 0, val = 0, act = 0, part = 0, splits = 1;
   auto up = [](size_t& d, size_t v) { if (v > d) d = v; };
   for (int i = 0; i < m->num_layers; ++i) {
     const tmx_dense_layer_desc& l = m->dense_layers[i];
@@ -28,7 +40,6 @@ DenseWorkspace dense_carve(const tmx_model_desc* m, int rows, char* base) {
     up(splits, dense_num_splits(m->act, rows, l.o.K, l.o.N));
     if (l.mixer == TMX_MIXER_HEADS) {
       up(q, (size_t)l.heads * l.dim_p);
-      heads = 1;
       if (m->act == TMX_ACT_BF16) up(part, head_attn_partial_bytes(rows, l.heads, l.vdim_p));
     } else {
       up(q, (size_t)l.heads * (l.rank_p + l.rot_p));
@@ -49,7 +60,7 @@ DenseWorkspace dense_carve(const tmx_model_desc* m, int rows, char* base) {
   w.val = take(Bt * val * e);
   w.y = take(B * Dp * e);
   w.act = take(Bt * act * e);
-  w.first = (int32_t*)take(heads * B * 4);
+  w.place = (int2*)take(chunk_sizes(m).size() * B * 8);
   w.attn_partial = (float*)take(part);
   w.y_part = (float*)take(splits > 1 ? splits * B * Dp * 4 : 0);
   const size_t Vp = pad_to(m->vocab_size, 32);
@@ -233,25 +244,31 @@ int dense_layers(hipStream_t st, const tmx_model_desc* m, const tmx_decode_state
     }
     return TMX_OK;
   };
+  const std::vector<int> chunks = chunk_sizes(m);
+  auto place_of = [&](int chunk) { return w.place + (std::find(chunks.begin(), chunks.end(), chunk) - chunks.begin()) * (size_t)M; };
+  for (int chunk : chunks) {
+    RowPlacesArgs a = {};
+    a.positions = s->positions; a.input_mask = s->input_mask; a.step = s->step; a.buf_len = L; a.tpp = T; a.C = C;
+    a.chunk = chunk; a.place = place_of(chunk);
+    TMX_TRY(TMX_K_ROPE, row_places(st, a, M));
+  }
   auto heads_mixer = [&](const tmx_dense_layer_desc& l, char* kcache) {
     char* vcache = kcache + (size_t)n_seq * C * l.kv_heads * l.dim_p * e;
-    {
-      HeadRowsArgs a = {};
-      a.z = w.z; a.ldz = l.in.N; a.q_norm_w = l.q_norm_w; a.k_norm_w = l.k_norm_w; a.eps = m->norm_eps;
-      a.table = l.table; a.max_positions = m->max_positions;
-      a.positions = s->positions; a.input_mask = s->input_mask; a.step = s->step; a.buf_len = L; a.tpp = T;
-      a.q = w.q; a.kcache = kcache; a.vcache = vcache; a.first = w.first;
-      a.H = l.heads; a.Kh = l.kv_heads; a.dim = l.dim; a.dk = l.dim_p; a.dv = l.vdim_p; a.rot = l.rot_dim; a.C = C;
-      a.chunk = l.chunk;
-      TMX_TRY(TMX_K_ROPE, head_rows(st, act, a, M));
-    }
+    HeadRowsArgs r = {};
+    r.z = w.z; r.ldz = l.in.N; r.q_norm_w = l.q_norm_w; r.k_norm_w = l.k_norm_w; r.eps = m->norm_eps;
+    r.table = l.table; r.max_positions = m->max_positions;
+    r.place = place_of(l.chunk); r.step = s->step; r.buf_len = L; r.tpp = T;
+    r.q = w.q; r.kcache = kcache; r.vcache = vcache;
+    r.H = l.heads; r.Kh = l.kv_heads; r.dim = l.dim; r.dk = l.dim_p; r.dv = l.vdim_p; r.rot = l.rot_dim; r.C = C;
+    const bool fused = head_rows_fused(act, T, l.heads, l.kv_heads);
+    if (!fused) TMX_TRY(TMX_K_ROPE, head_rows(st, act, r, M));
     HeadAttnArgs a = {};
-    a.q = w.q; a.kcache = kcache; a.vcache = vcache; a.sink = l.sink; a.first = w.first;
+    a.q = w.q; a.kcache = kcache; a.vcache = vcache; a.sink = l.sink; a.place = r.place;
     a.input_mask = s->input_mask; a.step = s->step; a.buf_len = L;
     a.out = w.val; a.out_tiled = tiled; a.partial = w.attn_partial;
     a.n_seq = n_seq; a.tpp = T; a.H = l.heads; a.Kh = l.kv_heads; a.dk = l.dim_p; a.dv = l.vdim_p; a.C = C;
     a.chunk = l.chunk; a.scale = l.scale;
-    TMX_TRY(TMX_K_ATTN, head_attention(st, act, a));
+    TMX_TRY(TMX_K_ATTN, head_attention(st, act, a, fused ? &r : nullptr));
     return TMX_OK;
   };
   for (int i = 0; i < m->num_layers; ++i) {

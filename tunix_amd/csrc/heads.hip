@@ -1,8 +1,10 @@
 // Grouped-query attention of dense models: query / key heads and value heads of their own widths, any number of query
 // heads per key head, optionally a norm per head, a rotation of the first dimensions, chunks (a token sees the earlier
 // tokens of its own chunk of positions) and a softmax sink.
-//   head_rows_kernel      norm and rotation of queries and keys, cache rows, first visible slot of every row
-//   head_attn_kernel      the walk over the cache on the matrix pipe (one or many tokens per sequence)
+//   row_places_kernel     first slot every row sees and its position, once per pass and chunk size
+//   head_rows_kernel      norm and rotation of queries and keys, cache rows
+//   head_attn_kernel      the walk over the cache on the matrix pipe (one or many tokens per sequence); for one token per
+//                         sequence the row part is in front of it in the same launch
 //   head_combine_kernel   merge of the splits of a query row
 //   head_attn_f32_kernel  the same attention in f32 on the vector ALU
 // The cache holds K [sequence][Kh][C][dk] and V [sequence][Kh][C][dv]: the rows one workgroup walks are consecutive.
@@ -12,14 +14,11 @@ namespace tmx {
 
 __device__ __forceinline__ float act_get(const uint16_t* p) { return bf2f(*p); }
 __device__ __forceinline__ float act_get(const float* p) { return *p; }
-__device__ __forceinline__ void act_set(uint16_t* p, float v) { *p = f2bf(v); }
-__device__ __forceinline__ void act_set(float* p, float v) { *p = v; }
 
 // First slot of the chunk of the token at slot `col`.  Without unused slots in between it lies position - chunk start
 // slots back; that guess is right when the slot holds a token at the chunk's first position, else the (never
 // decreasing) positions are searched.
 __device__ __forceinline__ int first_slot(const int32_t* pos, const uint8_t* mask, int col, int chunk) {
-  if (chunk <= 0) return 0;
   const int p = max(pos[col], 0), start = p - p % chunk, guess = col - (p - start);
   if (guess >= 0 && mask[guess] && pos[guess] == start) return guess;
   int lo = 0, hi = col;  // the first slot in [lo, hi] whose position is at least `start`
@@ -31,59 +30,139 @@ __device__ __forceinline__ int first_slot(const int32_t* pos, const uint8_t* mas
   return lo;
 }
 
-// A wave per head of a row: blockIdx.x = row * groups of 4 heads + group.
-template <typename T>
+__global__ __launch_bounds__(256) void row_places_kernel(RowPlacesArgs a, int M) {
+  const int m = blockIdx.x * 256 + threadIdx.x;
+  if (m >= M) return;
+  const int seq = m / a.tpp, slot = min(*a.step + m % a.tpp, min(a.buf_len, a.C) - 1);
+  const size_t off = (size_t)seq * a.buf_len;
+  const int first = a.chunk > 0 ? first_slot(a.positions + off, a.input_mask + off, slot, a.chunk) : 0;
+  a.place[m] = make_int2(first, max(a.positions[off + slot], 0));
+}
+
+// E consecutive values of an act tensor at an offset that is a multiple of E.
+template <int E>
+__device__ __forceinline__ void load_e(const uint16_t* p, float* v) {
+  if constexpr (E == 1) {
+    v[0] = bf2f(*p);
+  } else {
+#pragma unroll
+    for (int i = 0; i < E / 2; ++i) {
+      const uint32_t w = reinterpret_cast<const uint32_t*>(p)[i];
+      v[2 * i] = bf_lo(w);
+      v[2 * i + 1] = bf_hi(w);
+    }
+  }
+}
+template <int E>
+__device__ __forceinline__ void load_e(const float* p, float* v) {
+#pragma unroll
+  for (int i = 0; i < E; ++i) v[i] = p[i];
+}
+template <int E>
+__device__ __forceinline__ void store_e(uint16_t* p, const float* v) {
+  if constexpr (E == 1) {
+    *p = f2bf(v[0]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < E / 2; ++i) reinterpret_cast<uint32_t*>(p)[i] = pack_bf2(v[2 * i], v[2 * i + 1]);
+  }
+}
+template <int E>
+__device__ __forceinline__ void store_e(float* p, const float* v) {
+#pragma unroll
+  for (int i = 0; i < E; ++i) p[i] = v[i];
+}
+
+// What a lane needs of the rotation at one position: it owns the E columns c = E lane .. of a head of 64 E columns, whose
+// partners begin at column `mate` (E consecutive ones when half a rotation is a multiple of E).
+template <int E>
+struct HeadLane {
+  int c, half, rot, mate;
+  float cs[E], sn[E];  // sn carries the sign of the column's half; 1, 0 past the rotated columns
+  __device__ __forceinline__ HeadLane(const HeadRowsArgs& a, int lane, int pos) : c(E * lane), half(a.rot >> 1), rot(a.rot) {
+    const float2* tab = reinterpret_cast<const float2*>(a.table) + (size_t)pos * half;
+    mate = c < half ? c + half : c - half;
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+      const int k = c + e;
+      cs[e] = 1.f;
+      sn[e] = 0.f;
+      if (k < rot) {
+        const float2 t = tab[k < half ? k : k - half];
+        cs[e] = t.x;
+        sn[e] = k < half ? -t.y : t.y;
+      }
+    }
+  }
+  // partners of the lane's columns in a head at src (its own columns in v where there are none)
+  template <typename T>
+  __device__ __forceinline__ void partners(const T* src, const float* v, float* u) const {
+    if (half % E == 0) {
+      if (c < rot) load_e<E>(src + mate, u);
+      else {
+#pragma unroll
+        for (int e = 0; e < E; ++e) u[e] = v[e];
+      }
+      return;
+    }
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+      const int k = c + e;
+      u[e] = k < rot ? act_get(src + (k < half ? k + half : k - half)) : v[e];
+    }
+  }
+  // v <- the head's normed and rotated values
+  __device__ __forceinline__ void finish(float* v, const float* u, const float* nw, int dim, float eps) const {
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < E; ++e) ss += v[e] * v[e];
+    const float inv = nw ? 1.f / sqrtf(wave_sum(ss) / (float)dim + eps) : 1.f;
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+      const int k = c + e, p = k < rot ? (k < half ? k + half : k - half) : k;
+      const float x = v[e] * inv * (nw ? nw[k] : 1.f), y = u[e] * inv * (nw ? nw[p] : 1.f);
+      v[e] = x * cs[e] + y * sn[e];
+    }
+  }
+};
+
+// Four heads of a row per wave: blockIdx.x = row * groups of 16 heads + group.  E: columns of a query / key head / 64.
+template <typename T, int E>
 __global__ __launch_bounds__(256) void head_rows_kernel(HeadRowsArgs a) {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int heads = a.H + 2 * a.Kh, groups = (heads + 3) / 4;
-  const int m = blockIdx.x / groups, hd = (blockIdx.x % groups) * 4 + wave;
-  if (hd >= heads) return;
+  const int heads = a.H + 2 * a.Kh, groups = (heads + 15) / 16, qk = a.H + a.Kh;
+  const int m = blockIdx.x / groups, hd0 = (blockIdx.x % groups) * 16 + wave * 4;
+  if (hd0 >= heads) return;
   const int tpp = a.tpp > 0 ? a.tpp : 1;
   const int seq = m / tpp, slot = min(*a.step + m % tpp, min(a.buf_len, a.C) - 1);
-  const int32_t* prow = a.positions + (size_t)seq * a.buf_len;
   const T* z = reinterpret_cast<const T*>(a.z) + (size_t)m * a.ldz;
-  if (hd >= a.H + a.Kh) {  // value head: copied
-    const int g = hd - a.H - a.Kh;
-    const T* src = z + (size_t)(a.H + a.Kh) * a.dk + (size_t)g * a.dv;
-    T* dst = reinterpret_cast<T*>(a.vcache) + (((size_t)seq * a.Kh + g) * a.C + slot) * a.dv;
-    for (int c = lane; c < a.dv; c += 64) dst[c] = src[c];
-    return;
-  }
-  if (hd == 0 && lane == 0 && a.first) a.first[m] = first_slot(prow, a.input_mask + (size_t)seq * a.buf_len, slot, a.chunk);
-  const int half = a.rot >> 1;
-  const int pos = min(max(prow[slot], 0), a.max_positions - 1);
-  const float2* tab = reinterpret_cast<const float2*>(a.table) + (size_t)pos * half;
-  const bool key = hd >= a.H;
-  const float* nw = key ? a.k_norm_w : a.q_norm_w;
-  const T* src = z + (size_t)hd * a.dk;
-  T* dst = key ? reinterpret_cast<T*>(a.kcache) + (((size_t)seq * a.Kh + hd - a.H) * a.C + slot) * a.dk
-               : reinterpret_cast<T*>(a.q) + ((size_t)m * a.H + hd) * a.dk;
-  constexpr int E = TMX_MAX_HEAD_DIM / 64;
-  float v[E], u[E];  // this lane's values and their partners in the rotation
-  float ss = 0.f;
+  if (hd0 < qk) {
+    const HeadLane<E> hl(a, lane, min(a.place[m].y, a.max_positions - 1));
+    float v[4][E], u[4][E];
 #pragma unroll
-  for (int j = 0; j < E; ++j) {
-    const int c = lane + 64 * j;
-    v[j] = u[j] = 0.f;
-    if (c < a.dk) {
-      v[j] = act_get(src + c);
-      if (c < a.rot) u[j] = act_get(src + (c < half ? c + half : c - half));
+    for (int i = 0; i < 4; ++i) {  // (heads past the last key repeat it)
+      const T* src = z + (size_t)min(hd0 + i, qk - 1) * (64 * E);
+      load_e<E>(src + hl.c, v[i]);
+      hl.partners(src, v[i], u[i]);
     }
-    ss += v[j] * v[j];
-  }
-  const float inv = nw ? 1.f / sqrtf(wave_sum(ss) / (float)a.dim + a.eps) : 1.f;
 #pragma unroll
-  for (int j = 0; j < E; ++j) {
-    const int c = lane + 64 * j;
-    if (c >= a.dk) continue;
-    float o = v[j] * inv * (nw ? nw[c] : 1.f);
-    if (c < a.rot) {
-      const int i = c < half ? c : c - half, p = c < half ? c + half : i;
-      const float w = u[j] * inv * (nw ? nw[p] : 1.f);
-      const float2 cs = tab[i];
-      o = c < half ? o * cs.x - w * cs.y : o * cs.x + w * cs.y;
+    for (int i = 0; i < 4; ++i) {
+      const int hd = hd0 + i;
+      if (hd >= qk) break;
+      const bool key = hd >= a.H;
+      hl.finish(v[i], u[i], key ? a.k_norm_w : a.q_norm_w, a.dim, a.eps);
+      T* dst = key ? reinterpret_cast<T*>(a.kcache) + (((size_t)seq * a.Kh + hd - a.H) * a.C + slot) * (64 * E)
+                   : reinterpret_cast<T*>(a.q) + ((size_t)m * a.H + hd) * (64 * E);
+      store_e<E>(dst + hl.c, v[i]);
     }
-    act_set(dst + c, o);
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {  // value heads are copied
+    const int g = hd0 + i - qk;
+    if (g < 0 || g >= a.Kh) continue;
+    const uint32_t* src = reinterpret_cast<const uint32_t*>(z + (size_t)qk * a.dk + (size_t)g * a.dv);
+    uint32_t* dst = reinterpret_cast<uint32_t*>(reinterpret_cast<T*>(a.vcache) + (((size_t)seq * a.Kh + g) * a.C + slot) * a.dv);
+    for (int c = lane; c < a.dv * (int)sizeof(T) / 4; c += 64) dst[c] = src[c];
   }
 }
 
@@ -95,8 +174,10 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HeadRowsArgs a) {
 //   SHARED (many query rows): the four waves hold different query rows and walk the same blocks, double-buffered;
 //   else (up to 32 query rows): the waves hold the same rows and walk different blocks in tiles of their own, and meet
 //   through LDS at the end.
+//   ROWS (not SHARED, one token per sequence): the workgroup makes its queries and the new cache row from the fused
+//   projection itself; they wait in LDS, from where the new row replaces what its slot held in the tile.
 // KT, VT: padded widths / 64.
-template <int KT, int VT, bool SHARED>
+template <int KT, int VT, bool SHARED, bool ROWS>
 struct HeadShape {
   static constexpr int DK = KT * 64, DV = VT * 64;
   static constexpr int WQ = SHARED ? 4 : 1, WP = SHARED ? 1 : 4;
@@ -104,7 +185,8 @@ struct HeadShape {
   static constexpr int kBufs = SHARED || kTile * 2 * 4 * 2 <= 64 * 1024 ? 2 : 1;
   static constexpr size_t kTiles = (size_t)kBufs * WP * kTile * 2;
   static constexpr size_t kMerge = SHARED ? 0 : (size_t)2 * (DV * 32 * 4 + 2 * 32 * 4);
-  static constexpr size_t kBytes = kTiles > kMerge ? kTiles : kMerge;
+  static constexpr size_t kStage = (kTiles > kMerge ? kTiles : kMerge);  // queries [32][DK], key [DK], value [DV] bf16
+  static constexpr size_t kBytes = kStage + (ROWS ? (size_t)(33 * DK + DV) * 2 : 0);
 };
 
 // 16-byte chunk c of row r lies at chunk c ^ swz(r); CPR: chunks per row.  Rows of at least 256 bytes are told apart by
@@ -114,9 +196,10 @@ __device__ __forceinline__ constexpr int head_swz(int row) {
   return CPR % 16 == 0 ? ((row & 3) << 2) | ((row >> 2) & 3) : (((row >> 1) & 1) << 2) | ((row >> 2) & 3);
 }
 
-template <int KT, int VT, bool SHARED>
-__global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(HeadAttnArgs a) {
-  using SH = HeadShape<KT, VT, SHARED>;
+template <int KT, int VT, bool SHARED, bool ROWS>
+__global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(HeadAttnArgs a, HeadRowsArgs ra) {
+  static_assert(!(SHARED && ROWS), "one token per sequence only");
+  using SH = HeadShape<KT, VT, SHARED, ROWS>;
   extern __shared__ __align__(16) unsigned char ha_smem[];
   constexpr int DK = SH::DK, DV = SH::DV, CK = DK / 8, CV = DV / 8, KS = DK / 16, VC = DV / 32;
   constexpr int WPW = 4 / SH::WP;  // waves that share a tile
@@ -161,11 +244,56 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
   };
 
   const int step0 = max(min(*a.step, min(a.C, a.buf_len) - a.tpp), 0);  // clamped: every slot read lies in the cache
-  const int32_t* frow = a.first + (size_t)seq * a.tpp;
-  const int first = max(frow[tok], 0);                        // oldest slot this query sees (it does not decrease along the tokens)
-  const int b_beg = max(frow[q0 / G], 0) >> 5;                // blocks of the workgroup
+  const int2* place = a.place + (size_t)seq * a.tpp;
+  const int first = place[tok].x;                             // oldest slot this query sees (it does not decrease along the tokens)
+  const int b_beg = place[q0 / G].x >> 5;                     // blocks of the workgroup
+  const int b_end = (step0 + (min(q0 + 32 * SH::WQ, rows) - 1) / G + 32) >> 5;
+  const int b_new = step0 >> 5;                               // ROWS: the block of the new row
+  uint16_t* const stage = reinterpret_cast<uint16_t*>(ha_smem + SH::kStage);
   u32x4_t qf[KS];
-  {
+  if constexpr (ROWS) {
+    constexpr int EM = KT > VT ? KT : VT;
+    const HeadLane<KT> hl(ra, lane, min(place[0].y, ra.max_positions - 1));
+    const uint16_t* z = reinterpret_cast<const uint16_t*>(ra.z) + (size_t)seq * ra.ldz;
+    const bool owner = ((b_new - b_beg) / SH::WP) % a.nsplit == split;  // this workgroup walks the new row's block
+    // key (item 0), value (1), then the group's queries, dealt out to the waves, two at a time; the first tile is
+    // requested behind the first items
+    for (int i0 = wave; i0 < G + 2 || i0 < 4; i0 += 8) {
+      float v[2][EM], u[2][KT];
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        const int i = i0 + 4 * k;
+        if (i >= G + 2) break;
+        if (i == 1) {
+          load_e<VT>(z + (size_t)(a.H + a.Kh) * DK + (size_t)kvh * DV + VT * lane, v[k]);
+        } else {
+          const uint16_t* src = z + (size_t)(i == 0 ? a.H + kvh : kvh * G + i - 2) * DK;
+          load_e<KT>(src + hl.c, v[k]);
+          hl.partners(src, v[k], u[k]);
+        }
+      }
+      if (i0 == wave) {
+        const int blk = b_beg + split * SH::WP + wp;
+        if (blk < b_end) fetch(blk, 0);
+      }
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        const int i = i0 + 4 * k;
+        if (i >= G + 2) break;
+        if (i == 1) {
+          store_e<VT>(stage + 33 * DK + VT * lane, v[k]);
+          if (owner) store_e<VT>(reinterpret_cast<uint16_t*>(ra.vcache) + ((size_t)pair * a.C + step0) * DV + VT * lane, v[k]);
+          continue;
+        }
+        hl.finish(v[k], u[k], i == 0 ? ra.k_norm_w : ra.q_norm_w, ra.dim, ra.eps);
+        store_e<KT>(stage + (i == 0 ? 32 : i - 2) * DK + hl.c, v[k]);
+        if (i == 0 && owner) store_e<KT>(reinterpret_cast<uint16_t*>(ra.kcache) + ((size_t)pair * a.C + step0) * DK + hl.c, v[k]);
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < KS; ++t) qf[t] = *reinterpret_cast<const u32x4_t*>(stage + qr_l * DK + (DK / 2) * h + 8 * t);
+  } else {
     const uint16_t* qp = reinterpret_cast<const uint16_t*>(a.q) + qrow * DK + (DK / 2) * h;
 #pragma unroll
     for (int t = 0; t < KS; ++t) qf[t] = *reinterpret_cast<const u32x4_t*>(qp + 8 * t);
@@ -173,7 +301,6 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
   const int limit = step0 + tok;                              // newest slot this query sees
   const int limit0 = step0 + min(q0 + wq * 32, rows - 1) / G;  // the smallest one in the wave
   const int first1 = __shfl(first, 31, 64);                   // the largest one in the wave
-  const int b_end = (step0 + (min(q0 + 32 * SH::WQ, rows) - 1) / G + 32) >> 5;
 
   f32x16_t o[VC];
 #pragma unroll
@@ -300,12 +427,22 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
     const int stride = a.nsplit * SH::WP;
     int blk = b_beg + split * SH::WP + wp, buf = 0;
     uint8_t mb = mask_byte(blk);
-    if (blk < b_end) fetch(blk, 0);
+    if (!ROWS && blk < b_end) fetch(blk, 0);
     for (; blk < b_end; blk += stride) {
       const uint32_t mbits = (uint32_t)__ballot(mb != 0);
       __builtin_amdgcn_s_waitcnt(0x0F70);  // the wave's own tile has landed
       __builtin_amdgcn_sched_barrier(0);
       mb = mask_byte(blk + stride);
+      if (ROWS && blk == b_new) {
+        uint16_t* kt = tiles + buf * SH::kTile;
+        const int r = step0 & 31;
+        if (lane < CK)
+          *reinterpret_cast<u32x4_t*>(kt + r * DK + ((lane ^ head_swz<CK>(r)) << 3)) = *reinterpret_cast<const u32x4_t*>(stage + 32 * DK + lane * 8);
+        if (lane < CV)
+          *reinterpret_cast<u32x4_t*>(kt + 32 * DK + r * DV + ((lane ^ head_swz<CV>(r)) << 3)) =
+              *reinterpret_cast<const u32x4_t*>(stage + 33 * DK + lane * 8);
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      }
       const bool more = blk + stride < b_end;
       if (SH::kBufs == 2 && more) fetch(blk + stride, buf ^ 1);
       block(blk, mbits, buf);
@@ -424,7 +561,7 @@ __global__ __launch_bounds__(256) void head_attn_f32_kernel(HeadAttnArgs a) {
   const int hd = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int seq = row / a.tpp, kvh = hd / (a.H / a.Kh);
   const int step0 = max(min(*a.step, min(a.C, a.buf_len) - a.tpp), 0);
-  const int limit = step0 + row % a.tpp, first = max(a.first[row], 0);
+  const int limit = step0 + row % a.tpp, first = a.place[row].x;
   const size_t qrow = (size_t)row * a.H + hd, pair = (size_t)seq * a.Kh + kvh;
   for (int i = tid; i < a.dk; i += 256) qs[i] = reinterpret_cast<const float*>(a.q)[qrow * a.dk + i];
   const float* kc = reinterpret_cast<const float*>(a.kcache) + pair * a.C * a.dk;
@@ -472,22 +609,40 @@ bool head_attn_ok(int dk, int dv) {
   return ok(dk) && ok(dv);
 }
 
-int head_rows(hipStream_t st, int act, const HeadRowsArgs& a, int M) {
-  if (M <= 0 || a.H <= 0 || a.Kh <= 0 || a.H % a.Kh || a.dim <= 0 || a.dim > a.dk || a.rot < 0 || a.rot % 2 || a.rot > a.dim ||
-      a.C <= 0 || a.chunk < 0 || !head_attn_ok(a.dk, a.dv))
-    return TMX_ERR_SHAPE;
-  const long wgs = (long)M * ((a.H + 2 * a.Kh + 3) / 4);
-  if (wgs > 0x7FFFFFFF) return TMX_ERR_SHAPE;
-  if (act == TMX_ACT_BF16) hipLaunchKernelGGL(head_rows_kernel<uint16_t>, dim3(wgs), dim3(256), 0, st, a);
-  else if (act == TMX_ACT_F32) hipLaunchKernelGGL(head_rows_kernel<float>, dim3(wgs), dim3(256), 0, st, a);
-  else return TMX_ERR_ARG;
+int row_places(hipStream_t st, const RowPlacesArgs& a, int M) {
+  if (M <= 0 || a.tpp <= 0 || a.buf_len <= 0 || a.C <= 0) return TMX_ERR_SHAPE;
+  hipLaunchKernelGGL(row_places_kernel, dim3((M + 255) / 256), dim3(256), 0, st, a, M);
   return check_launch();
+}
+
+static bool head_rows_ok(const HeadRowsArgs& a) {
+  return a.H > 0 && a.Kh > 0 && a.H % a.Kh == 0 && a.dim > 0 && a.dim <= a.dk && a.rot >= 0 && a.rot % 2 == 0 && a.rot <= a.dim &&
+         a.C > 0 && a.buf_len > 0 && a.max_positions > 0 && head_attn_ok(a.dk, a.dv) && a.ldz % 4 == 0 &&
+         a.ldz >= (a.H + a.Kh) * a.dk + a.Kh * a.dv;
+}
+
+template <typename T>
+static int launch_head_rows(hipStream_t st, const HeadRowsArgs& a, int M) {
+  const long wgs = (long)M * ((a.H + 2 * a.Kh + 15) / 16);
+  if (wgs > 0x7FFFFFFF) return TMX_ERR_SHAPE;
+  switch (a.dk) {
+    case 64: hipLaunchKernelGGL((head_rows_kernel<T, 1>), dim3(wgs), dim3(256), 0, st, a); break;
+    case 128: hipLaunchKernelGGL((head_rows_kernel<T, 2>), dim3(wgs), dim3(256), 0, st, a); break;
+    default: hipLaunchKernelGGL((head_rows_kernel<T, 4>), dim3(wgs), dim3(256), 0, st, a); break;
+  }
+  return check_launch();
+}
+
+int head_rows(hipStream_t st, int act, const HeadRowsArgs& a, int M) {
+  if (M <= 0 || !head_rows_ok(a)) return TMX_ERR_SHAPE;
+  if (act == TMX_ACT_BF16) return launch_head_rows<uint16_t>(st, a, M);
+  return act == TMX_ACT_F32 ? launch_head_rows<float>(st, a, M) : TMX_ERR_ARG;
 }
 
 // A workgroup holds 128 query rows of a (sequence, kv head), or up to 32 with its waves on different blocks; the slots a
 // row sees are split until the CUs are full, as long as a split keeps its waves busy for a while.
 struct HeadPlan { bool shared; int nsplit; };
-constexpr int kHeadWgs = 512, kHeadMaxSplits = 32, kHeadSplitSlots = 256;
+constexpr int kHeadWgs = 512, kHeadMaxSplits = 32, kHeadSplitSlots = 128;
 static HeadPlan head_plan(int n_seq, int T, int H, int Kh, int C, int chunk) {
   HeadPlan p;
   const int rows = T * (H / Kh);
@@ -510,30 +665,40 @@ size_t head_attn_partial_bytes(int rows, int H, int dv) {
   return parts * (dv + 4) * 4;
 }
 
-template <int KT, int VT, bool SHARED>
-static int launch_head(hipStream_t st, const HeadAttnArgs& a) {
-  using L = HeadShape<KT, VT, SHARED>;
-  static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&head_attn_kernel<KT, VT, SHARED>),
+template <int KT, int VT, bool SHARED, bool ROWS>
+static int launch_head(hipStream_t st, const HeadAttnArgs& a, const HeadRowsArgs& r) {
+  using L = HeadShape<KT, VT, SHARED, ROWS>;
+  static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&head_attn_kernel<KT, VT, SHARED, ROWS>),
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, (int)L::kBytes);
   if (attr != hipSuccess) return TMX_ERR_LAUNCH;
   const int rows = a.tpp * (a.H / a.Kh), per = 32 * L::WQ;
-  hipLaunchKernelGGL((head_attn_kernel<KT, VT, SHARED>), dim3((size_t)a.n_seq * a.Kh * ((rows + per - 1) / per), 1, a.nsplit),
-                     dim3(256), L::kBytes, st, a);
+  hipLaunchKernelGGL((head_attn_kernel<KT, VT, SHARED, ROWS>), dim3((size_t)a.n_seq * a.Kh * ((rows + per - 1) / per), 1, a.nsplit),
+                     dim3(256), L::kBytes, st, a, r);
   return check_launch();
 }
+template <int KT, int VT>
+static int launch_head_kv(hipStream_t st, const HeadAttnArgs& a, bool shared, const HeadRowsArgs* r) {
+  if (r) return launch_head<KT, VT, false, true>(st, a, *r);
+  return shared ? launch_head<KT, VT, true, false>(st, a, HeadRowsArgs()) : launch_head<KT, VT, false, false>(st, a, HeadRowsArgs());
+}
 template <int KT>
-static int launch_head_v(hipStream_t st, const HeadAttnArgs& a, bool shared) {
+static int launch_head_v(hipStream_t st, const HeadAttnArgs& a, bool shared, const HeadRowsArgs* r) {
   switch (a.dv) {
-    case 64: return shared ? launch_head<KT, 1, true>(st, a) : launch_head<KT, 1, false>(st, a);
-    case 128: return shared ? launch_head<KT, 2, true>(st, a) : launch_head<KT, 2, false>(st, a);
-    default: return shared ? launch_head<KT, 4, true>(st, a) : launch_head<KT, 4, false>(st, a);
+    case 64: return launch_head_kv<KT, 1>(st, a, shared, r);
+    case 128: return launch_head_kv<KT, 2>(st, a, shared, r);
+    default: return launch_head_kv<KT, 4>(st, a, shared, r);
   }
 }
 
-int head_attention(hipStream_t st, int act, HeadAttnArgs a) {
+bool head_rows_fused(int act, int T, int H, int Kh) { return act == TMX_ACT_BF16 && T == 1 && H / Kh <= 32; }
+
+int head_attention(hipStream_t st, int act, HeadAttnArgs a, const HeadRowsArgs* r) {
   if (a.n_seq <= 0 || a.tpp <= 0 || a.H <= 0 || a.Kh <= 0 || a.H % a.Kh || a.C <= 0 || a.tpp > a.C || a.tpp > a.buf_len ||
       a.chunk < 0 || !head_attn_ok(a.dk, a.dv) || (long)a.n_seq * a.tpp * a.H > 0x3FFFFFFF)
     return TMX_ERR_SHAPE;
+  if (r && (!head_rows_fused(act, a.tpp, a.H, a.Kh) || !head_rows_ok(*r) || r->H != a.H || r->Kh != a.Kh || r->dk != a.dk ||
+            r->dv != a.dv || r->C != a.C || r->buf_len != a.buf_len))
+    return TMX_ERR_ARG;
   if (act == TMX_ACT_F32) {
     if ((long)a.n_seq * a.tpp > 65535) return TMX_ERR_SHAPE;
     hipLaunchKernelGGL(head_attn_f32_kernel, dim3(a.H, a.n_seq * a.tpp), dim3(256), 0, st, a);
@@ -548,9 +713,9 @@ int head_attention(hipStream_t st, int act, HeadAttnArgs a) {
   if (a.nsplit > 1 && !a.partial) return TMX_ERR_ARG;
   int rc;
   switch (a.dk) {
-    case 64: rc = launch_head_v<1>(st, a, p.shared); break;
-    case 128: rc = launch_head_v<2>(st, a, p.shared); break;
-    default: rc = launch_head_v<4>(st, a, p.shared); break;
+    case 64: rc = launch_head_v<1>(st, a, p.shared, r); break;
+    case 128: rc = launch_head_v<2>(st, a, p.shared, r); break;
+    default: rc = launch_head_v<4>(st, a, p.shared, r); break;
   }
   if (rc != TMX_OK || a.nsplit == 1) return rc;
   const int total = a.n_seq * a.tpp * a.H;
@@ -562,18 +727,36 @@ int head_attention(hipStream_t st, int act, HeadAttnArgs a) {
 
 using namespace tmx;
 
-extern "C" int tmx_head_rows(void* stream, int act, const void* z, int ldz, const float* q_norm_w, const float* k_norm_w,
-                             float eps, const float* table, int positions_max, const int32_t* positions,
-                             const uint8_t* input_mask, const int32_t* step, int buf_len, void* q, void* kcache,
-                             void* vcache, int32_t* first, int M, int T, int H, int Kh, int dim, int dk, int dv, int rot,
-                             int C, int chunk) {
-  if (!z || !positions || !input_mask || !step || !q || !kcache || !vcache || !first || (rot > 0 && !table)) return TMX_ERR_ARG;
-  if (T <= 0 || M % T || positions_max <= 0 || buf_len <= 0) return TMX_ERR_SHAPE;
-  HeadRowsArgs a = {};
+extern "C" int tmx_row_places(void* stream, const int32_t* positions, const uint8_t* input_mask, const int32_t* step,
+                              int buf_len, int32_t* place, int M, int T, int C, int chunk) {
+  if (!positions || !input_mask || !step || !place) return TMX_ERR_ARG;
+  if (T <= 0 || M % T || chunk < 0) return TMX_ERR_SHAPE;
+  RowPlacesArgs a = {};
+  a.positions = positions; a.input_mask = input_mask; a.step = step; a.buf_len = buf_len; a.tpp = T; a.C = C; a.chunk = chunk;
+  a.place = (int2*)place;
+  return row_places((hipStream_t)stream, a, M);
+}
+
+static int head_rows_args(HeadRowsArgs& a, const void* z, int ldz, const float* q_norm_w, const float* k_norm_w, float eps,
+                          const float* table, int positions_max, const int32_t* place, const int32_t* step, int buf_len,
+                          void* q, void* kcache, void* vcache, int T, int H, int Kh, int dim, int dk, int dv, int rot, int C) {
+  if (!z || !place || !step || !kcache || !vcache || (rot > 0 && !table)) return TMX_ERR_ARG;
   a.z = z; a.ldz = ldz; a.q_norm_w = q_norm_w; a.k_norm_w = k_norm_w; a.eps = eps;
-  a.table = table; a.max_positions = positions_max; a.positions = positions; a.input_mask = input_mask; a.step = step;
-  a.buf_len = buf_len; a.tpp = T; a.q = q; a.kcache = kcache; a.vcache = vcache; a.first = first;
-  a.H = H; a.Kh = Kh; a.dim = dim; a.dk = dk; a.dv = dv; a.rot = rot; a.C = C; a.chunk = chunk;
+  a.table = table; a.max_positions = positions_max; a.place = (const int2*)place; a.step = step;
+  a.buf_len = buf_len; a.tpp = T; a.q = q; a.kcache = kcache; a.vcache = vcache;
+  a.H = H; a.Kh = Kh; a.dim = dim; a.dk = dk; a.dv = dv; a.rot = rot; a.C = C;
+  return TMX_OK;
+}
+
+extern "C" int tmx_head_rows(void* stream, int act, const void* z, int ldz, const float* q_norm_w, const float* k_norm_w,
+                             float eps, const float* table, int positions_max, const int32_t* place,
+                             const int32_t* step, int buf_len, void* q, void* kcache, void* vcache, int M, int T, int H,
+                             int Kh, int dim, int dk, int dv, int rot, int C) {
+  HeadRowsArgs a = {};
+  if (!q || head_rows_args(a, z, ldz, q_norm_w, k_norm_w, eps, table, positions_max, place, step, buf_len, q, kcache, vcache,
+                           T, H, Kh, dim, dk, dv, rot, C))
+    return TMX_ERR_ARG;
+  if (T <= 0 || M % T) return TMX_ERR_SHAPE;
   return head_rows((hipStream_t)stream, act, a, M);
 }
 
@@ -584,13 +767,29 @@ extern "C" size_t tmx_head_attention_workspace_bytes(int n_seq, int T, int H, in
 }
 
 extern "C" int tmx_head_attention(void* stream, int act, const void* q, const void* kcache, const void* vcache,
-                                  const float* sink, const int32_t* first, const uint8_t* input_mask, const int32_t* step,
+                                  const float* sink, const int32_t* place, const uint8_t* input_mask, const int32_t* step,
                                   int buf_len, void* out, void* workspace, int n_seq, int T, int H, int Kh, int dk, int dv,
                                   int C, int chunk, float scale) {
-  if (!q || !kcache || !vcache || !first || !input_mask || !step || !out) return TMX_ERR_ARG;
+  if (!q || !kcache || !vcache || !place || !input_mask || !step || !out) return TMX_ERR_ARG;
   HeadAttnArgs a = {};
-  a.q = q; a.kcache = kcache; a.vcache = vcache; a.sink = sink; a.first = first; a.input_mask = input_mask; a.step = step;
+  a.q = q; a.kcache = kcache; a.vcache = vcache; a.sink = sink; a.place = (const int2*)place; a.input_mask = input_mask; a.step = step;
   a.buf_len = buf_len; a.out = out; a.partial = (float*)workspace; a.n_seq = n_seq; a.tpp = T; a.H = H; a.Kh = Kh;
   a.dk = dk; a.dv = dv; a.C = C; a.chunk = chunk; a.scale = scale;
-  return head_attention((hipStream_t)stream, act, a);
+  return head_attention((hipStream_t)stream, act, a, nullptr);
+}
+
+extern "C" int tmx_head_decode(void* stream, const void* z, int ldz, const float* q_norm_w, const float* k_norm_w, float eps,
+                               const float* table, int positions_max, const int32_t* place, void* kcache, void* vcache,
+                               const float* sink, const uint8_t* input_mask, const int32_t* step, int buf_len,
+                               void* out, void* workspace, int n_seq, int H, int Kh, int dim, int dk, int dv,
+                               int rot, int C, int chunk, float scale) {
+  HeadRowsArgs r = {};
+  if (!input_mask || !out || head_rows_args(r, z, ldz, q_norm_w, k_norm_w, eps, table, positions_max, place, step,
+                                                      buf_len, nullptr, kcache, vcache, 1, H, Kh, dim, dk, dv, rot, C))
+    return TMX_ERR_ARG;
+  HeadAttnArgs a = {};
+  a.kcache = kcache; a.vcache = vcache; a.sink = sink; a.place = (const int2*)place; a.input_mask = input_mask; a.step = step;
+  a.buf_len = buf_len; a.out = out; a.partial = (float*)workspace; a.n_seq = n_seq; a.tpp = 1; a.H = H; a.Kh = Kh;
+  a.dk = dk; a.dv = dv; a.C = C; a.chunk = chunk; a.scale = scale;
+  return head_attention((hipStream_t)stream, TMX_ACT_BF16, a, &r);
 }

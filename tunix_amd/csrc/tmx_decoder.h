@@ -33,7 +33,7 @@ struct Prof {
 struct DenseWorkspace {
   float* xs;            // residual streams [rows][S][Dp]
   void *xn, *z, *q, *lat, *val, *y, *act;
-  int32_t* first;       // first slot every row sees (TMX_MIXER_HEADS)
+  int2* place;          // per chunk size of the layers: tmx_row_places of every row (TMX_MIXER_HEADS)
   float* attn_partial;
   float* y_part;        // f32 planes of a projection whose K is split [nsplit][rows][Dp]
   float* logits;        // f32 models: products of the head [rows][Vp]

@@ -368,6 +368,14 @@ struct ResidualArgs {
   int buf_len, tpp;
 };
 
+struct RowPlacesArgs {  // see tmx_row_places
+  const int32_t* positions;
+  const uint8_t* input_mask;
+  const int32_t* step;
+  int buf_len, tpp, C, chunk;
+  int2* place;
+};
+
 struct HeadRowsArgs {  // see tmx_head_rows
   const void* z;
   int ldz;
@@ -375,19 +383,17 @@ struct HeadRowsArgs {  // see tmx_head_rows
   float eps;
   const float* table;
   int max_positions;
-  const int32_t* positions;
-  const uint8_t* input_mask;
+  const int2* place;
   const int32_t* step;
   int buf_len, tpp;
   void *q, *kcache, *vcache;
-  int32_t* first;
-  int H, Kh, dim, dk, dv, rot, C, chunk;
+  int H, Kh, dim, dk, dv, rot, C;
 };
 
 struct HeadAttnArgs {  // see tmx_head_attention
   const void *q, *kcache, *vcache;
   const float* sink;
-  const int32_t* first;
+  const int2* place;
   const uint8_t* input_mask;
   const int32_t* step;
   int buf_len;
@@ -400,7 +406,10 @@ struct HeadAttnArgs {  // see tmx_head_attention
 
 int residual_rows(hipStream_t st, int act, const ResidualArgs& a, int M);
 int head_rows(hipStream_t st, int act, const HeadRowsArgs& a, int M);
-int head_attention(hipStream_t st, int act, HeadAttnArgs a);
+int row_places(hipStream_t st, const RowPlacesArgs& a, int M);
+// rows: the row part in the same launch (a.q is not read), where head_rows_fused says so
+int head_attention(hipStream_t st, int act, HeadAttnArgs a, const HeadRowsArgs* rows);
+bool head_rows_fused(int act, int T, int H, int Kh);
 bool head_attn_ok(int dk, int dv);
 size_t head_attn_partial_bytes(int rows, int H, int dv);  // room for every split of `rows` query rows
 
