@@ -39,6 +39,16 @@ def test_a_layer_may_borrow_from_one_that_borrows():
   assert GroupedConfig.from_dict(raw).layers[5].weights_of == 0
 
 
+def test_a_layer_may_borrow_from_a_later_one():
+  layers = [GC.layer(*GC._A, weights_of=1), GC.layer(*GC._A), GC.layer(*GC._B)]
+  cfg = GC.config(layers)
+  st = GC.make_state(cfg)
+  assert not any(k.startswith('l0.') for k in st)
+  m = GC.product(cfg, st, device='cpu')
+  assert m.layers[0] is m.layers[1] and m.desc().num_layers == 3
+  assert np.isfinite(GC.plain(cfg, st, tokens(cfg, 5))).all()
+
+
 @pytest.mark.parametrize('edit, text', [
     (lambda c: c['layers'][0].update(type='other'), 'unknown mixer'),
     (lambda c: c['layers'][0]['mlp'].update(kind='sparse'), 'feed-forward kind'),

@@ -73,56 +73,55 @@ __device__ __forceinline__ void store_e(float* p, const float* v) {
   for (int i = 0; i < E; ++i) p[i] = v[i];
 }
 
-// What a lane needs of the rotation at one position: it owns the E columns c = E lane .. of a head of 64 E columns, whose
-// partners begin at column `mate` (E consecutive ones when half a rotation is a multiple of E).
+// What a lane needs of the rotation at one position: it owns the E columns c = E lane .. of a head of 64 E columns, with
+// partners p (a column past the rotated ones is its own).  The loads are free of branches, so that those of several heads
+// are in flight together.
 template <int E>
 struct HeadLane {
-  int c, half, rot, mate;
+  int c, p[E];
   float cs[E], sn[E];  // sn carries the sign of the column's half; 1, 0 past the rotated columns
-  __device__ __forceinline__ HeadLane(const HeadRowsArgs& a, int lane, int pos) : c(E * lane), half(a.rot >> 1), rot(a.rot) {
-    const float2* tab = reinterpret_cast<const float2*>(a.table) + (size_t)pos * half;
-    mate = c < half ? c + half : c - half;
+  __device__ __forceinline__ HeadLane(const HeadRowsArgs& a, int lane, int pos) : c(E * lane) {
+    const int rot = a.rot, half = rot >> 1;
+    // (without a rotation the loads below read some 8 valid bytes)
+    const float2* tab = rot > 0 ? reinterpret_cast<const float2*>(a.table) + (size_t)pos * half : reinterpret_cast<const float2*>(a.place);
+    float2 t[E];
 #pragma unroll
     for (int e = 0; e < E; ++e) {
       const int k = c + e;
-      cs[e] = 1.f;
-      sn[e] = 0.f;
-      if (k < rot) {
-        const float2 t = tab[k < half ? k : k - half];
-        cs[e] = t.x;
-        sn[e] = k < half ? -t.y : t.y;
-      }
+      t[e] = tab[k < half ? k : (k < rot ? k - half : 0)];
+      p[e] = k < half ? k + half : (k < rot ? k - half : k);
+    }
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+      const int k = c + e;
+      cs[e] = k < rot ? t[e].x : 1.f;
+      sn[e] = k < half ? -t[e].y : (k < rot ? t[e].y : 0.f);
     }
   }
-  // partners of the lane's columns in a head at src (its own columns in v where there are none)
+  // a head's values of this lane: its own columns and their partners, with the norm's weights
+  struct Head {
+    float v[E], u[E], wv[E], wu[E];
+  };
   template <typename T>
-  __device__ __forceinline__ void partners(const T* src, const float* v, float* u) const {
-    if (half % E == 0) {
-      if (c < rot) load_e<E>(src + mate, u);
-      else {
-#pragma unroll
-        for (int e = 0; e < E; ++e) u[e] = v[e];
-      }
-      return;
-    }
+  __device__ __forceinline__ void load(Head& d, const T* src, const float* nw) const {
+    load_e<E>(src + c, d.v);
+    const float* w = nw ? nw : reinterpret_cast<const float*>(src);  // (without a norm the values read are not used)
 #pragma unroll
     for (int e = 0; e < E; ++e) {
-      const int k = c + e;
-      u[e] = k < rot ? act_get(src + (k < half ? k + half : k - half)) : v[e];
+      d.u[e] = act_get(src + p[e]);
+      d.wv[e] = w[c + e];
+      d.wu[e] = w[p[e]];
     }
   }
-  // v <- the head's normed and rotated values
-  __device__ __forceinline__ void finish(float* v, const float* u, const float* nw, int dim, float eps) const {
+  // the head's normed and rotated values
+  __device__ __forceinline__ void finish(Head& d, bool norm, int dim, float eps) const {
     float ss = 0.f;
 #pragma unroll
-    for (int e = 0; e < E; ++e) ss += v[e] * v[e];
-    const float inv = nw ? 1.f / sqrtf(wave_sum(ss) / (float)dim + eps) : 1.f;
+    for (int e = 0; e < E; ++e) ss += d.v[e] * d.v[e];
+    const float inv = norm ? 1.f / sqrtf(wave_sum(ss) / (float)dim + eps) : 1.f;
 #pragma unroll
-    for (int e = 0; e < E; ++e) {
-      const int k = c + e, p = k < rot ? (k < half ? k + half : k - half) : k;
-      const float x = v[e] * inv * (nw ? nw[k] : 1.f), y = u[e] * inv * (nw ? nw[p] : 1.f);
-      v[e] = x * cs[e] + y * sn[e];
-    }
+    for (int e = 0; e < E; ++e)
+      d.v[e] = d.v[e] * inv * (norm ? d.wv[e] : 1.f) * cs[e] + d.u[e] * inv * (norm ? d.wu[e] : 1.f) * sn[e];
   }
 };
 
@@ -138,22 +137,21 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HeadRowsArgs a) {
   const T* z = reinterpret_cast<const T*>(a.z) + (size_t)m * a.ldz;
   if (hd0 < qk) {
     const HeadLane<E> hl(a, lane, min(a.place[m].y, a.max_positions - 1));
-    float v[4][E], u[4][E];
+    typename HeadLane<E>::Head d[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {  // (heads past the last key repeat it)
-      const T* src = z + (size_t)min(hd0 + i, qk - 1) * (64 * E);
-      load_e<E>(src + hl.c, v[i]);
-      hl.partners(src, v[i], u[i]);
+      const int hd = min(hd0 + i, qk - 1);
+      hl.load(d[i], z + (size_t)hd * (64 * E), hd >= a.H ? a.k_norm_w : a.q_norm_w);
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int hd = hd0 + i;
       if (hd >= qk) break;
       const bool key = hd >= a.H;
-      hl.finish(v[i], u[i], key ? a.k_norm_w : a.q_norm_w, a.dim, a.eps);
+      hl.finish(d[i], key ? a.k_norm_w : a.q_norm_w, a.dim, a.eps);
       T* dst = key ? reinterpret_cast<T*>(a.kcache) + (((size_t)seq * a.Kh + hd - a.H) * a.C + slot) * (64 * E)
                    : reinterpret_cast<T*>(a.q) + ((size_t)m * a.H + hd) * (64 * E);
-      store_e<E>(dst + hl.c, v[i]);
+      store_e<E>(dst + hl.c, d[i].v);
     }
   }
 #pragma unroll
@@ -230,17 +228,30 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
     const int g = (wg + WPW * i) * 64 + lane, row = g / CV, slot = g % CV;
     voff[i] = (row * CV + (slot ^ head_swz<CV>(row))) * 16;
   }
+  auto fetch_k = [&](int blk, int buf) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < kLk; ++i) load_row_to_lds(rk, tiles + buf * SH::kTile + (wg + WPW * i) * 512, koff[i], blk * (32 * DK * 2));
+  };
+  auto fetch_v = [&](int blk, int buf) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < kLv; ++i)
+      load_row_to_lds(rv, tiles + buf * SH::kTile + 32 * DK + (wg + WPW * i) * 512, voff[i], blk * (32 * DV * 2));
+  };
   auto fetch = [&](int blk, int buf) __attribute__((always_inline)) {
-    uint16_t* kt = tiles + buf * SH::kTile;
-#pragma unroll
-    for (int i = 0; i < kLk; ++i) load_row_to_lds(rk, kt + (wg + WPW * i) * 512, koff[i], blk * (32 * DK * 2));
-#pragma unroll
-    for (int i = 0; i < kLv; ++i) load_row_to_lds(rv, kt + 32 * DK + (wg + WPW * i) * 512, voff[i], blk * (32 * DV * 2));
+    fetch_k(blk, buf);
+    fetch_v(blk, buf);
+  };
+  // all but the youngest n loads have arrived
+  auto wait_loads = [&](auto nc) __attribute__((always_inline)) {
+    constexpr int n = decltype(nc)::value;
+    __builtin_amdgcn_sched_barrier(0);
+    __builtin_amdgcn_s_waitcnt(0x0F70 | (n & 15) | ((n >> 4) << 14));
+    __builtin_amdgcn_sched_barrier(0);
   };
   const uint8_t* mrow = a.input_mask + (size_t)seq * a.buf_len;
-  auto mask_byte = [&](int blk) __attribute__((always_inline)) {
-    const int p = blk * 32 + qi;
-    return (h == 0 && p < a.buf_len) ? mrow[p] : (uint8_t)0;
+  auto mask_byte = [&](int blk) __attribute__((always_inline)) { return mrow[min(blk * 32 + qi, a.buf_len - 1)]; };
+  auto mask_bits = [&](uint8_t mb, int blk) __attribute__((always_inline)) {
+    return (uint32_t)__ballot(mb != 0 && blk * 32 + qi < a.buf_len);  // (both halves of the wave say the same)
   };
 
   const int step0 = max(min(*a.step, min(a.C, a.buf_len) - a.tpp), 0);  // clamped: every slot read lies in the cache
@@ -250,47 +261,43 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
   const int b_end = (step0 + (min(q0 + 32 * SH::WQ, rows) - 1) / G + 32) >> 5;
   const int b_new = step0 >> 5;                               // ROWS: the block of the new row
   uint16_t* const stage = reinterpret_cast<uint16_t*>(ha_smem + SH::kStage);
+  int blk = b_beg + split * SH::WP + wp;                      // the block this wave begins with
+  uint8_t mb = 0;
   u32x4_t qf[KS];
   if constexpr (ROWS) {
-    constexpr int EM = KT > VT ? KT : VT;
     const HeadLane<KT> hl(ra, lane, min(place[0].y, ra.max_positions - 1));
     const uint16_t* z = reinterpret_cast<const uint16_t*>(ra.z) + (size_t)seq * ra.ldz;
     const bool owner = ((b_new - b_beg) / SH::WP) % a.nsplit == split;  // this workgroup walks the new row's block
-    // key (item 0), value (1), then the group's queries, dealt out to the waves, two at a time; the first tile is
-    // requested behind the first items
-    for (int i0 = wave; i0 < G + 2 || i0 < 4; i0 += 8) {
-      float v[2][EM], u[2][KT];
-#pragma unroll
-      for (int k = 0; k < 2; ++k) {
-        const int i = i0 + 4 * k;
-        if (i >= G + 2) break;
-        if (i == 1) {
-          load_e<VT>(z + (size_t)(a.H + a.Kh) * DK + (size_t)kvh * DV + VT * lane, v[k]);
-        } else {
-          const uint16_t* src = z + (size_t)(i == 0 ? a.H + kvh : kvh * G + i - 2) * DK;
-          load_e<KT>(src + hl.c, v[k]);
-          hl.partners(src, v[k], u[k]);
-        }
+    // key (item 0), value (1), then the group's queries, dealt out to the waves, two at a time
+    auto items = [&](int i0, auto behind_loads) __attribute__((always_inline)) {
+      typename HeadLane<KT>::Head d[2];
+      typedef uint16_t val_t __attribute__((ext_vector_type(VT)));
+      const bool two = i0 + 4 < G + 2, key = i0 == 0;
+      // (all of it is loaded by every wave; items past the last query repeat it)
+      const val_t val = *reinterpret_cast<const val_t*>(z + (size_t)(a.H + a.Kh) * DK + (size_t)kvh * DV + VT * lane);
+      hl.load(d[0], z + (size_t)(key ? a.H + kvh : kvh * G + max(min(i0 - 2, G - 1), 0)) * DK, key ? ra.k_norm_w : ra.q_norm_w);
+      hl.load(d[1], z + (size_t)(kvh * G + min(i0 + 2, G - 1)) * DK, ra.q_norm_w);
+      behind_loads();
+      if (i0 == 1) {
+        *reinterpret_cast<val_t*>(stage + 33 * DK + VT * lane) = val;
+        if (owner) *reinterpret_cast<val_t*>(reinterpret_cast<uint16_t*>(ra.vcache) + ((size_t)pair * a.C + step0) * DV + VT * lane) = val;
+      } else if (i0 < G + 2) {
+        hl.finish(d[0], key ? ra.k_norm_w : ra.q_norm_w, ra.dim, ra.eps);
+        store_e<KT>(stage + (key ? 32 : i0 - 2) * DK + hl.c, d[0].v);
+        if (key && owner) store_e<KT>(reinterpret_cast<uint16_t*>(ra.kcache) + ((size_t)pair * a.C + step0) * DK + hl.c, d[0].v);
       }
-      if (i0 == wave) {
-        const int blk = b_beg + split * SH::WP + wp;
-        if (blk < b_end) fetch(blk, 0);
+      if (two) {
+        hl.finish(d[1], ra.q_norm_w, ra.dim, ra.eps);
+        store_e<KT>(stage + (i0 + 2) * DK + hl.c, d[1].v);
       }
-#pragma unroll
-      for (int k = 0; k < 2; ++k) {
-        const int i = i0 + 4 * k;
-        if (i >= G + 2) break;
-        if (i == 1) {
-          store_e<VT>(stage + 33 * DK + VT * lane, v[k]);
-          if (owner) store_e<VT>(reinterpret_cast<uint16_t*>(ra.vcache) + ((size_t)pair * a.C + step0) * DV + VT * lane, v[k]);
-          continue;
-        }
-        hl.finish(v[k], u[k], i == 0 ? ra.k_norm_w : ra.q_norm_w, ra.dim, ra.eps);
-        store_e<KT>(stage + (i == 0 ? 32 : i - 2) * DK + hl.c, v[k]);
-        if (i == 0 && owner) store_e<KT>(reinterpret_cast<uint16_t*>(ra.kcache) + ((size_t)pair * a.C + step0) * DK + hl.c, v[k]);
-      }
-    }
-    __syncthreads();
+    };
+    mb = mask_byte(blk);
+    items(wave, [&]() __attribute__((always_inline)) {
+      if (blk < b_end) fetch(blk, 0);
+    });
+    for (int i0 = wave + 8; i0 < G + 2; i0 += 8) items(i0, [] {});
+    // (the tile under way and the stores of the new row need not be waited for)
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
 #pragma unroll
     for (int t = 0; t < KS; ++t) qf[t] = *reinterpret_cast<const u32x4_t*>(stage + qr_l * DK + (DK / 2) * h + 8 * t);
   } else {
@@ -375,15 +382,21 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
   auto lds_addr = [](const uint16_t* p) __attribute__((always_inline)) {
     return (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const uint16_t*)p;
   };
-  auto block = [&](int blk, uint32_t mbits, int buf) __attribute__((always_inline)) {
+  // behind_scores runs when the block's K rows have been read, v_ready in front of the first read of its V rows
+  constexpr bool kLateV = !SHARED && SH::kBufs == 1;
+  auto block = [&](int blk, uint32_t mbits, int buf, auto behind_scores, auto v_ready) __attribute__((always_inline)) {
     const uint16_t* kt = tiles + buf * SH::kTile;
     const uint32_t vb = lds_addr(kt) + vbase;
     f32x16_t sacc;
     float mn;
     u32x4_t p[4];  // probabilities as bf16 hi (p[0], p[1]) and lo (p[2], p[3]), 16 positions each
+    auto request_v = [&]() __attribute__((always_inline)) {
+      static_for<R>([&](auto fc) __attribute__((always_inline)) { load_v(vb, fc); });
+      __builtin_amdgcn_sched_barrier(0);
+    };
     scores(kt, blk, mbits, sacc, mn);
-    static_for<R>([&](auto fc) __attribute__((always_inline)) { load_v(vb, fc); });  // they do not wait for the softmax
-    __builtin_amdgcn_sched_barrier(0);
+    behind_scores();
+    if (!kLateV) request_v();  // they do not wait for the softmax
     move_reference(mn);
 #pragma unroll
     for (int r = 0; r < 16; r += 2) {
@@ -392,6 +405,10 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
       p[r >> 3][(r >> 1) & 3] = hi;
       p[2 + (r >> 3)][(r >> 1) & 3] = pack_bf2(p0 - bf_lo(hi), p1 - bf_hi(hi));
       l += p0 + p1;
+    }
+    if (kLateV) {
+      v_ready();
+      request_v();
     }
     // out^T += V^T . P^T, 16 positions (accumulator registers 8 kb2 .. 8 kb2 + 7) per MFMA
     static_for<2 * VC>([&](auto fc) __attribute__((always_inline)) {
@@ -410,30 +427,34 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
   };
 
   if constexpr (SHARED) {
-    const int blk0 = b_beg + split;
-    const int rounds = b_end > blk0 ? (b_end - blk0 + a.nsplit - 1) / a.nsplit : 0;  // the same in every wave
-    uint8_t mb = mask_byte(blk0);
-    if (rounds > 0) fetch(blk0, 0);
-    for (int round = 0; round < rounds; ++round) {
-      const int blk = blk0 + round * a.nsplit, buf = round & 1;
-      const uint32_t mbits = (uint32_t)__ballot(mb != 0);
+    const int rounds = b_end > blk ? (b_end - blk + a.nsplit - 1) / a.nsplit : 0;  // the same in every wave
+    mb = mask_byte(blk);
+    if (rounds > 0) fetch(blk, 0);
+    for (int round = 0; round < rounds; ++round, blk += a.nsplit) {
+      const int buf = round & 1;
+      const uint32_t mbits = mask_bits(mb, blk);
       __builtin_amdgcn_s_waitcnt(0x0F70);  // this round's tile has landed
       __syncthreads();                     // ... in every wave, and the other buffer's readers are done
       mb = mask_byte(blk + a.nsplit);
       if (round + 1 < rounds) fetch(blk + a.nsplit, buf ^ 1);
-      block(blk, mbits, buf);
+      block(blk, mbits, buf, [] {}, [] {});
     }
   } else {
     const int stride = a.nsplit * SH::WP;
-    int blk = b_beg + split * SH::WP + wp, buf = 0;
-    uint8_t mb = mask_byte(blk);
-    if (!ROWS && blk < b_end) fetch(blk, 0);
+    int buf = 0;
+    if constexpr (!ROWS) {
+      mb = mask_byte(blk);
+      if (blk < b_end) fetch(blk, 0);
+    }
+    uint32_t mbits = mask_bits(mb, blk);
     for (; blk < b_end; blk += stride) {
-      const uint32_t mbits = (uint32_t)__ballot(mb != 0);
-      __builtin_amdgcn_s_waitcnt(0x0F70);  // the wave's own tile has landed
-      __builtin_amdgcn_sched_barrier(0);
-      mb = mask_byte(blk + stride);
-      if (ROWS && blk == b_new) {
+      const bool more = blk + stride < b_end;
+      const bool made = ROWS && blk == b_new;  // the block of the row that waits in LDS
+      if (SH::kBufs == 2) mbits = mask_bits(mb, blk);
+      // two buffers: the tile has landed; one: its K rows have, the V rows behind them follow
+      if (SH::kBufs == 2 || made) wait_loads(IC<0>{});
+      else wait_loads(IC<kLv>{});
+      if (made) {
         uint16_t* kt = tiles + buf * SH::kTile;
         const int r = step0 & 31;
         if (lane < CK)
@@ -443,13 +464,29 @@ __global__ __launch_bounds__(256, (KT + VT > 4 ? 1 : 2)) void head_attn_kernel(H
               *reinterpret_cast<const u32x4_t*>(stage + 33 * DK + lane * 8);
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
       }
-      const bool more = blk + stride < b_end;
-      if (SH::kBufs == 2 && more) fetch(blk + stride, buf ^ 1);
-      block(blk, mbits, buf);
-      if (SH::kBufs == 2) buf ^= 1;
-      else if (more) {
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // the tile's reads are complete
-        fetch(blk + stride, 0);
+      if (SH::kBufs == 2) {
+        mb = mask_byte(blk + stride);
+        if (more) fetch(blk + stride, buf ^ 1);
+        block(blk, mbits, buf, [] {}, [] {});
+        buf ^= 1;
+      } else {
+        // the next K rows travel beside the softmax and the product, the next V rows beside the next scores
+        block(blk, mbits, 0,
+              [&]() __attribute__((always_inline)) {
+                asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+                mb = mask_byte(blk + stride);
+                if (more) fetch_k(blk + stride, 0);
+              },
+              [&]() __attribute__((always_inline)) {
+                if (more) {
+                  wait_loads(IC<kLk>{});
+                  mbits = mask_bits(mb, blk + stride);  // (older than the next K rows)
+                } else {
+                  wait_loads(IC<0>{});
+                }
+              });
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        if (more) fetch_v(blk + stride, 0);
       }
     }
   }

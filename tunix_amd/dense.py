@@ -221,10 +221,10 @@ class DenseModel:
   def _build(self, tensor):
     """Everything from tensor(name)."""
     self._outer(tensor('embed'), tensor('final.norm'), tensor('head'))
-    for i, l in enumerate(self.config.layers):
-      src = getattr(l, 'weights_of', None)
-      # a layer without tensors of its own shares the operands of an earlier one
-      self.layers.append(self.layers[src] if src is not None else self._layer(l, lambda n, i=i: tensor(f'l{i}.{n}')))
+    layers = self.config.layers
+    owner = [i if getattr(l, 'weights_of', None) is None else l.weights_of for i, l in enumerate(layers)]
+    own = {i: self._layer(l, lambda n, i=i: tensor(f'l{i}.{n}')) for i, l in enumerate(layers) if owner[i] == i}
+    self.layers = [own[i] for i in owner]  # a layer without tensors of its own shares the operands of another one
 
   @classmethod
   def from_state(cls, config, state, device='cuda'):
