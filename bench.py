@@ -144,7 +144,8 @@ def class_work(model, rows, keys, decode):
     qk, v = (l.heads + l.kv_heads) * l.dim, l.kv_heads * l.vdim
     out['row_norm'] = (rows * c.embed_dim * (2 * 4 + 4), rows * c.embed_dim * 6)
     out['qkv_linear'] = dense(c.embed_dim, qk + v)
-    out['rope_kvwrite'] = (rows * 4.0 * (qk + v), 0)
+    if not decode:  # one token per sequence: inside the attention launch
+      out['rope_kvwrite'] = (rows * 4.0 * (qk + v), 0)
     kv = 2.0 * l.kv_heads * (l.dim + l.vdim)
     out['attention'] = ((rows * keys if decode else keys) * kv + rows * 2.0 * l.heads * (l.dim + l.vdim),
                         2.0 * rows * keys * l.heads * (l.dim + l.vdim))
